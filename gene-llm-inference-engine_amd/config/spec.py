@@ -81,6 +81,13 @@ class RmsNormSpec:
 
 
 @dataclass(frozen=True)
+class NoNormSpec:
+    """No norm: the rows as they are, for an arrangement that has a place for a norm where an architecture has none."""
+    kind: ClassVar[str] = "none"
+    size: int
+
+
+@dataclass(frozen=True)
 class AttentionSpec:
     """Causal attention with grouped key/value heads over a paged cache."""
     kind: ClassVar[str] = "attention"
@@ -119,6 +126,12 @@ class AttentionSpec:
     # head by head.
     qk_norm_whole: bool = False
     score_cap: Optional[float] = None    # a scaled score s becomes cap * tanh(s / cap) before the softmax
+    # The values are the projected keys, as they are before the keys' norm (v_proj is then not read and may be empty; value_dim is head_dim).
+    values_are_keys: bool = False
+    # (coef, every): the query at position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1), behind norm and rotation.
+    query_growth: Optional[Tuple[float, float]] = None
+    sink_score: Optional[float] = None   # one fixed score for all heads that joins the softmax's denominator and has no value (`sinks` must then be absent)
+    output_gate: Optional[str] = None    # tensor [heads*value_dim, hidden]: the heads' outputs times sigmoid(it . the mixer's input), channel by channel
 
 
 @dataclass(frozen=True)
@@ -248,6 +261,32 @@ class SelectiveScanSpec:
 
 
 @dataclass(frozen=True)
+class LightningSpec:
+    """Linear attention whose memory fades by a constant per head.  q, k [heads, key_dim] and v [heads, value_dim] pass SiLU; per head,
+    with S [key_dim, value_dim] zero at a sequence's start and d the head's entry of `decay`:
+        S <- d S + k v^T        o = S^T q
+    The heads' outputs side by side are divided by their common root mean square (`norm_eps` inside the root), multiplied by `out_norm`
+    [heads*value_dim] and by sigmoid(gate(x)), and go through `o_proj`.  A request's state is S of every head, in 32-bit."""
+    kind: ClassVar[str] = "lightning"
+    hidden_size: int
+    n_heads: int
+    key_dim: int
+    value_dim: int
+    decay: Tuple[float, ...]
+    norm_eps: float
+    q_proj: str
+    k_proj: str
+    v_proj: str
+    gate_proj: str
+    out_norm: str
+    o_proj: str
+
+    def __post_init__(self):
+        if len(self.decay) != self.n_heads:
+            raise ValueError(f"lightning attention: {self.n_heads} heads need as many decays, not {len(self.decay)}")
+
+
+@dataclass(frozen=True)
 class SideBySideSpec:
     """Several mixers that read the same rows; the layer's mixer output is sum_i weights[i] * members[i](h).  Each member keeps the
     cache or state it would keep alone."""
@@ -366,6 +405,16 @@ class ScaleSpec:
     """Rows multiplied by a constant (for instance a token table that is stored unscaled)."""
     kind: ClassVar[str] = "scale"
     factor: float
+
+
+@dataclass(frozen=True)
+class LearnedPositionsSpec:
+    """Row p of a learned table [positions, hidden] added to the row of the token at position p (behind the token table).  A sequence
+    cannot be longer than the table."""
+    kind: ClassVar[str] = "learned_positions"
+    hidden_size: int
+    positions: int
+    table: str
 
 
 @dataclass(frozen=True)

@@ -30,13 +30,16 @@ __device__ __forceinline__ float exp2_fast(float x) { return __builtin_amdgcn_ex
 //   chunk   a row at position p sees no key before p - p % chunk (a mask cut into chunks counted from the sequence's start);
 //   sinks   [n_heads]: exp(sinks[h]) joins the softmax's denominator of head h (a score without a key or a value), once a row:
 //           where a row's keys are shared out over splits or waves, the first of them counts it;
-//   gate    [rows, gate_stride]: head h's output of row t is multiplied by sigmoid(gate[t * gate_stride + h]).
+//   gate    [rows, gate_stride]: head h's output of row t is multiplied by sigmoid(gate[t * gate_stride + h]), or, with
+//           gate_channels = the head's channels, channel d of it by sigmoid(gate[t * gate_stride + h * gate_channels + d]) (rows that
+//           start at multiples of 16 bytes).
 //   cap     > 0: a scaled score s becomes cap * tanh(s / cap) before the softmax.
 struct Extras {
     int chunk;
     const float* sinks;
     const float* gate;
     long gate_stride;
+    int gate_channels;
     float cap;
 };
 // Capped scores, in units of log2 e: with a cap the kernels take scale2 = 1 and turn every product s into
@@ -60,8 +63,21 @@ __device__ __forceinline__ void add_sink(float sink, float& m, float& l) {
     if (m == -INFINITY) { m = s2; l = 1.f; }
     else l += exp2_fast(s2 - m);
 }
+__device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float gate_of(const Extras& x, size_t row, int head) {
-    return x.gate ? 1.0f / (1.0f + expf(-x.gate[row * x.gate_stride + head])) : 1.0f;
+    return x.gate && !x.gate_channels ? sigmoid_f(x.gate[row * x.gate_stride + head]) : 1.0f;
+}
+// The factor of one channel where there is a gate per channel, 1 otherwise.
+__device__ __forceinline__ float channel_gate_of(const Extras& x, size_t row, int head, int d) {
+    return x.gate && x.gate_channels ? sigmoid_f(x.gate[row * x.gate_stride + (size_t)head * x.gate_channels + d]) : 1.0f;
+}
+// Four neighbouring channels of a head, times what they are to be multiplied by, as two packed pairs.
+__device__ __forceinline__ uint2 gated4(const Extras& x, size_t row, int head, int d, float a, float b, float c, float e) {
+    if (x.gate && x.gate_channels) {
+        const float4 z = *reinterpret_cast<const float4*>(x.gate + row * x.gate_stride + (size_t)head * x.gate_channels + d);
+        a *= sigmoid_f(z.x), b *= sigmoid_f(z.y), c *= sigmoid_f(z.z), e *= sigmoid_f(z.w);
+    }
+    return uint2{pack2(a, b), pack2(c, e)};
 }
 
 // =========================================================================================== prompt
@@ -372,8 +388,8 @@ __global__ __launch_bounds__(128 * NW * PAIR) void attention_prompt_kernel(const
 #pragma unroll
         for (int v4 = 0; v4 < 4; ++v4) {                                  // element v: channel 32*i + 8*(v/4) + 4*hf + v%4
             const int d = 32 * i + 8 * v4 + 4 * hf;
-            *reinterpret_cast<uint2*>(orow + d) = uint2{pack2(o[i][4 * v4] * inv, o[i][4 * v4 + 1] * inv),
-                                                        pack2(o[i][4 * v4 + 2] * inv, o[i][4 * v4 + 3] * inv)};
+            *reinterpret_cast<uint2*>(orow + d) = gated4(extra, (size_t)(row0 + my_row), head, d, o[i][4 * v4] * inv, o[i][4 * v4 + 1] * inv, o[i][4 * v4 + 2] * inv,
+                                                         o[i][4 * v4 + 3] * inv);
         }
 }
 
@@ -621,8 +637,8 @@ __global__ __launch_bounds__(64 * NW, HD == 128 ? 2 : 3) void attention_prompt_w
 #pragma unroll
         for (int v4 = 0; v4 < 4; ++v4) {                      // element v: channel 32*i + 8*(v/4) + 4*hf + v%4
             const int d = 32 * i + 8 * v4 + 4 * hf;
-            *reinterpret_cast<uint2*>(orow + d) = uint2{pack2(o[i][4 * v4] * inv, o[i][4 * v4 + 1] * inv),
-                                                        pack2(o[i][4 * v4 + 2] * inv, o[i][4 * v4 + 3] * inv)};
+            *reinterpret_cast<uint2*>(orow + d) = gated4(extra, (size_t)(row0 + my_row), head, d, o[i][4 * v4] * inv, o[i][4 * v4 + 1] * inv, o[i][4 * v4 + 2] * inv,
+                                                         o[i][4 * v4 + 3] * inv);
         }
 }
 
@@ -961,7 +977,7 @@ __global__ __launch_bounds__(64 * DecodeShape<HD>::MAX_WAVES) void attention_dec
         }
         if (extra.sinks != nullptr && split == 0) add_sink(extra.sinks[out_head], big, denom);
         if (n_splits == 1) {
-            out[((size_t)row * n_heads + out_head) * HD + d] = f32_to_bf16(acc / denom * gate_of(extra, (size_t)row, out_head));
+            out[((size_t)row * n_heads + out_head) * HD + d] = f32_to_bf16(acc / denom * gate_of(extra, (size_t)row, out_head) * channel_gate_of(extra, (size_t)row, out_head, d));
         } else {                                             // part[row_index][head][split] = {m, l, O[HD]}
             float* dst = part + (((size_t)blockIdx.x * n_heads + out_head) * n_splits + split) * (HD + 2);
             if (d == 0) {
@@ -1017,7 +1033,8 @@ __global__ __launch_bounds__(64) void attention_decode_combine_kernel(const floa
     __syncthreads();
     float denom = 0.f;
     for (int s = 0; s < n_splits; ++s) denom += weighted_l[s];
-    const float inv = gate_of(extra, (size_t)(rows ? rows[idx] : idx), head) / denom;
+    const size_t row = rows ? rows[idx] : idx;
+    const float inv = gate_of(extra, row, head) / denom;
     const int n_early = min(n_splits, EARLY);
     for (int d = lane, c = 0; d < hd; d += 64, ++c) {
         float acc = 0.f;
@@ -1028,7 +1045,7 @@ __global__ __launch_bounds__(64) void attention_decode_combine_kernel(const floa
         }
 #pragma unroll 8
         for (int s = c < 2 ? n_early : 0; s < n_splits; ++s) acc = fmaf(weight[s], src[(size_t)s * (hd + 2) + 2 + d], acc);
-        out[((size_t)(rows ? rows[idx] : idx) * n_heads + head) * hd + d] = f32_to_bf16(acc * inv);
+        out[(row * n_heads + head) * hd + d] = f32_to_bf16(acc * inv * channel_gate_of(extra, row, head, d));
     }
 }
 
@@ -1048,9 +1065,12 @@ GI_API int gi_attention_bf16_supports(int hd, int page_size, int prompt) {
 GI_API int gi_attention_prompt_bf16(const void* q, const void* cache, void* out, const int* tiles, int n_tiles, int rows_per_tile, int paired,
                                     const int* table, int table_stride, long page_stride, int page_size, int n_heads, int n_kv, int hd,
                                     int window, float scale, int n_splits, const int* tile_first, const int* rows, int n_rows, float* part,
-                                    long part_floats, int chunk, const float* sinks, const float* gate, long gate_stride, float cap, hipStream_t stream) {
-    GI_REQUIRE(chunk >= 0 && cap >= 0.f && (gate == nullptr || gate_stride >= n_heads), "attention_prompt: bad chunk, cap or gate stride");
-    const Extras extra = {chunk, sinks, gate, gate_stride, cap};
+                                    long part_floats, int chunk, const float* sinks, const float* gate, long gate_stride, int gate_channels, float cap,
+                                    hipStream_t stream) {
+    GI_REQUIRE(chunk >= 0 && cap >= 0.f && (gate_channels == 0 || gate_channels == hd) && (gate == nullptr || gate_stride >= (long)n_heads * (gate_channels ? hd : 1)) &&
+                   (gate == nullptr || gate_channels == 0 || (gate_stride % 4 == 0 && ((uintptr_t)gate & 15) == 0)),
+               "attention_prompt: bad chunk, cap or gate stride, or a channels' gate whose rows do not start at multiples of 16 bytes");
+    const Extras extra = {chunk, sinks, gate, gate_stride, gate_channels, cap};
     GI_REQUIRE(rows_per_tile == 64 || rows_per_tile == 128, "attention_prompt: tiles of %d rows are not supported (64 or 128)", rows_per_tile);
     GI_REQUIRE(n_tiles > 0 && n_heads > 0 && n_kv > 0 && n_heads % n_kv == 0, "attention_prompt: bad counts (%d tiles, %d heads, %d kv heads)",
                n_tiles, n_heads, n_kv);
@@ -1166,9 +1186,12 @@ GI_API int gi_attention_decode_bf16(const void* q, const float* qf, const float*
                                     const float* cos_t, const float* sin_t, void* cache, void* out, float* part, long part_floats,
                                     const int* rows, int n_rows, const int* pos, const int* slots, const int* table, int table_stride,
                                     long page_stride, int page_size, int n_heads, int n_kv, int hd, int window, float scale, int n_splits,
-                                    int n_waves, int chunk, const float* sinks, const float* gate, long gate_stride, float cap, hipStream_t stream) {
-    GI_REQUIRE(chunk >= 0 && cap >= 0.f && (gate == nullptr || gate_stride >= n_heads), "attention_decode: bad chunk, cap or gate stride");
-    const Extras extra = {chunk, sinks, gate, gate_stride, cap};
+                                    int n_waves, int chunk, const float* sinks, const float* gate, long gate_stride, int gate_channels, float cap,
+                                    hipStream_t stream) {
+    GI_REQUIRE(chunk >= 0 && cap >= 0.f && (gate_channels == 0 || gate_channels == hd) && (gate == nullptr || gate_stride >= (long)n_heads * (gate_channels ? hd : 1)) &&
+                   (gate == nullptr || gate_channels == 0 || (gate_stride % 4 == 0 && ((uintptr_t)gate & 15) == 0)),
+               "attention_decode: bad chunk, cap or gate stride, or a channels' gate whose rows do not start at multiples of 16 bytes");
+    const Extras extra = {chunk, sinks, gate, gate_stride, gate_channels, cap};
     GI_REQUIRE(n_rows > 0 && n_heads > 0 && n_kv > 0 && n_heads % n_kv == 0, "attention_decode: bad counts (%d rows, %d heads, %d kv heads)",
                n_rows, n_heads, n_kv);
     GI_REQUIRE(gi_attention_bf16_supports(hd, page_size, 0), "attention_decode: head size %d with page size %d is not supported", hd, page_size);

@@ -419,7 +419,9 @@ GI_API int gi_rmsnorm_add(const float* y, const void* w, int w_dtype, float* x, 
 // `flags`: NRS_NORM_ALL takes the norm over all heads of the projection at once, with weights [heads * hd] ([kv heads * hd]); NRS_NEIGHBOURS turns the pairs (2i, 2i + 1), i < rot/2, instead (angle i for pair i); NRS_UNIT_RMS divides every query and
 // key head by its root mean square without weights (q_norm and k_norm must then be absent); NRS_NORM_LAST takes the norm, of
 // either form, behind the rotation instead of in front of it.  `v_scale` multiplies the values on their way into the pages (the
-// attention's result is linear in them: a layer that weighs its attention's result can weigh the values instead).
+// attention's result is linear in them: a layer that weighs its attention's result can weigh the values instead).  With q_every > 0 the
+// finished query of the row at position p is multiplied by 1 + q_coef ln(floor((p + 1) / q_every) + 1).  k and v may be the same columns
+// (the values are then the keys as projected: nothing here changes its inputs).
 constexpr int NRS_MAX_HD = 512;
 constexpr int NRS_NEIGHBOURS = 1, NRS_UNIT_RMS = 2, NRS_NORM_LAST = 4, NRS_NORM_ALL = 8;
 
@@ -457,7 +459,7 @@ __global__ __launch_bounds__(64) void norm_rope_store_kernel(const float* __rest
                                                             const float* __restrict__ q_bias, const float* __restrict__ k_bias,
                                                             const float* __restrict__ v_bias, const float* __restrict__ v_other, long ld_other,
                                                             const float* __restrict__ v_blend, float* __restrict__ v_keep, long ld_keep, int flags,
-                                                            float v_scale, const float* __restrict__ rows_r) {
+                                                            float v_scale, const float* __restrict__ rows_r, float q_coef, double q_every) {
     __shared__ float s[NRS_MAX_HD];
     const int t = blockIdx.x, item = blockIdx.y, lane = threadIdx.x;
     const int p = pos[t];
@@ -498,6 +500,7 @@ __global__ __launch_bounds__(64) void norm_rope_store_kernel(const float* __rest
     const bool turn = cos_t != nullptr && rot > 0, neighbours = flags & NRS_NEIGHBOURS;
     TC* kdst = nullptr;
     TQ* qdst = nullptr;
+    const float grown = is_q && q_every > 0.0 ? fmaf(q_coef, logf((float)(floor((double)(p + 1) / q_every) + 1.0)), 1.0f) : 1.0f;
     if (is_q) qdst = q_out + ((size_t)t * n_heads + h) * hd;
     else {
         const long page = table[(size_t)slot[t] * table_stride + p / page_size];
@@ -516,7 +519,7 @@ __global__ __launch_bounds__(64) void norm_rope_store_kernel(const float* __rest
             }
         }
         if (norm_last) out = w != nullptr ? load_f32(w, d) * (r * out) : r * out;
-        if (is_q) store_f32(qdst, d, out); else store_f32(kdst, d, out);
+        if (is_q) store_f32(qdst, d, out * grown); else store_f32(kdst, d, out);
     }
 }
 
@@ -525,7 +528,8 @@ GI_API int gi_norm_rope_store(const float* q, const float* k, const float* v, lo
                               const int* table, int table_stride, void* q_out, int q_dtype, void* cache, int cache_dtype, long page_stride,
                               int page_size, int n_rows, int n_heads, int n_kv, int hd, int vd, const float* q_bias, const float* k_bias,
                               const float* v_bias, const float* v_other, long ld_other, const float* v_blend, float* v_keep, long ld_keep,
-                              int flags, float v_scale, float* rows_r, hipStream_t stream) {
+                              int flags, float v_scale, float* rows_r, float q_coef, double q_every, hipStream_t stream) {
+    GI_REQUIRE(q_every >= 0.0, "norm_rope_store: queries grow every so many positions, a positive number (0: not)");
     if (flags & NRS_NORM_ALL) {
         GI_REQUIRE(rows_r != nullptr && !(flags & NRS_UNIT_RMS) && q_norm != nullptr && (k == nullptr || k_norm != nullptr),
                    "norm_rope_store: a norm over whole projections needs its weights and room for two numbers a row");
@@ -547,7 +551,7 @@ GI_API int gi_norm_rope_store(const float* q, const float* k, const float* v, lo
 #define LAUNCH(TQ, TC, TW)                                                                                                                    \
     norm_rope_store_kernel<TQ, TC, TW><<<grid, 64, 0, stream>>>(q, k, v, ldq, ldk, ldv, (const TW*)q_norm, (const TW*)k_norm, eps, cos_t, sin_t, rot, pos, \
                                                                 slot, table, table_stride, (TQ*)q_out, (TC*)cache, page_stride, page_size, n_heads, n_kv, hd, vd, \
-                                                                q_bias, k_bias, v_bias, v_other, ld_other, v_blend, v_keep, ld_keep, flags, v_scale, rows_r)
+                                                                q_bias, k_bias, v_bias, v_other, ld_other, v_blend, v_keep, ld_keep, flags, v_scale, rows_r, q_coef, q_every)
     if (q_dtype == GI_F32 && cache_dtype == GI_F32 && norm_dtype == GI_F32) LAUNCH(float, float, float);
     else if (q_dtype == GI_BF16 && cache_dtype == GI_BF16 && norm_dtype == GI_BF16) LAUNCH(bf16_t, bf16_t, bf16_t);
     else if (q_dtype == GI_BF16 && cache_dtype == GI_BF16 && norm_dtype == GI_F32) LAUNCH(bf16_t, bf16_t, float);
@@ -791,5 +795,109 @@ GI_API int gi_gate_token_columns(const float* u, long ldu, const void* table, in
     else return gi_fail("gate_token_columns: unknown dtypes %d, %d", table_dtype, out_dtype);
 #undef LAUNCH
     GI_CHECK_LAUNCH("gate_token_columns");
+    return 0;
+}
+
+// ------------------------------------------------------- token rows times a scale plus a learned row per position
+// x[t] = table[tokens[t]] * scale + where[pos[t]], and, if `low` is given, x[t] once more in bfloat16 (as a product without a norm in front
+// of it reads the rows).  A workgroup takes 1,024 columns of a row.
+template <typename TT, typename TP>
+__global__ __launch_bounds__(256) void embed_positioned_kernel(const TT* __restrict__ table, const int* __restrict__ tokens, float scale, const TP* __restrict__ where,
+                                                              int n_positions, const int* __restrict__ pos, float* __restrict__ x, bf16_t* __restrict__ low, int dim) {
+    const size_t t = blockIdx.x;
+    const TT* row = table ? table + (size_t)tokens[t] * dim : nullptr;      // (no table: x holds the rows already)
+    const TP* at = where + (size_t)min(max(pos[t], 0), n_positions - 1) * dim;
+    for (int d = blockIdx.y * 1024 + threadIdx.x; d < min(dim, ((int)blockIdx.y + 1) * 1024); d += 256) {
+        const float v = (row ? load_f32(row, d) * scale : x[t * dim + d]) + load_f32(at, d);
+        x[t * dim + d] = v;
+        if (low) low[t * dim + d] = f32_to_bf16(v);
+    }
+}
+
+GI_API int gi_embed_positioned(const void* table, int table_dtype, const int* tokens, float scale, const void* where, int where_dtype, int n_positions, const int* pos,
+                               float* x, void* low, int n_rows, int dim, hipStream_t stream) {
+    GI_REQUIRE(n_rows > 0 && dim > 0 && n_positions > 0 && where != nullptr && pos != nullptr && (table == nullptr || tokens != nullptr),
+               "embed_positioned: bad sizes (rows %d, columns %d, positions %d)", n_rows, dim, n_positions);
+    GI_REQUIRE((dim + 1023) / 1024 <= 65535, "embed_positioned: rows too long");
+    dim3 grid(n_rows, (dim + 1023) / 1024);
+#define LAUNCH(TT, TP) embed_positioned_kernel<TT, TP><<<grid, 256, 0, stream>>>((const TT*)table, tokens, scale, (const TP*)where, n_positions, pos, x, (bf16_t*)low, dim)
+    if (table_dtype == GI_F32 && where_dtype == GI_F32) LAUNCH(float, float);
+    else if (table_dtype == GI_F32 && where_dtype == GI_BF16) LAUNCH(float, bf16_t);
+    else if (table_dtype == GI_BF16 && where_dtype == GI_F32) LAUNCH(bf16_t, float);
+    else if (table_dtype == GI_BF16 && where_dtype == GI_BF16) LAUNCH(bf16_t, bf16_t);
+    else return gi_fail("embed_positioned: unknown dtypes %d, %d", table_dtype, where_dtype);
+#undef LAUNCH
+    GI_CHECK_LAUNCH("embed_positioned");
+    return 0;
+}
+
+// ------------------------------------------------- a norm on a sublayer's output, added on, and the sum as a product reads it
+// x[t] += w * norm(y[t]), and low[t] = bfloat16(x[t]): what a layer does whose norms follow its sublayers and whose next sublayer reads x
+// itself.  NV > 0: rows whose length is a multiple of 4 and at most 1024 NV, aligned: a thread asks for all its numbers at once and
+// keeps them.
+template <int NV, typename TW>
+__global__ __launch_bounds__(256) void rmsnorm_add_store_kernel(const float* __restrict__ y, const TW* __restrict__ w, float* __restrict__ x, bf16_t* __restrict__ low,
+                                                               int dim, float eps, size_t y_stride, size_t x_stride, size_t low_stride) {
+    __shared__ float red[4];
+    const float* yr = y + (size_t)blockIdx.x * y_stride;
+    float* xr = x + (size_t)blockIdx.x * x_stride;
+    bf16_t* lr = low + (size_t)blockIdx.x * low_stride;
+    if constexpr (NV > 0) {
+        float4 yv[NV], xv[NV], wv[NV];
+        float ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int d = min(4 * ((int)threadIdx.x + 256 * i), dim - 4);
+            yv[i] = load4(yr + d), xv[i] = load4(xr + d), wv[i] = load4(w + d);
+        }
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const float s = (yv[i].x * yv[i].x + yv[i].y * yv[i].y) + (yv[i].z * yv[i].z + yv[i].w * yv[i].w);
+            ss += 4 * ((int)threadIdx.x + 256 * i) < dim ? s : 0.f;
+        }
+        const float r = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)dim + eps);
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int d = 4 * ((int)threadIdx.x + 256 * i);
+            if (d < dim) {
+                const float a = xv[i].x + wv[i].x * (r * yv[i].x), b = xv[i].y + wv[i].y * (r * yv[i].y);
+                const float c = xv[i].z + wv[i].z * (r * yv[i].z), e = xv[i].w + wv[i].w * (r * yv[i].w);
+                store4(xr + d, a, b, c, e);
+                store4(lr + d, a, b, c, e);
+            }
+        }
+    } else {
+        float ss = 0.f;
+        for (int d = threadIdx.x; d < dim; d += 256) ss = fmaf(yr[d], yr[d], ss);
+        const float r = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)dim + eps);
+        for (int d = threadIdx.x; d < dim; d += 256) {
+            const float v = xr[d] + load_f32(w, d) * (r * yr[d]);
+            xr[d] = v;
+            lr[d] = f32_to_bf16(v);
+        }
+    }
+}
+
+GI_API int gi_rmsnorm_add_store(const float* y, const void* w, int w_dtype, float* x, void* low, int n_rows, int dim, float eps, long y_stride, long x_stride, long low_stride,
+                                hipStream_t stream) {
+    GI_REQUIRE(n_rows > 0 && dim > 0 && y_stride >= dim && x_stride >= dim && low_stride >= dim && low != nullptr, "rmsnorm_add_store: bad sizes (rows %d, dim %d)", n_rows, dim);
+    const bool fast = dim % 4 == 0 && dim <= 8192 && y_stride % 4 == 0 && x_stride % 4 == 0 && low_stride % 4 == 0 &&
+                      (((uintptr_t)y | (uintptr_t)x | (uintptr_t)w | (uintptr_t)low) & 15) == 0;
+    const int nv = (dim + 1023) / 1024;
+#define GO(NV, TW) rmsnorm_add_store_kernel<NV, TW><<<n_rows, 256, 0, stream>>>(y, (const TW*)w, x, (bf16_t*)low, dim, eps, (size_t)y_stride, (size_t)x_stride, (size_t)low_stride)
+#define LAUNCH(TW)                         \
+    do {                                   \
+        if (!fast) GO(0, TW);              \
+        else if (nv <= 1) GO(1, TW);       \
+        else if (nv <= 2) GO(2, TW);       \
+        else if (nv <= 4) GO(4, TW);       \
+        else GO(8, TW);                    \
+    } while (0)
+    if (w_dtype == GI_F32) LAUNCH(float);
+    else if (w_dtype == GI_BF16) LAUNCH(bf16_t);
+    else return gi_fail("rmsnorm_add_store: unknown dtype %d", w_dtype);
+#undef LAUNCH
+#undef GO
+    GI_CHECK_LAUNCH("rmsnorm_add_store");
     return 0;
 }

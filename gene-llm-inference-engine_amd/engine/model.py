@@ -2,6 +2,7 @@
 norm, output head.  It knows parts and the order they run in, not an architecture."""
 from __future__ import annotations
 
+import math
 from pathlib import Path
 from typing import Dict, List, Optional
 
@@ -11,7 +12,8 @@ from ..config import ModelSpec, read_config
 from ..kernels import ops
 from ..parts import LayerCache, StepContext, block_class, linear, model_tensor_needs, norm_class, row_transform_class, stream_part_class, weight_bytes
 from ..parts.linear import activation_dtype_for
-from ..parts.norm import HandedRows, norm_to_hand_on
+from ..parts.norm import HandedRows, ReadyRows, norm_to_hand_on
+from ..parts.transform import LearnedPositions, ScaleRows
 from ..weights import load_tensors, random_tensors
 
 _DTYPES = {"bfloat16": torch.bfloat16, "bf16": torch.bfloat16, "float32": torch.float32, "fp32": torch.float32,
@@ -54,6 +56,8 @@ class DecoderModel:
         self.head = _Head(self.lm_head, self.head_in_dtype)
         self.after_embedding = [row_transform_class(t)(t, tensors, dtype, device) for t in spec.after_embedding]
         self.after_head = [row_transform_class(t)(t, tensors, dtype, device) for t in spec.after_head]
+        # the longest sequence the parts behind the token table allow (a table of positions ends somewhere), or None
+        self.position_limit = min((t.position_limit for t in self.after_embedding if getattr(t, "position_limit", None) is not None), default=None)
         self.run_order = spec.run_order
         for e in spec.run_order:                   # a mixer whose pages another entry reads keeps nothing but keys and values there
             if e.cache_of is not None:
@@ -100,20 +104,21 @@ class DecoderModel:
             if self.before_entry[i] is not None:          # (it changes x: a norm handed on by whoever wrote x last is void)
                 self.before_entry[i].forward(x, ctx)
                 handed = None
-            if getattr(layer, "hands_norm_on", False):
-                if extras or (i + 1 < len(self.run_order) and self.before_entry[i + 1] is not None):
-                    reader = None         # x changes again before anybody reads it
-                elif i + 1 < len(self.run_order):
-                    after = self.layers[self.run_order[i + 1].layer]
-                    reader = after.first_reader() if getattr(after, "hands_norm_on", False) else None
-                else:                     # the head reads every row of the final norm, or a selection, which is not handed on
-                    reader = (self.final_norm, self.head) if ctx.every_row_wanted and trace is None else None
-                handed = layer.forward(x, ctx, cache.layer_cache(i), handed=handed, next_reader=reader)
+            if i + 1 == len(self.run_order):              # the head reads every row of the final norm, or a selection, which is not handed on
+                behind = (self.final_norm, self.head) if ctx.every_row_wanted and trace is None else None
+            elif self.before_entry[i + 1] is not None:    # (x changes again before anybody reads it)
+                behind = None
             else:
-                layer.forward(x, ctx, cache.layer_cache(i))
-                handed = None
-            for part in extras:
-                part.forward(x, ctx)
+                behind = self._first_reader(self.layers[self.run_order[i + 1].layer])
+            stages = [layer, *extras]                     # the block and what follows it, each a reader of x and a writer of it
+            for j, stage in enumerate(stages):
+                caches = (cache.layer_cache(i),) if j == 0 else ()
+                if getattr(stage, "hands_norm_on", False):
+                    reader = self._first_reader(stages[j + 1]) if j + 1 < len(stages) else behind
+                    handed = stage.forward(x, ctx, *caches, handed=handed, next_reader=reader)
+                else:
+                    stage.forward(x, ctx, *caches)
+                    handed = None
             if extras and trace is not None:
                 trace("layer_out", i, x)
         ctx.trace = None
@@ -137,6 +142,10 @@ class DecoderModel:
             transform(logits)
         return logits
 
+    @staticmethod
+    def _first_reader(stage):
+        return stage.first_reader() if getattr(stage, "hands_norm_on", False) else None
+
     def _embed(self, ctx: StepContext, x: torch.Tensor):
         """The rows of the token table into x.  Where the first block's first norm can be taken half applied (`HandedRows`: a few
         single rows of decoding requests in bfloat16, a norm of the form g * x * rsqrt(mean square + eps), a reader whose product
@@ -150,9 +159,23 @@ class DecoderModel:
                 squares = torch.empty((ctx.n_rows, 1), dtype=torch.float32, device=self.device)
                 ops.embed_handing(self.embedding, ctx.tokens, x, norm.handed_weight(), scaled, squares)
                 return HandedRows(norm, x, scaled, squares)
+        transforms = self.after_embedding
+        # a scale and a table of positions behind the token table are one kernel with the fetch, which also leaves the rows as the
+        # first product reads them where they are read without a norm
+        if transforms and type(transforms[-1]) is LearnedPositions and all(type(t) is ScaleRows for t in transforms[:-1]):
+            reader = self._first_reader(first) if first is not None and self.before_entry[0] is None else None
+            norm, part = reader if reader is not None else (None, None)
+            low = None
+            if getattr(norm, "is_identity", False) and getattr(part, "in_dtype", self.dtype) == torch.bfloat16:
+                low = torch.empty(x.shape, dtype=torch.bfloat16, device=self.device)
+            ops.embed_positioned(self.embedding, ctx.tokens, math.prod(float(t.spec.factor) for t in transforms[:-1]), transforms[-1].table, ctx.row_pos, x, low)
+            return None if low is None else ReadyRows(norm, x, low)
         ops.embed(self.embedding, ctx.tokens, x)
-        for transform in self.after_embedding:
-            transform(x)
+        for transform in transforms:
+            if transform.needs_context:
+                transform(x, ctx)
+            else:
+                transform(x)
         return None
 
     def set_trace(self, trace) -> None:
@@ -168,11 +191,11 @@ def load_model(folder, dtype="bfloat16", device="cuda:0") -> DecoderModel:
     configuration is chosen by config.json."""
     dtype = compute_dtype(dtype)
     config = read_config(folder)
-    if hasattr(config, "fit_to_tensors"):          # an architecture some of whose parts a folder may lack looks at the tensors' names
+    if hasattr(config, "fit_to_tensors"):          # an architecture some of whose parts or sizes only the tensors tell looks at their names and shapes
         from ..weights.safetensors_io import SafetensorsFile
         st = SafetensorsFile(Path(folder) / "model.safetensors")
         try:
-            config = config.fit_to_tensors(list(st.entries))
+            config = config.fit_to_tensors({name: entry.shape for name, entry in st.entries.items()})
         finally:
             st.close()
     spec = config.model_spec()

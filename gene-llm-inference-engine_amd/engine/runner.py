@@ -83,6 +83,8 @@ class Runner:
         self.page_size = int(page_size)
         self.max_rows = int(max_rows)
         self.max_positions = int(max_positions or model.spec.max_positions)
+        if getattr(model, "position_limit", None) is not None:          # (a table of positions ends somewhere, whatever the caller would like)
+            self.max_positions = min(self.max_positions, model.position_limit)
         needs, reads_from = model.cache_needs()
         n_pages = max(1, -(-int(max_tokens) // self.page_size))
         self.cache = CacheManager(needs, reads_from, page_size=self.page_size, n_pages=n_pages, max_requests=max_requests,

@@ -35,12 +35,12 @@ _SIGNATURES = {
     "gi_softcap_rows": [c_void_p, c_int, c_int, c_long, c_float, c_void_p],
     "gi_gemm_exact": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_long, c_long, c_long, c_void_p],
     "gi_attention_exact": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_long, c_int,
-                           c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_void_p, c_long, c_void_p],
+                           c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_void_p, c_long, c_int, c_void_p],
     "gi_rmsnorm_add": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_float, c_long, c_long, c_void_p],
     "gi_rmsnorm_add_norm": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_float, c_long, c_long, c_long, c_void_p],
     "gi_norm_rope_store": [c_void_p, c_void_p, c_void_p, c_long, c_long, c_long, c_void_p, c_void_p, c_int, c_float, c_void_p, c_void_p, c_int,
                            c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int, c_int, c_int,
-                           c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_long, c_int, c_float, c_void_p, c_void_p],
+                           c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_long, c_int, c_float, c_void_p, c_float, ctypes.c_double, c_void_p],
     "gi_concat_rows": [c_void_p, c_long, c_int, c_void_p, c_long, c_int, c_void_p, c_int, c_long, c_int, c_void_p],
     "gi_add_weighted": [c_void_p, c_long, c_void_p, c_long, c_float, c_void_p, c_long, c_float, c_int, c_int, c_void_p],
     "gi_add_vector": [c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_void_p],
@@ -81,16 +81,21 @@ _SIGNATURES = {
                               c_void_p],
     "gi_head_gate": [c_void_p, c_int, c_long, c_void_p, c_long, c_int, c_int, c_int, c_void_p],
     "gi_add_rows_gated": [c_void_p, c_long, c_void_p, c_long, c_void_p, c_long, c_int, c_int, c_void_p],
+    "gi_lightning_scan": [c_void_p, c_long, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_long, c_void_p, c_long, c_int, c_int, c_int, c_int,
+                          c_void_p, c_void_p],
+    "gi_row_norm_gate": [c_void_p, c_long, c_void_p, c_long, c_void_p, c_int, c_void_p, c_int, c_long, c_int, c_int, c_float, c_void_p],
+    "gi_embed_positioned": [c_void_p, c_int, c_void_p, c_float, c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p],
+    "gi_rmsnorm_add_store": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_float, c_long, c_long, c_long, c_void_p],
     "gi_segments": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p],
     "gi_mlstm_scan": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_float, c_float, c_void_p, c_void_p, c_int, c_void_p,
                       c_void_p, c_long, c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_void_p],
     "gi_head_norm_gate": [c_void_p, c_long, c_void_p, c_void_p, c_long, c_void_p, c_int, c_void_p, c_int, c_long, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p],
     "gi_gemm_bf16": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_int, c_int, c_int, c_long, c_long, c_long, c_void_p, c_long, c_void_p],
     "gi_attention_prompt_bf16": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int, c_int,
-                                 c_float, c_int, c_void_p, c_void_p, c_int, c_void_p, c_long, c_int, c_void_p, c_void_p, c_long, c_float, c_void_p],
+                                 c_float, c_int, c_void_p, c_void_p, c_int, c_void_p, c_long, c_int, c_void_p, c_void_p, c_long, c_int, c_float, c_void_p],
     "gi_attention_decode_bf16": [c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_long, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                  c_long, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int, c_int,
-                                 c_float, c_int, c_int, c_int, c_void_p, c_void_p, c_long, c_float, c_void_p],
+                                 c_float, c_int, c_int, c_int, c_void_p, c_void_p, c_long, c_int, c_float, c_void_p],
     "gi_random_normal": [c_void_p, c_int, c_long, ctypes.c_ulonglong, ctypes.c_double, ctypes.c_double, c_void_p],
     "gi_probe_stream": [c_void_p, c_void_p, c_long, c_void_p, c_int, c_int, c_void_p],
     "gi_probe_mfma": [c_int, c_void_p, c_int, c_void_p],
@@ -306,6 +311,28 @@ def embed_handing(table, tokens, out, g, scaled, squares):
     return out
 
 
+def embed_positioned(table, tokens, scale, where, positions, x, low=None):
+    """x[t] = table[tokens[t]] * scale + where[positions[t]], float32, and the same in bfloat16 as `low` if given.  where: [positions, dim].
+    table None: x holds the token rows already and gets the positions' rows added."""
+    _dev(table, tokens, where, positions, x, low)
+    n, dim = x.shape
+    if not (where.dim() == 2 and where.shape[1] == dim and where.is_contiguous() and (table is None or (table.dim() == 2 and table.shape[1] == dim and table.is_contiguous()))):
+        raise KernelError("embed_positioned: the tables must be [entries, dim], contiguous")
+    if not (x.dtype == torch.float32 and x.is_contiguous() and (low is None or (low.dtype == torch.bfloat16 and low.shape == x.shape and low.is_contiguous()))):
+        raise KernelError("embed_positioned: x must be float32 [n, dim] and its copy bfloat16 [n, dim], contiguous")
+    if table is not None:
+        _i32(tokens, "embed_positioned: tokens", n)
+    _i32(positions, "embed_positioned: positions", n)
+    _call("gi_embed_positioned", _ptr(table), _code(table, "embed_positioned: table") if table is not None else F32, _ptr(tokens), float(scale), where.data_ptr(),
+          _code(where, "embed_positioned: positions"), where.shape[0], positions.data_ptr(), x.data_ptr(), _ptr(low), n, dim, _stream())
+    return x
+
+
+def add_position_rows(x, where, positions):
+    """x[t] += where[positions[t]]; x float32 [n, dim]."""
+    return embed_positioned(None, None, 1.0, where, positions, x)
+
+
 def rmsnorm_can_gather(x, weight, out) -> bool:
     dim = x.shape[1]
     return (dim % 4 == 0 and dim <= 4096 and x.stride(0) % 4 == 0 and out.stride(0) % 4 == 0 and x.data_ptr() % 16 == 0
@@ -470,12 +497,13 @@ def _check_paged(cache, table, what):
 
 
 def attention_exact(q, cache, out, positions, slots, table, n_heads, n_kv, hd, window=None, scale=None, *, page_size=None, value_dim=None,
-                    chunk=None, sinks=None, gate=None, cap=None):
+                    chunk=None, sinks=None, gate=None, cap=None, channel_gate=None):
     """Each row attends over its request's cached keys up to its own position, no further back than `window` positions and not
     beyond the start of its own chunk of `chunk` positions.  value_dim: channels of a value head (hd if not given); sinks:
     float32 [heads], a score per head that joins the softmax's denominator only; gate: float32 [n, >= heads] (unit inner
-    stride), head h's output is multiplied by sigmoid(gate[t, h]); cap: a scaled score s becomes cap * tanh(s / cap)."""
-    _dev(q, cache, out, positions, slots, table, sinks, gate)
+    stride), head h's output is multiplied by sigmoid(gate[t, h]); channel_gate: float32 [n, heads*value_dim], the output is
+    multiplied by its sigmoid element by element; cap: a scaled score s becomes cap * tanh(s / cap)."""
+    _dev(q, cache, out, positions, slots, table, sinks, gate, channel_gate)
     if cap is not None and not cap > 0:
         raise KernelError("attention: the scores' cap must be positive")
     n = q.shape[0]
@@ -489,15 +517,26 @@ def attention_exact(q, cache, out, positions, slots, table, n_heads, n_kv, hd, w
         _check_paged(cache, table, "attention")
     if sinks is not None and not (sinks.dtype == torch.float32 and sinks.is_contiguous() and sinks.numel() == n_heads):
         raise KernelError("attention: sinks must be float32 [heads]")
-    if gate is not None and not (gate.dtype == torch.float32 and gate.dim() == 2 and gate.shape[0] == n and gate.shape[1] >= n_heads and gate.stride(1) == 1):
-        raise KernelError("attention: the heads' gates must be float32 [n, heads] with unit inner stride")
+    gate, gate_stride, gate_channels = _gates(gate, channel_gate, n, n_heads, vd)
     _i32(positions, "attention: positions", n)
     _i32(slots, "attention: slots", n)
     _call("gi_attention_exact", q.data_ptr(), _code(q, "attention: q"), cache.data_ptr(), _code(cache, "attention: cache"), out.data_ptr(),
           _code(out, "attention: out"), positions.data_ptr(), slots.data_ptr(), table.data_ptr(), table.stride(0), cache.stride(0),
           page_size, n, n_heads, n_kv, hd, vd, int(window or 0), int(chunk or 0), float(scale if scale is not None else hd ** -0.5),
-          float(cap or 0.0), _ptr(sinks), _ptr(gate), gate.stride(0) if gate is not None else 0, _stream())
+          float(cap or 0.0), _ptr(sinks), _ptr(gate), gate_stride, gate_channels, _stream())
     return out
+
+
+def _gates(gate, channel_gate, n, n_heads, vd):
+    """The gate on an attention's output as the kernels take it: (tensor or None, row stride, channels a head: 0 for a gate per head)."""
+    if gate is not None and channel_gate is not None:
+        raise KernelError("attention: a gate per head or one per channel, not both")
+    if gate is not None and not (gate.dtype == torch.float32 and gate.dim() == 2 and gate.shape[0] == n and gate.shape[1] >= n_heads and gate.stride(1) == 1):
+        raise KernelError("attention: the heads' gates must be float32 [n, heads] with unit inner stride")
+    if channel_gate is not None and not (channel_gate.dtype == torch.float32 and channel_gate.shape == (n, n_heads * vd) and channel_gate.stride(1) == 1):
+        raise KernelError("attention: the channels' gates must be float32 [n, heads*value_dim] with unit inner stride")
+    g = gate if gate is not None else channel_gate
+    return g, (g.stride(0) if g is not None else 0), (vd if channel_gate is not None else 0)
 
 
 def rmsnorm_add(y, weight, eps, x):
@@ -510,6 +549,20 @@ def rmsnorm_add(y, weight, eps, x):
         raise KernelError("rmsnorm_add: weight must be [dim]")
     _call("gi_rmsnorm_add", y.data_ptr(), weight.data_ptr(), _code(weight, "rmsnorm_add: weight"), x.data_ptr(), n, dim, float(eps), y.stride(0), x.stride(0), _stream())
     return x
+
+
+def rmsnorm_add_store(y, weight, eps, x, low):
+    """x += weight * norm(y), and low = the rows so made in bfloat16, in one kernel; x and y float32 [n, dim].  Returns low."""
+    _dev(y, weight, x, low)
+    n, dim = x.shape
+    if not (x.dtype == torch.float32 and y.dtype == torch.float32 and y.shape == (n, dim) and low.dtype == torch.bfloat16 and low.shape == (n, dim)
+            and x.stride(1) == 1 and y.stride(1) == 1 and low.stride(1) == 1):
+        raise KernelError("rmsnorm_add_store: x and y must be float32 [n, dim] and the copy bfloat16 [n, dim], with unit inner stride")
+    if not (weight.shape == (dim,) and weight.is_contiguous()):
+        raise KernelError("rmsnorm_add_store: weight must be [dim]")
+    _call("gi_rmsnorm_add_store", y.data_ptr(), weight.data_ptr(), _code(weight, "rmsnorm_add_store: weight"), x.data_ptr(), low.data_ptr(), n, dim, float(eps), y.stride(0),
+          x.stride(0), low.stride(0), _stream())
+    return low
 
 
 def rmsnorm_add_norm(y, weight, eps, x, next_weight, next_eps, out):
@@ -527,7 +580,7 @@ def rmsnorm_add_norm(y, weight, eps, x, next_weight, next_eps, out):
 
 
 def norm_rope_store(q, k, v, q_norm, k_norm, eps, cos, sin, rotary_dim, positions, slots, table, q_out, cache, page_size, n_heads, n_kv, hd, vd,
-                    biases=None, blend=None, keep=None, neighbours=False, unit_rms=False, norm_last=False, v_scale=1.0, norm_all=False):
+                    biases=None, blend=None, keep=None, neighbours=False, unit_rms=False, norm_last=False, v_scale=1.0, norm_all=False, query_growth=None):
     """The general form of `rope_store`: every query and key head is first RMS-normed with q_norm / k_norm [hd] (None: not), then
     the pairs (i, i + rotary_dim/2) of its first rotary_dim channels are turned (cos, sin float32 [n, rotary_dim/2]; None: not);
     queries go to q_out, keys and the values (vd channels a head) into the cache's pages.  k None: the pages are another layer's.
@@ -537,7 +590,11 @@ def norm_rope_store(q, k, v, q_norm, k_norm, eps, cos, sin, rotary_dim, position
     their bias, before any blending).  neighbours: the pairs turned are (2i, 2i + 1).  unit_rms: every query and key head is divided
     by its root mean square (eps inside the root), without weights.  norm_last: the heads' norm comes behind the rotation.
     v_scale: multiplies the values on their way into the pages.  norm_all: q_norm is [heads*hd] and k_norm [kv_heads*hd], and the norm is
-    taken over all heads of a projection at once."""
+    taken over all heads of a projection at once.  query_growth = (coef, every): the finished query of the row at position p times
+    1 + coef * ln(floor((p + 1) / every) + 1).  v may be the same columns as k: the values are then the keys as projected."""
+    coef, every = query_growth if query_growth is not None else (0.0, 0.0)
+    if query_growth is not None and not every > 0:
+        raise KernelError("norm_rope_store: queries grow every so many positions, a positive number")
     if unit_rms and (q_norm is not None or k_norm is not None):
         raise KernelError("norm_rope_store: heads divided by their root mean square have no norm weights")
     _dev(q, k, v, q_norm, k_norm, cos, sin, positions, slots, table, q_out, cache)
@@ -584,7 +641,7 @@ def norm_rope_store(q, k, v, q_norm, k_norm, eps, cos, sin, rotary_dim, position
           _code(q_out, "norm_rope_store: q_out"), _ptr(cache) if k is not None else None, cache_code, cache.stride(0) if k is not None else 0,
           int(page_size), n, n_heads, n_kv, hd, vd, _ptr(q_bias), _ptr(k_bias), _ptr(v_bias), _ptr(other), other.stride(0) if other is not None else 0,
           _ptr(weight), _ptr(keep), keep.stride(0) if keep is not None else 0, (1 if neighbours else 0) | (2 if unit_rms else 0) | (4 if norm_last else 0) | (8 if norm_all else 0), float(v_scale),
-          _ptr(rows_r), _stream())
+          _ptr(rows_r), float(coef), float(every), _stream())
 
 
 def xielu(x, out, params):
@@ -699,6 +756,65 @@ def head_norm_gate(o, gate, weight, eps, out, n_heads, dv, den=None, gate_activa
         raise KernelError(f"head_norm_gate: unknown gate {gate_activation!r}; known: {', '.join(GATES)}")
     _call("gi_head_norm_gate", o.data_ptr(), o.stride(0), _ptr(den), gate.data_ptr(), gate.stride(0), weight.data_ptr(), _code(weight, "head_norm_gate: weight"),
           out.data_ptr(), _code(out, "head_norm_gate: out"), out.stride(0), n, n_heads, dv, float(eps), 1 if shared else 0, GATES[gate_activation], _stream())
+    return out
+
+
+# ------------------------------------------------------------------------------------------------ linear attention with fading memories
+LIGHTNING_MAX_KEY_DIM = 512
+LIGHTNING_CHUNK_ROWS = 64          # rows of a chunk where a long run of rows is cut into chunks that run at once (the library's gi_lightning_chunk_rows)
+LIGHTNING_CHUNKS_FROM = 32         # rows of a step's longest request from which that is done
+
+
+def lightning_powers(decay, device):
+    """The table the kernels read: float32 [heads, 65], every head's decay to the powers 0 .. 64 (taken in 64-bit)."""
+    table = [[float(d) ** i for i in range(LIGHTNING_CHUNK_ROWS + 1)] for d in decay]
+    return torch.tensor(table, dtype=torch.float64).to(torch.float32).to(device).contiguous()
+
+
+def lightning_scan(proj, offsets, powers, seg_start, seg_len, row_slot, state, out, n_heads, dk, dv, rows_per_request=None):
+    """S <- d S + SiLU(k) SiLU(v)^T, out = S^T SiLU(q), per head over every request's rows, from its state slot and back into it.
+    proj: float32 [n, columns] whose columns from `offsets` = (q, k, v) on hold q, k [heads*dk] and v [heads*dv]; powers: what
+    `lightning_powers` gives; state: float32 [slots, >= heads*dk*dv]; out: float32 [n, heads*dv].
+    rows_per_request: the requests' numbers of rows as the host knows them (what seg_len holds).  Given, with a request of
+    LIGHTNING_CHUNKS_FROM rows or more, the rows are cut into chunks that run at once: the same sums in another order, so the results
+    differ by 32-bit rounding from those of rows taken one after the other."""
+    _dev(proj, powers, seg_start, seg_len, row_slot, state, out)
+    n = out.shape[0]
+    q_off, k_off, v_off = offsets
+    _f32_rows(proj, "lightning_scan: the projections", n)
+    if min(offsets) < 0 or max(max(q_off, k_off) + n_heads * dk, v_off + n_heads * dv) > proj.shape[1]:
+        raise KernelError("lightning_scan: the columns named lie outside the projections")
+    if not 1 <= dk <= LIGHTNING_MAX_KEY_DIM:
+        raise KernelError(f"lightning_scan: {dk} key channels are outside what the kernels take (1 to {LIGHTNING_MAX_KEY_DIM})")
+    if not (powers.dtype == torch.float32 and powers.shape == (n_heads, LIGHTNING_CHUNK_ROWS + 1) and powers.is_contiguous()):
+        raise KernelError("lightning_scan: the decays' powers must be float32 [heads, 65]")
+    if not (state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1 and state.shape[1] >= n_heads * dk * dv):
+        raise KernelError("lightning_scan: the state must be float32 [slots, heads*dk*dv]")
+    if not (out.dtype == torch.float32 and out.shape[1] == n_heads * dv and out.stride(1) == 1):
+        raise KernelError("lightning_scan: out must be float32 [n, heads*dv]")
+    _i32(row_slot, "lightning_scan: slots", n)
+    n_chunks, states = 0, None
+    if rows_per_request is not None and max(rows_per_request) >= LIGHTNING_CHUNKS_FROM:
+        if len(rows_per_request) != seg_start.numel() or sum(rows_per_request) != n:
+            raise KernelError("lightning_scan: the requests' numbers of rows do not add up to the step's rows")
+        n_chunks = sum(-(-int(r) // LIGHTNING_CHUNK_ROWS) for r in rows_per_request)
+        states = torch.empty((n_chunks, n_heads, dk, dv), dtype=torch.float32, device=proj.device)
+    _call("gi_lightning_scan", proj.data_ptr(), proj.stride(0), int(q_off), int(k_off), int(v_off), powers.data_ptr(), seg_start.data_ptr(), seg_len.data_ptr(), seg_start.numel(),
+          row_slot.data_ptr(), state.data_ptr(), state.stride(0), out.data_ptr(), out.stride(0), n_heads, dk, dv, n_chunks, _ptr(states), _stream())
+    return out
+
+
+def row_norm_gate(o, gate, weight, eps, out):
+    """out = weight * o * rsqrt(mean(o^2) + eps) * sigmoid(gate), the mean over the whole row; o, gate float32 [n, columns] (unit inner
+    stride), out [n, columns]."""
+    _dev(o, gate, weight, out)
+    n, dim = out.shape
+    for t, name in ((o, "o"), (gate, "gate")):
+        _f32_rows(t, f"row_norm_gate: {name}", n, dim)
+    if not (weight.shape == (dim,) and weight.is_contiguous() and out.stride(1) == 1):
+        raise KernelError("row_norm_gate: weight must be [columns] and out [n, columns]")
+    _call("gi_row_norm_gate", o.data_ptr(), o.stride(0), gate.data_ptr(), gate.stride(0), weight.data_ptr(), _code(weight, "row_norm_gate: weight"), out.data_ptr(),
+          _code(out, "row_norm_gate: out"), out.stride(0), n, dim, float(eps), _stream())
     return out
 
 
@@ -1029,7 +1145,7 @@ def decode_attention_shape(n_decode, n_heads, n_kv, hd, span, target_waves=4096,
 
 
 def attention_bf16(q, cache, out, plan: AttentionPlan, positions, slots, table, n_heads, n_kv, hd, window=None, scale=None,
-                   target_waves: int = 4096, products=None, chunk=None, sinks=None, gate=None, cap=None):
+                   target_waves: int = 4096, products=None, chunk=None, sinks=None, gate=None, cap=None, channel_gate=None):
     """Attention of a step's rows with the matrix-core kernels (bfloat16 cache and out).
 
     `q` holds the rotated queries in bfloat16 and the cache the rows' keys and values; or, for a step
@@ -1037,18 +1153,17 @@ def attention_bf16(q, cache, out, plan: AttentionPlan, positions, slots, table, 
     float32 products and the rotation's tables (k, v None: the pages are another layer's; cos, sin
     None: no rotation): the decode kernel then rotates, writes the cache and attends in one launch.
 
-    chunk, sinks, gate: as `attention_exact` takes them (a mask cut into chunks, a score per head that joins the softmax's
-    denominator only, a gate per row and head on the output)."""
+    chunk, sinks, gate, channel_gate: as `attention_exact` takes them (a mask cut into chunks, a score per head that joins the softmax's
+    denominator only, a gate per row and head on the output, or one per row and channel, whose rows must start at multiples of 16 bytes)."""
     n = out.shape[0]
-    _dev(q, cache, out, positions, slots, table, sinks, gate)
+    _dev(q, cache, out, positions, slots, table, sinks, gate, channel_gate)
     if sinks is not None and not (sinks.dtype == torch.float32 and sinks.is_contiguous() and sinks.numel() == n_heads):
         raise KernelError("attention: sinks must be float32 [heads]")
-    if gate is not None and not (gate.dtype == torch.float32 and gate.dim() == 2 and gate.shape[0] == n and gate.shape[1] >= n_heads and gate.stride(1) == 1):
-        raise KernelError("attention: the heads' gates must be float32 [n, heads] with unit inner stride")
+    gate, gate_stride, gate_channels = _gates(gate, channel_gate, n, n_heads, hd)
     chunk = int(chunk or 0)
     if cap is not None and not cap > 0:
         raise KernelError("attention: the scores' cap must be positive")
-    extras = (chunk, _ptr(sinks), _ptr(gate), gate.stride(0) if gate is not None else 0, float(cap or 0.0))
+    extras = (chunk, _ptr(sinks), _ptr(gate), gate_stride, gate_channels, float(cap or 0.0))
     seen = lambda context, slack: min([context] + ([window + slack] if window else []) + ([chunk + slack] if chunk else []))
     for t, name in ((q, "q"), (cache, "cache"), (out, "out")):
         if not (t is None or t.dtype == torch.bfloat16):
@@ -1114,17 +1229,19 @@ def attention(q, cache, out, ctx, table, n_heads, n_kv, hd, window=None):
 
 
 def attention_general(q, cache, out, ctx, table, n_heads, n_kv, hd, *, page_size, value_dim=None, window=None, chunk=None, scale=None, sinks=None, gate=None,
-                      cap=None):
+                      cap=None, channel_gate=None):
     """Attention of a step's rows for layers with any of: value heads of another size, a scale of their own, a mask cut into
-    chunks, sinks, a gate per head, capped scores."""
+    chunks, sinks, a gate per head or per channel, capped scores."""
     vd = int(value_dim or hd)
     if (vd == hd and cache.dim() == 5 and q.dtype == torch.bfloat16 and cache.dtype == torch.bfloat16 and out.dtype == torch.bfloat16
-            and (gate is None or gate.dtype == torch.float32) and (cap is None or hd <= 128)):          # (capped scores on the matrix cores: tested up to heads of 128)
+            and (gate is None or gate.dtype == torch.float32) and (channel_gate is None or (channel_gate.stride(0) % 4 == 0 and channel_gate.data_ptr() % 16 == 0))
+            and (cap is None or hd <= 128)):          # (capped scores on the matrix cores: tested up to heads of 128)
         plan = _plan_of(ctx)
         if (not plan.n_tiles or attention_bf16_supports(hd, page_size, True)) and (not plan.n_decode or attention_bf16_supports(hd, page_size, False)):
-            return attention_bf16(q, cache, out, plan, ctx.row_pos, ctx.row_slot, table, n_heads, n_kv, hd, window, scale, chunk=chunk, sinks=sinks, gate=gate, cap=cap)
+            return attention_bf16(q, cache, out, plan, ctx.row_pos, ctx.row_slot, table, n_heads, n_kv, hd, window, scale, chunk=chunk, sinks=sinks, gate=gate, cap=cap,
+                                  channel_gate=channel_gate)
     return attention_exact(q, cache, out, ctx.row_pos, ctx.row_slot, table, n_heads, n_kv, hd, window, scale, page_size=page_size,
-                           value_dim=value_dim, chunk=chunk, sinks=sinks, gate=gate, cap=cap)
+                           value_dim=value_dim, chunk=chunk, sinks=sinks, gate=gate, cap=cap, channel_gate=channel_gate)
 
 
 # Up to so many rows the decode kernel rotates and writes the pages itself.  It saves the rotation kernel's launch wherever the

@@ -87,8 +87,9 @@ def _pad_rows(w, multiple=16):
 class Attention(Mixer):
     """Plain (Llama) attention takes the kernels chosen in `qkv_rotate_store_attend`.  A spec that names any of the further
     features (value heads of another size, a scale of its own, a mask cut into chunks, sinks, norms on query and key heads or over
-    the whole projections, a gate per head, a rotation of a part of the head, capped scores) takes the general path: one product with [q; k; v; head gates], one kernel
-    that norms, turns and stores, and the attention kernel that knows all of these."""
+    the whole projections, a gate per head or per channel, a rotation of a part of the head, capped scores, keys that serve as values,
+    queries that grow with the position) takes the general path: one product with [q; k; v; gates], one kernel that norms, turns and
+    stores, and the attention kernel that knows all of these."""
     accepts_deferred_norm = True      # its input goes into `linear` only
     hands_norm_on = True              # `forward` takes `then`, the norm that reads the residual next
     can_overwrite = True              # `forward(..., overwrite=True)` stores its result in `residual` instead of adding onto it
@@ -107,12 +108,28 @@ class Attention(Mixer):
         if not 0 < self.value_dim <= ops.attention_max_head_size():
             raise ValueError(f"attention: value heads of {self.value_dim} channels are outside what the attention kernels take")
         if self.general:
-            stacked = [tensors[s.q_proj]] + ([tensors[s.k_proj], tensors[s.v_proj]] if s.k_proj is not None else [])
+            self.values_are_keys = bool(getattr(s, "values_are_keys", False))
+            if self.values_are_keys and (s.k_proj is None or self.value_dim != s.head_dim or s.v_bias is not None or s.value_family is not None):
+                raise ValueError("attention: keys that serve as values are projected by this layer, one size for both, without a bias or a blend of their own")
+            if self.values_are_keys and self.position is not None and type(self.position).half_split_tables is PositionEncoding.half_split_tables and not (
+                    hasattr(self.position, "partial_tables") or hasattr(self.position, "pair_tables")):
+                raise ValueError("attention: keys that serve as values must not be turned in place before they are stored")
+            stacked = [tensors[s.q_proj]] + ([] if s.k_proj is None else [tensors[s.k_proj]] if self.values_are_keys else [tensors[s.k_proj], tensors[s.v_proj]])
             self.gate_at = sum(w.shape[0] for w in stacked)
-            if s.head_gate is not None:
-                stacked.append(tensors[s.head_gate])
+            self.output_gate = getattr(s, "output_gate", None)
+            if self.output_gate is not None and s.head_gate is not None:
+                raise ValueError("attention: a gate per head or one per channel, not both")
+            if s.head_gate is not None or self.output_gate is not None:
+                stacked.append(tensors[s.head_gate if s.head_gate is not None else self.output_gate])
             self.w_qkv = _pad_rows(torch.cat(stacked, dim=0).contiguous())
             self.sinks = None if s.sinks is None else tensors[s.sinks].float().contiguous()
+            if getattr(s, "sink_score", None) is not None:
+                if self.sinks is not None:
+                    raise ValueError("attention: sinks of its own per head or one score for all, not both")
+                self.sinks = torch.full((s.n_heads,), float(s.sink_score), dtype=torch.float32, device=device)
+            self.query_growth = getattr(s, "query_growth", None)
+            if self.query_growth is not None and not self.query_growth[1] > 0:
+                raise ValueError("attention: queries grow every so many positions, a positive number")
             self.q_norm = None if s.q_norm is None else tensors[s.q_norm]
             self.k_norm = None if s.k_norm is None else tensors[s.k_norm]
             as_f32 = lambda name: None if name is None else tensors[name].float().contiguous()
@@ -145,15 +162,18 @@ class Attention(Mixer):
     @staticmethod
     def _is_general(s) -> bool:
         return (s.k_proj is None or any(v is not None for v in (s.value_dim, s.scale, s.chunk, s.sinks, s.q_norm, s.k_norm, s.head_gate, s.q_bias,
-                                                                 s.k_bias, s.v_bias, s.value_family, s.value_blend, getattr(s, "score_cap", None)))
-                or getattr(s, "qk_unit_rms", False) or getattr(s.position, "kind", None) in ("rotary_partial", "rotary_interleaved"))
+                                                                 s.k_bias, s.v_bias, s.value_family, s.value_blend, getattr(s, "score_cap", None),
+                                                                 getattr(s, "query_growth", None), getattr(s, "sink_score", None), getattr(s, "output_gate", None)))
+                or getattr(s, "values_are_keys", False) or getattr(s, "qk_unit_rms", False) or getattr(s.position, "kind", None) in ("rotary_partial", "rotary_interleaved"))
 
     @classmethod
     def tensor_needs(cls, spec):
         a, kv, d, vd = spec.n_heads * spec.head_dim, spec.n_kv_heads * spec.head_dim, spec.hidden_size, spec.value_dim or spec.head_dim
         needs = [TensorNeed(spec.q_proj, (a, d))]
         if spec.k_proj is not None:            # (a layer that reads another layer's pages has no keys and values of its own)
-            needs += [TensorNeed(spec.k_proj, (kv, d)), TensorNeed(spec.v_proj, (spec.n_kv_heads * vd, d))]
+            needs.append(TensorNeed(spec.k_proj, (kv, d)))
+            if not getattr(spec, "values_are_keys", False):
+                needs.append(TensorNeed(spec.v_proj, (spec.n_kv_heads * vd, d)))
         needs.append(TensorNeed(spec.o_proj, (d, spec.n_heads * vd)))
         whole = getattr(spec, "qk_norm_whole", False)          # one norm over all heads of a projection, with a weight per channel of all heads
         if spec.q_norm is not None:
@@ -164,6 +184,8 @@ class Attention(Mixer):
             needs.append(TensorNeed(spec.sinks, (spec.n_heads,)))
         if spec.head_gate is not None:
             needs.append(TensorNeed(spec.head_gate, (spec.n_heads, d)))
+        if getattr(spec, "output_gate", None) is not None:
+            needs.append(TensorNeed(spec.output_gate, (spec.n_heads * vd, d)))
         if spec.q_bias is not None:
             needs.append(TensorNeed(spec.q_bias, (a,)))
         if spec.k_proj is not None:
@@ -199,8 +221,13 @@ class Attention(Mixer):
             linear(h, self.w_qkv, proj)
         q, k, v = proj[:, :self.a_dim], None, None
         if s.k_proj is not None and cache.writes:
-            k, v = proj[:, self.a_dim:self.a_dim + self.kv_dim], proj[:, self.a_dim + self.kv_dim:self.a_dim + self.kv_dim + s.n_kv_heads * vd]
-        gate = proj[:, self.gate_at:self.gate_at + s.n_heads] if s.head_gate is not None else None
+            k = proj[:, self.a_dim:self.a_dim + self.kv_dim]
+            v = k if self.values_are_keys else proj[:, self.a_dim + self.kv_dim:self.a_dim + self.kv_dim + s.n_kv_heads * vd]
+        gate = channel_gate = None
+        if s.head_gate is not None:
+            gate = proj[:, self.gate_at:self.gate_at + s.n_heads]
+        elif self.output_gate is not None:
+            channel_gate = proj[:, self.gate_at:self.gate_at + s.n_heads * vd]
         neighbours = self.position is not None and hasattr(self.position, "pair_tables")          # pairs (2i, 2i + 1) of a head's first channels
         tables = (*self.position.pair_tables(ctx), self.position.rotary_dim) if neighbours else rotation_tables(self.position, ctx)
         if self.position is not None and tables is None:          # an encoding with kernels of its own turns q and k in place
@@ -220,10 +247,11 @@ class Attention(Mixer):
         ops.norm_rope_store(q, k, v, self.q_norm, self.k_norm if k is not None else None, s.qk_norm_eps, cos, sin, turned, ctx.row_pos, ctx.row_slot,
                             cache.table, q_ready, cache.kv, cache.page_size, s.n_heads, s.n_kv_heads, s.head_dim, vd,
                             biases=biases if any(b is not None for b in biases) else None, blend=blend, keep=keep, neighbours=neighbours,
-                            unit_rms=self.unit_rms, norm_last=self.unit_rms, v_scale=self.out_scale, norm_all=self.norm_whole)
+                            unit_rms=self.unit_rms, norm_last=self.unit_rms, v_scale=self.out_scale, norm_all=self.norm_whole, query_growth=self.query_growth)
         att = torch.empty((T, s.n_heads * vd), dtype=cache.kv.dtype, device=ctx.device)
         return ops.attention_general(q_ready, cache.kv, att, ctx, cache.table, s.n_heads, s.n_kv_heads, s.head_dim, page_size=cache.page_size,
-                                     value_dim=vd, window=s.window, chunk=s.chunk, scale=s.scale, sinks=self.sinks, gate=gate, cap=self.score_cap)
+                                     value_dim=vd, window=s.window, chunk=s.chunk, scale=s.scale, sinks=self.sinks, gate=gate, cap=self.score_cap,
+                                     channel_gate=channel_gate)
 
     out_scale = 1.0
 
@@ -232,7 +260,7 @@ class Attention(Mixer):
         the layer's own pages (the attention is linear in them).  False: the caller weighs the result itself.  (Another layer that
         reads these pages would read the weighed values: a layer whose pages are shared is not asked.)"""
         s = self.spec
-        if not (self.general and s.k_proj is not None and s.value_family is None and s.head_gate is None):
+        if not (self.general and s.k_proj is not None and s.value_family is None and s.head_gate is None and self.output_gate is None):
             return False
         self.out_scale = float(scale)
         return True

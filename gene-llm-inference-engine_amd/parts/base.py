@@ -169,7 +169,8 @@ class PositionEncoding(Part):
 class StreamPart(Part):
     """Something that changes the residual stream x (float32 [T, hidden]) in place between layers: a second input from the
     tokens, a product that mixes the stream with the token rows again.  It reads what it needs of the step from `ctx` (the
-    tokens on the device; `ctx.memo["token_rows"]`, float32 [T, hidden], if it says `needs_token_rows`)."""
+    tokens on the device; `ctx.memo["token_rows"]`, float32 [T, hidden], if it says `needs_token_rows`).  One that says
+    `hands_norm_on` has a block's `first_reader()` and takes a block's keywords `handed` and `next_reader` (behind a layer)."""
     needs_token_rows = False
 
     def forward(self, x: torch.Tensor, ctx: StepContext) -> None:
@@ -178,7 +179,10 @@ class StreamPart(Part):
 
 class RowTransform(Part):
     """An elementwise change of float32 rows in place: what a model may ask for between the token table and the
-    first layer, and on the logits."""
+    first layer, and on the logits.  One that says `needs_context` (behind the token table only) is called with the step's context as
+    well; one that serves so many positions only says how many in `position_limit`."""
+    needs_context = False
+    position_limit: Optional[int] = None
 
     def __call__(self, x: torch.Tensor) -> None:
         raise NotImplementedError

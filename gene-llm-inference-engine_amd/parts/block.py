@@ -4,6 +4,7 @@
     x += mixer(norm_1(x));  x += feed_forward(norm_2(x))
 "sandwich": a norm before and a norm after each half; the feed-forward half may be absent:
     x += post_1(mixer(norm_1(x)));  x += post_2(feed_forward(norm_2(x)))
+    (with `NoNormSpec` in the place before: a norm on each half's output only, the halves read x itself)
 "parallel": one norm, read by the mixer and by the feed-forward (which may be absent):
     h = norm_1(x);  x += mixer(h) + feed_forward(h)
 The residual stream x is float32 [T, hidden] and is changed in place."""
@@ -140,6 +141,8 @@ class SandwichBlock:
             y = torch.zeros_like(x)
             part.forward(h, y, ctx, *cache)
         then, reads = reader if reader is not None else (None, None)
+        if getattr(then, "is_identity", False) and hasattr(post, "add_onto_and_store"):
+            return post.add_onto_and_store(y, x, then, getattr(reads, "in_dtype", ctx.dtype))
         if (then is not None and hasattr(post, "add_onto_then") and type(then) is type(post) and then.weight.dtype == post.weight.dtype
                 and then.weight.shape == post.weight.shape):
             return post.add_onto_then(y, x, then, getattr(reads, "in_dtype", ctx.dtype))

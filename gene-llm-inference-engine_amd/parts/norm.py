@@ -96,6 +96,13 @@ class RmsNorm(Norm):
         ops.rmsnorm_add_norm(y, self.weight, self.eps, x, then.weight, then.eps, out)
         return ReadyRows(then, x, out)
 
+    def add_onto_and_store(self, y, x, then: "NoNorm", out_dtype) -> ReadyRows:
+        """x += norm(y), and x as a reader without a norm takes it (a copy in its dtype, made on the way)."""
+        if out_dtype == torch.float32:
+            self.add_onto(y, x)
+            return ReadyRows(then, x, x)
+        return ReadyRows(then, x, ops.rmsnorm_add_store(y, self.weight, self.eps, x, torch.empty(x.shape, dtype=out_dtype, device=x.device)))
+
     def deferred(self, x, out_dtype, rows=None) -> NormedRows:
         return NormedRows(self, x, out_dtype, rows)
 
@@ -109,4 +116,14 @@ class RmsNorm(Norm):
         return [self.weight]
 
 
+class NoNorm(Norm):
+    """The rows as they are, stored as the reader takes them (float32: the rows themselves, no copy)."""
+    graph_safe = True
+    is_identity = True
+
+    def __call__(self, x, out_dtype):
+        return x if out_dtype == torch.float32 else ops.concat_rows(x, None, torch.empty(x.shape, dtype=out_dtype, device=x.device))
+
+
 register_norm("rmsnorm", RmsNorm)
+register_norm("none", NoNorm)

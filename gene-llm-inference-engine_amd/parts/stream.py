@@ -6,14 +6,19 @@ from __future__ import annotations
 
 import torch
 
+from ..config.spec import NoNormSpec
 from ..kernels import ops
 from ..weights.loader import TensorNeed
 from .base import StreamPart, norm_class, register_stream_part
 from .linear import activation_dtype_for, linear
+from .norm import NoNorm
 
 
 class TokenSideInput(StreamPart):
     graph_safe = True
+    # It reads the stream without a norm: whoever writes the stream before it may leave the rows as its first product reads them, and
+    # its own norm does the same for a reader behind it that has no norm either.
+    hands_norm_on = True
 
     def __init__(self, spec, tensors, dtype, device):
         super().__init__(spec, tensors, dtype, device)
@@ -28,6 +33,10 @@ class TokenSideInput(StreamPart):
             raise ValueError("token side input: the norm must be one that can add its result onto rows")
         self.in_dtype = activation_dtype_for(self.w_gate, dtype)
         self.mid_dtype = activation_dtype_for(self.w_out, dtype)
+        self.rows = NoNorm(NoNormSpec(s.hidden_size), tensors, dtype, device)
+
+    def first_reader(self):
+        return self.rows, self
 
     @classmethod
     def tensor_needs(cls, spec):
@@ -40,23 +49,30 @@ class TokenSideInput(StreamPart):
 
     FEW_ROWS = 16      # up to so many rows (bfloat16) the stream's rounding, the first product and the gate are one kernel
 
-    def forward(self, x, ctx):
+    def _join(self, y, x, ctx, reader):
+        """x += norm(y); the rows a reader without a norm takes, if there is one."""
+        then, reads = reader if reader is not None else (None, None)
+        if getattr(then, "is_identity", False) and hasattr(self.norm, "add_onto_and_store"):
+            return self.norm.add_onto_and_store(y, x, then, getattr(reads, "in_dtype", ctx.dtype))
+        self.norm.add_onto(y, x)
+        return None
+
+    def forward(self, x, ctx, handed=None, next_reader=None):
         s, T, dev = self.spec, ctx.n_rows, ctx.device
         if (T <= self.FEW_ROWS and self.in_dtype == torch.bfloat16 and self.w_gate.dtype == self.table.dtype == self.mid_dtype == torch.bfloat16):
             g = torch.empty((T, s.dim), dtype=torch.bfloat16, device=dev)
             ops.gate_token_columns_rows(x, self.w_gate, self.table, s.first_column, ctx.tokens, g, s.activation)
             y = torch.empty((T, s.hidden_size), dtype=torch.float32, device=dev)
             linear(g, self.w_out, y)
-            self.norm.add_onto(y, x)
-            return
-        rows = x if self.in_dtype == torch.float32 else ops.concat_rows(x, None, torch.empty((T, s.hidden_size), dtype=self.in_dtype, device=dev))
+            return self._join(y, x, ctx, next_reader)
+        rows = handed.materialize() if handed is not None and handed.norm is self.rows else self.rows(x, self.in_dtype)
         u = torch.empty((T, s.dim), dtype=torch.float32, device=dev)
         linear(rows, self.w_gate, u)
         g = torch.empty((T, s.dim), dtype=self.mid_dtype, device=dev)
         ops.gate_token_columns(u, self.table, s.first_column, ctx.tokens, g, s.activation)
         y = torch.empty((T, s.hidden_size), dtype=torch.float32, device=dev)
         linear(g, self.w_out, y)
-        self.norm.add_onto(y, x)
+        return self._join(y, x, ctx, next_reader)
 
 
 class Rejoin(StreamPart):

@@ -1,8 +1,10 @@
 """Elementwise changes of float32 rows in place, for the two places a model may ask for one: between the token
-table and the first layer (`ModelSpec.after_embedding`) and on the logits (`ModelSpec.after_head`)."""
+table and the first layer (`ModelSpec.after_embedding`; a row of a learned table per position among them) and on the logits
+(`ModelSpec.after_head`)."""
 from __future__ import annotations
 
 from ..kernels import ops
+from ..weights.loader import TensorNeed
 from .base import RowTransform, register_row_transform
 
 
@@ -20,5 +22,27 @@ class SoftCap(RowTransform):
         ops.softcap_rows(x, float(self.spec.cap))
 
 
+class LearnedPositions(RowTransform):
+    """x[t] += table[position of row t].  (Behind a scale, or alone, it runs as one kernel with the token table's: `DecoderModel._embed`.)"""
+    graph_safe = True
+    needs_context = True
+
+    def __init__(self, spec, tensors, dtype, device):
+        super().__init__(spec, tensors, dtype, device)
+        self.table = tensors[spec.table]
+        self.position_limit = int(spec.positions)
+
+    @classmethod
+    def tensor_needs(cls, spec):
+        return [TensorNeed(spec.table, (spec.positions, spec.hidden_size))]
+
+    def weights_read_per_step(self):
+        return []                         # (a row per token, as the token table)
+
+    def __call__(self, x, ctx):
+        ops.add_position_rows(x, self.table, ctx.row_pos)
+
+
 register_row_transform("scale", ScaleRows)
+register_row_transform("learned_positions", LearnedPositions)
 register_row_transform("softcap", SoftCap)
