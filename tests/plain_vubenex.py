@@ -109,8 +109,8 @@ def attention_mixer(h, w, m, eps, store=same):
     q, k = (h @ w["q"].T).reshape(T, H, d), (h @ w["k"].T).reshape(T, G, d)
     v = k                                                     # the values are the keys as projected, before their norm
     q, k = rms_norm(q, w["q.norm"], eps), rms_norm(k, w["k.norm"], eps)
-    grow = torch.tensor([query_growth(p, m["q_temp"]["coef"], m["q_temp"]["every"]) for p in range(T)], dtype=q.dtype)
-    q = q * grow[:, None, None]
+    if m.get("q_temp") is not None:
+        q = q * torch.tensor([query_growth(p, m["q_temp"]["coef"], m["q_temp"]["every"]) for p in range(T)], dtype=q.dtype)[:, None, None]
     y = attention_with_an_empty_seat(store(q), store(k), store(v), m["scale"]).reshape(T, H * d)
     return store(y * torch.sigmoid(h @ w["g"].T)) @ w["o"].T
 
@@ -129,10 +129,11 @@ def token_side_input(x, tokens, table, layer, dim, gate, proj, norm, eps, store=
 
 # ------------------------------------------------------------------------------------------------ the model
 class PlainVubenex:
-    def __init__(self, folder, dtype=torch.float64, storage=None):
-        from safetensors.torch import load_file
-        self.cfg = json.loads((Path(folder) / "config.json").read_text())
-        self.w = {k: t.to(dtype) for k, t in load_file(str(Path(folder) / "model.safetensors")).items()}
+    def __init__(self, folder=None, dtype=torch.float64, storage=None, config=None, tensors=None):
+        if folder is not None:
+            from safetensors.torch import load_file
+            config, tensors = json.loads((Path(folder) / "config.json").read_text()), load_file(str(Path(folder) / "model.safetensors"))
+        self.cfg, self.w = config, {k: t.to(dtype) for k, t in tensors.items()}
         self.store = same if storage is None else to_bfloat16_and_back
 
     def layer(self, i, x, tokens):
@@ -158,3 +159,10 @@ class PlainVubenex:
 
     def logits(self, tokens):
         return self.layer_runs(tokens)[1]
+
+    def greedy(self, tokens, n):
+        """The n tokens that follow, the largest logit each time."""
+        tokens = list(tokens)
+        for _ in range(n):
+            tokens.append(int(self.logits(tokens)[-1].argmax()))
+        return tokens[-n:]
