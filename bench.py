@@ -270,6 +270,46 @@ def mimitar_beside_zidevik(args) -> int:
     return 0
 
 
+def vubenex_beside_fekorax(args) -> int:
+    """The Vubenex design at layer shapes of real models beside the Fekorax design (the nearest the engine has: memories without a
+    feed-forward and attention with one in turns, a norm on every sublayer's output, the token table as the head) and the Llama
+    decoder at the same shapes, random weights; measured as `fekorax_beside_llama` measures.  A Vubenex model of L layers here is L/2
+    times [fading memories; attention + feed-forward]: the attention with the Llama layer's heads over the whole context (a norm on
+    every query and key head, the keys as values, queries that grow every 1,024 positions, a gate on every channel), the memories with a
+    quarter as many heads of the same key size and twice the value size (as Fekorax's here); every layer reads 256 columns of the
+    tokens' second table.  The Fekorax model is `fekorax_beside_llama`'s.  One JSON line."""
+    import torch
+    T, batch, L, steps = args.prefill_tokens, args.batch, args.layers or 8, args.steps
+    gen = torch.Generator().manual_seed(1)
+    record = {"metric": "Vubenex beside Fekorax and Llama at equal layer shapes: prefill tok/s, decode ms a step, ms by kernel", "dtype": args.dtype, "layers": L,
+              "prefill_tokens": T, "decode_batch": batch, "data": "synthetic: random weights by formula, uniform random token ids", "sizes": {}}
+    for size in args.sizes.split(","):
+        D, H, G, hd, ff, vocab = FEKORAX_SIZES[size]
+        mlp, heads = dict(kind="dense", ff=ff), max(1, H // 4)
+        llama = dict(architectures=["LlamaForCausalLM"], hidden_size=D, intermediate_size=ff, num_hidden_layers=L, num_attention_heads=H,
+                     num_key_value_heads=G, head_dim=hd, vocab_size=vocab, max_position_embeddings=T + 1024, rope_theta=500000.0, rms_norm_eps=1e-5,
+                     tie_word_embeddings=True)
+        att = lambda source=None: dict(type="attention", mlp=mlp, mixer=dict(
+            heads=H, kv_heads=G, dim=hd, vdim=hd, scale=hd ** -0.5, rot=dict(dims=hd // 2, base=10000.0), mask=dict(size=1024),
+            **({} if source is None else dict(kv_from=source))))
+        mem = dict(type="mlstm", mlp=None, mixer=dict(heads=heads, dim=hd, vdim=2 * hd, gate_cap=12.0))
+        layers = []
+        for i in range(0, L, 4):
+            layers += [mem, att(), mem, att(i + 1)]
+        fekorax = dict(architecture="Fekorax", vocab=vocab, width=D, embedding=dict(scale=D ** 0.5), norm=dict(eps=1e-5), layers=layers[:L], max_positions=T + 1024)
+        fading = dict(type="lightning", mlp=None, mixer=dict(heads=heads, dim=hd, vdim=2 * hd, decay=[1.0 - 0.5 ** (1 + 10 * (i + 1) / heads) for i in range(heads)]))
+        v_att = dict(type="attention", mlp=mlp, mixer=dict(heads=H, kv_heads=G, dim=hd, vdim=hd, scale=hd ** -0.5, q_temp=dict(coef=0.1, every=1024)))
+        vubenex = dict(architecture="Vubenex", vocab=vocab, width=D, embedding=dict(scale=D ** 0.5), norm=dict(eps=1e-5), token_side=dict(dim=256), max_positions=T + 1024,
+                       layers=([fading, v_att] * ((L + 1) // 2))[:L])
+        record["sizes"][size] = {}
+        for name, cfg in (("llama", llama), ("fekorax", fekorax), ("vubenex", vubenex)):
+            if args.only and name not in args.only.split(","):
+                continue
+            record["sizes"][size][name] = _measure_design(cfg, args, T, batch, steps, vocab, gen)
+    print(json.dumps(record))
+    return 0
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -285,8 +325,9 @@ def main() -> int:
     ap.add_argument("--rigalorn", action="store_true", help="another measurement: the Rigalorn design beside Fekorax and Llama at equal layer shapes (see rigalorn_beside_fekorax)")
     ap.add_argument("--zidevik", action="store_true", help="another measurement: the Zidevik design beside Rigalorn and Llama at equal layer shapes (see zidevik_beside_rigalorn)")
     ap.add_argument("--mimitar", action="store_true", help="another measurement: the Mimitar design beside Zidevik, Rigalorn and Llama at equal layer shapes (see mimitar_beside_zidevik)")
-    ap.add_argument("--only", default="", help="with --rigalorn, --zidevik or --mimitar: the designs to measure, of llama, fekorax, rigalorn, zidevik, mimitar (default: all)")
-    ap.add_argument("--sizes", default="1b,8b", help="with --fekorax, --rigalorn, --zidevik or --mimitar: layer shapes, of " + ", ".join(FEKORAX_SIZES))
+    ap.add_argument("--vubenex", action="store_true", help="another measurement: the Vubenex design beside Fekorax and Llama at equal layer shapes (see vubenex_beside_fekorax)")
+    ap.add_argument("--only", default="", help="with --rigalorn, --zidevik, --mimitar or --vubenex: the designs to measure, of llama, fekorax, rigalorn, zidevik, mimitar, vubenex (default: all)")
+    ap.add_argument("--sizes", default="1b,8b", help="with --fekorax, --rigalorn, --zidevik, --mimitar or --vubenex: layer shapes, of " + ", ".join(FEKORAX_SIZES))
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py measures one GPU; --gpus {args.gpus} is not supported by this single-GPU engine")
@@ -300,6 +341,8 @@ def main() -> int:
         return zidevik_beside_rigalorn(args)
     if args.mimitar:
         return mimitar_beside_zidevik(args)
+    if args.vubenex:
+        return vubenex_beside_fekorax(args)
 
     import torch
     from geneinfer_amd.config import LlamaConfig
