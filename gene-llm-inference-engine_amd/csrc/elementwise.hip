@@ -395,9 +395,77 @@ __global__ __launch_bounds__(256) void rmsnorm_add_kernel(const float* __restric
     for (int d = threadIdx.x; d < dim; d += 256) xr[d] += load_f32(w, d) * (scale * yr[d]);
 }
 
+// The three kernels that do so (alone; with the norm that reads x next; with x as a product without a norm reads it), for rows whose length is
+// a multiple of 4 and at most 8,192, aligned: a thread asks for all its numbers of the row at once and keeps them, so the kernel waits for
+// memory once and reads nothing twice.  Which kernel runs is a matter of the row's length and place alone.
+enum AddThen { ADD_ONLY, ADD_NORM, ADD_STORE };
+template <int THEN, int NV, typename TW, typename TO>
+__global__ __launch_bounds__(256) void rmsnorm_add_rows_kernel(const float* __restrict__ y, const TW* __restrict__ w, const TW* __restrict__ w_next, float* __restrict__ x,
+                                                              TO* __restrict__ out, int dim, float eps, float eps_next, size_t y_stride, size_t x_stride, size_t out_stride) {
+    __shared__ float red[4];
+    const float* yr = y + (size_t)blockIdx.x * y_stride;
+    float* xr = x + (size_t)blockIdx.x * x_stride;
+    TO* orow = out + (size_t)blockIdx.x * out_stride;
+    float4 yv[NV], xv[NV], wv[NV], nv[NV];
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int d = min(4 * ((int)threadIdx.x + 256 * i), dim - 4);
+        yv[i] = load4(yr + d), xv[i] = load4(xr + d), wv[i] = load4(w + d);
+        if constexpr (THEN == ADD_NORM) nv[i] = load4(w_next + d);
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const float s = (yv[i].x * yv[i].x + yv[i].y * yv[i].y) + (yv[i].z * yv[i].z + yv[i].w * yv[i].w);
+        ss += 4 * ((int)threadIdx.x + 256 * i) < dim ? s : 0.f;
+    }
+    const float r = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)dim + eps);
+    float sx = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int d = 4 * ((int)threadIdx.x + 256 * i);
+        float4 v = xv[i];
+        v.x += wv[i].x * (r * yv[i].x), v.y += wv[i].y * (r * yv[i].y), v.z += wv[i].z * (r * yv[i].z), v.w += wv[i].w * (r * yv[i].w);
+        if (d < dim) {
+            store4(xr + d, v.x, v.y, v.z, v.w);
+            if constexpr (THEN == ADD_STORE) store4(orow + d, v.x, v.y, v.z, v.w);
+            sx += (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+        }
+        xv[i] = v;
+    }
+    if constexpr (THEN == ADD_NORM) {
+        const float rn = 1.0f / sqrtf(block_sum<256>(sx, red) / (float)dim + eps_next);
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int d = 4 * ((int)threadIdx.x + 256 * i);
+            if (d < dim) store4(orow + d, nv[i].x * (rn * xv[i].x), nv[i].y * (rn * xv[i].y), nv[i].z * (rn * xv[i].z), nv[i].w * (rn * xv[i].w));
+        }
+    }
+}
+
+static bool add_rows_takes(int dim, const void* y, long y_stride, const void* x, long x_stride, const void* w, const void* w_next, const void* out, long out_stride) {
+    return dim % 4 == 0 && dim <= 8192 && y_stride % 4 == 0 && x_stride % 4 == 0 && out_stride % 4 == 0 &&
+           (((uintptr_t)y | (uintptr_t)x | (uintptr_t)w | (uintptr_t)w_next | (uintptr_t)out) & 15) == 0;
+}
+
+template <int THEN, typename TW, typename TO>
+static void add_rows(const float* y, const TW* w, const TW* w_next, float* x, TO* out, int n_rows, int dim, float eps, float eps_next, long y_stride, long x_stride, long out_stride,
+                     hipStream_t stream) {
+#define GO(NV) rmsnorm_add_rows_kernel<THEN, NV, TW, TO><<<n_rows, 256, 0, stream>>>(y, w, w_next, x, out, dim, eps, eps_next, (size_t)y_stride, (size_t)x_stride, (size_t)out_stride)
+    if (dim <= 1024) GO(1); else if (dim <= 2048) GO(2); else if (dim <= 4096) GO(4); else GO(8);
+#undef GO
+}
+
 GI_API int gi_rmsnorm_add(const float* y, const void* w, int w_dtype, float* x, int n_rows, int dim, float eps, long y_stride, long x_stride,
                           hipStream_t stream) {
     GI_REQUIRE(n_rows > 0 && dim > 0 && y_stride >= dim && x_stride >= dim, "rmsnorm_add: bad sizes (rows %d, dim %d)", n_rows, dim);
+    if (add_rows_takes(dim, y, y_stride, x, x_stride, w, nullptr, nullptr, 0)) {
+        if (w_dtype == GI_F32) add_rows<ADD_ONLY>(y, (const float*)w, (const float*)nullptr, x, (float*)nullptr, n_rows, dim, eps, 0.f, y_stride, x_stride, 0, stream);
+        else if (w_dtype == GI_BF16) add_rows<ADD_ONLY>(y, (const bf16_t*)w, (const bf16_t*)nullptr, x, (float*)nullptr, n_rows, dim, eps, 0.f, y_stride, x_stride, 0, stream);
+        else return gi_fail("rmsnorm_add: unknown dtype %d", w_dtype);
+        GI_CHECK_LAUNCH("rmsnorm_add");
+        return 0;
+    }
     if (w_dtype == GI_F32) rmsnorm_add_kernel<float><<<n_rows, 256, 0, stream>>>(y, (const float*)w, x, dim, eps, (size_t)y_stride, (size_t)x_stride);
     else if (w_dtype == GI_BF16) rmsnorm_add_kernel<bf16_t><<<n_rows, 256, 0, stream>>>(y, (const bf16_t*)w, x, dim, eps, (size_t)y_stride, (size_t)x_stride);
     else return gi_fail("rmsnorm_add: unknown dtype %d", w_dtype);
@@ -523,6 +591,46 @@ __global__ __launch_bounds__(64) void norm_rope_store_kernel(const float* __rest
     }
 }
 
+// The same for layers whose heads are normed and not turned (no biases, no blend), heads of 16 to 256 channels, a power of two, aligned: four
+// channels a lane, so a wave takes several heads at once (of one row for the queries, whose heads lie side by side; of one key/value head
+// over neighbouring rows for the keys, whose values then leave as neighbouring places of a page), and where the values are the keys
+// they are read once.
+template <int LANES, typename TQ, typename TC, typename TW>
+__global__ __launch_bounds__(256) void norm_store_kernel(const float* __restrict__ q, const float* __restrict__ k, const float* __restrict__ v, long ldq, long ldk, long ldv,
+                                                        const TW* __restrict__ q_norm, const TW* __restrict__ k_norm, float eps, const int* __restrict__ pos,
+                                                        const int* __restrict__ slot, const int* __restrict__ table, int table_stride, TQ* __restrict__ q_out,
+                                                        TC* __restrict__ cache, long page_stride, int page_size, int n_rows, int n_heads, int n_kv, float v_scale,
+                                                        float q_coef, double q_every, int q_waves) {
+    constexpr int HD = 4 * LANES, HEADS = 64 / LANES;              // heads a wave takes
+    const int lane = threadIdx.x & 63, d = 4 * (lane % LANES);
+    int wave = blockIdx.x * 4 + (threadIdx.x >> 6);
+    const bool is_q = wave < q_waves;
+    if (!is_q) wave -= q_waves;
+    const int item = wave * HEADS + lane / LANES, items = n_rows * (is_q ? n_heads : n_kv), in = min(item, items - 1);
+    const int t = is_q ? in / n_heads : in % n_rows, h = is_q ? in % n_heads : in / n_rows;
+    const float4 x = load4((is_q ? q + (size_t)t * ldq : k + (size_t)t * ldk) + h * HD + d), w = load4((is_q ? q_norm : k_norm) + d);
+    const int p = pos[t];
+    float ss = (x.x * x.x + x.y * x.y) + (x.z * x.z + x.w * x.w);
+#pragma unroll
+    for (int off = LANES / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
+    const float r = 1.0f / sqrtf(ss / (float)HD + eps);
+    if (item >= items) return;
+    if (is_q) {
+        const float grown = q_every > 0.0 ? fmaf(q_coef, logf((float)(floor((double)(p + 1) / q_every) + 1.0)), 1.0f) : 1.0f;
+        store4(q_out + ((size_t)t * n_heads + h) * HD + d, w.x * (r * x.x) * grown, w.y * (r * x.y) * grown, w.z * (r * x.z) * grown, w.w * (r * x.w) * grown);
+        return;
+    }
+    TC* page = cache + (size_t)table[(size_t)slot[t] * table_stride + p / page_size] * page_stride;
+    const int place = p % page_size;
+    store4(page + ((size_t)h * page_size + place) * HD + d, w.x * (r * x.x), w.y * (r * x.y), w.z * (r * x.z), w.w * (r * x.w));
+    const float4 y = v == k ? x : load4(v + (size_t)t * ldv + h * HD + d);
+    TC* vdst = page + (size_t)n_kv * page_size * HD + ((size_t)h * HD + d) * page_size + place;
+    store_f32(vdst, 0, v_scale * y.x);
+    store_f32(vdst, page_size, v_scale * y.y);
+    store_f32(vdst, 2 * (size_t)page_size, v_scale * y.z);
+    store_f32(vdst, 3 * (size_t)page_size, v_scale * y.w);
+}
+
 GI_API int gi_norm_rope_store(const float* q, const float* k, const float* v, long ldq, long ldk, long ldv, const void* q_norm, const void* k_norm,
                               int norm_dtype, float eps, const float* cos_t, const float* sin_t, int rot, const int* pos, const int* slot,
                               const int* table, int table_stride, void* q_out, int q_dtype, void* cache, int cache_dtype, long page_stride,
@@ -547,6 +655,34 @@ GI_API int gi_norm_rope_store(const float* q, const float* k, const float* v, lo
     GI_REQUIRE(k == nullptr || (v != nullptr && cache != nullptr && table != nullptr && page_size > 0 && page_stride >= (long)n_kv * page_size * (hd + vd)),
                "norm_rope_store: a cache write needs v, a cache, a table and a page stride of at least n_kv*page_size*(hd+vd)");
     GI_REQUIRE(n_heads + 2 * n_kv <= 65535, "norm_rope_store: too many heads");
+    const bool plain = k != nullptr && q_norm != nullptr && k_norm != nullptr && cos_t == nullptr && flags == 0 && q_bias == nullptr && k_bias == nullptr && v_bias == nullptr &&
+                       v_other == nullptr && v_keep == nullptr && hd == vd && hd >= 16 && hd <= 256 && (hd & (hd - 1)) == 0 && ldq % 4 == 0 && ldk % 4 == 0 && ldv % 4 == 0 &&
+                       page_stride % 4 == 0 && (long)n_rows * n_heads < 2147483647L / 2 &&
+                       (((uintptr_t)q | (uintptr_t)k | (uintptr_t)v | (uintptr_t)q_norm | (uintptr_t)k_norm | (uintptr_t)q_out | (uintptr_t)cache) & 15) == 0;
+    if (plain) {
+        const int per = 256 / hd, q_waves = (n_rows * n_heads + per - 1) / per, k_waves = (n_rows * n_kv + per - 1) / per;
+        const unsigned blocks = (unsigned)((q_waves + k_waves + 3) / 4);
+#define LAUNCH_(L, TQ, TC, TW)                                                                                                                          \
+    norm_store_kernel<L, TQ, TC, TW><<<blocks, 256, 0, stream>>>(q, k, v, ldq, ldk, ldv, (const TW*)q_norm, (const TW*)k_norm, eps, pos, slot, table,    \
+                                                                 table_stride, (TQ*)q_out, (TC*)cache, page_stride, page_size, n_rows, n_heads, n_kv, v_scale, q_coef, \
+                                                                 q_every, q_waves)
+#define LAUNCH(TQ, TC, TW)                                                  \
+    do {                                                                    \
+        if (hd == 16) LAUNCH_(4, TQ, TC, TW);                               \
+        else if (hd == 32) LAUNCH_(8, TQ, TC, TW);                          \
+        else if (hd == 64) LAUNCH_(16, TQ, TC, TW);                         \
+        else if (hd == 128) LAUNCH_(32, TQ, TC, TW);                        \
+        else LAUNCH_(64, TQ, TC, TW);                                       \
+    } while (0)
+        if (q_dtype == GI_F32 && cache_dtype == GI_F32 && norm_dtype == GI_F32) LAUNCH(float, float, float);
+        else if (q_dtype == GI_BF16 && cache_dtype == GI_BF16 && norm_dtype == GI_BF16) LAUNCH(bf16_t, bf16_t, bf16_t);
+        else if (q_dtype == GI_BF16 && cache_dtype == GI_BF16 && norm_dtype == GI_F32) LAUNCH(bf16_t, bf16_t, float);
+        else return gi_fail("norm_rope_store: dtypes (%d, %d, %d) are not served", q_dtype, cache_dtype, norm_dtype);
+#undef LAUNCH
+#undef LAUNCH_
+        GI_CHECK_LAUNCH("norm_rope_store (plain)");
+        return 0;
+    }
     dim3 grid(n_rows, n_heads + (k ? 2 * n_kv : 0));
 #define LAUNCH(TQ, TC, TW)                                                                                                                    \
     norm_rope_store_kernel<TQ, TC, TW><<<grid, 64, 0, stream>>>(q, k, v, ldq, ldk, ldv, (const TW*)q_norm, (const TW*)k_norm, eps, cos_t, sin_t, rot, pos, \
@@ -648,9 +784,13 @@ __global__ __launch_bounds__(256) void rmsnorm_add_norm_kernel(const float* __re
 GI_API int gi_rmsnorm_add_norm(const float* y, const void* w, const void* w_next, int w_dtype, float* x, void* out, int out_dtype, int n_rows, int dim,
                                float eps, float eps_next, long y_stride, long x_stride, long out_stride, hipStream_t stream) {
     GI_REQUIRE(n_rows > 0 && dim > 0 && y_stride >= dim && x_stride >= dim && out_stride >= dim, "rmsnorm_add_norm: bad sizes (rows %d, dim %d)", n_rows, dim);
+    const bool whole = add_rows_takes(dim, y, y_stride, x, x_stride, w, w_next, out, out_stride);
 #define LAUNCH(TW, TO)                                                                                                                            \
-    rmsnorm_add_norm_kernel<TW, TO><<<n_rows, 256, 0, stream>>>(y, (const TW*)w, x, (const TW*)w_next, (TO*)out, dim, eps, eps_next, (size_t)y_stride, \
-                                                                (size_t)x_stride, (size_t)out_stride)
+    do {                                                                                                                                          \
+        if (whole) add_rows<ADD_NORM>(y, (const TW*)w, (const TW*)w_next, x, (TO*)out, n_rows, dim, eps, eps_next, y_stride, x_stride, out_stride, stream); \
+        else rmsnorm_add_norm_kernel<TW, TO><<<n_rows, 256, 0, stream>>>(y, (const TW*)w, x, (const TW*)w_next, (TO*)out, dim, eps, eps_next, (size_t)y_stride, \
+                                                                         (size_t)x_stride, (size_t)out_stride);                                   \
+    } while (0)
     if (w_dtype == GI_F32 && out_dtype == GI_F32) LAUNCH(float, float);
     else if (w_dtype == GI_F32 && out_dtype == GI_BF16) LAUNCH(float, bf16_t);
     else if (w_dtype == GI_BF16 && out_dtype == GI_F32) LAUNCH(bf16_t, float);
@@ -766,10 +906,84 @@ __global__ __launch_bounds__(256) void gate_token_columns_rows_kernel(const floa
     }
 }
 
-GI_API int gi_gate_token_columns_rows(const float* x, long ldx, const void* w, int w_dtype, long ldw, int width, const void* table, int table_dtype, long ldt, int first,
+// The same for rows that allow loads of 16 bytes, x in bfloat16 or rounded to it on the way: a workgroup makes two outputs of up to eight rows,
+// so that a weight is read once for all of them; a thread takes eight neighbouring columns of everything at once, and the sixteen sums are
+// added over the lanes by halves (a lane keeps eight of them, then four, two, one) and over the four waves through LDS.
+__device__ __forceinline__ void load8(const bf16_t* p, float* v) {
+    const uint4 raw = *reinterpret_cast<const uint4*>(p);
+    v[0] = __uint_as_float(raw.x << 16), v[1] = __uint_as_float(raw.x & 0xffff0000u), v[2] = __uint_as_float(raw.y << 16), v[3] = __uint_as_float(raw.y & 0xffff0000u);
+    v[4] = __uint_as_float(raw.z << 16), v[5] = __uint_as_float(raw.z & 0xffff0000u), v[6] = __uint_as_float(raw.w << 16), v[7] = __uint_as_float(raw.w & 0xffff0000u);
+}
+__device__ __forceinline__ void load8(const float* p, float* v) {
+    const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
+    const float raw[8] = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] = bf16_to_f32(f32_to_bf16(raw[i]));
+}
+
+template <typename TX>
+__global__ __launch_bounds__(256) void gate_token_columns_few_kernel(const TX* __restrict__ x, long ldx, const bf16_t* __restrict__ w, long ldw, int width,
+                                                                    const bf16_t* __restrict__ table, long ldt, int first, const int* __restrict__ tokens,
+                                                                    bf16_t* __restrict__ out, long ldo, int n_rows, int dim, int act) {
+    constexpr int RB = 8, JB = 2;                                 // rows and outputs of a workgroup
+    __shared__ float part[4][RB * JB];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, j0 = blockIdx.x * JB, t0 = blockIdx.y * RB;
+    // the sum this thread finishes at the end, if it is one of the first sixteen, and its number of the token's row, asked for first (two
+    // loads that depend on each other)
+    const int e = threadIdx.x % (RB * JB), t = t0 + e / JB, j = j0 + e % JB;
+    const float column = load_f32(table + (size_t)tokens[min(t, n_rows - 1)] * ldt + first, min(j, dim - 1));
+    float sum[RB * JB] = {};
+#pragma unroll 2
+    for (int d = threadIdx.x * 8; d < width; d += 2048) {
+        float wv[JB][8], xv[RB][8];
+#pragma unroll
+        for (int j = 0; j < JB; ++j) load8(w + (size_t)min(j0 + j, dim - 1) * ldw + d, wv[j]);
+#pragma unroll
+        for (int t = 0; t < RB; ++t) load8(x + (size_t)min(t0 + t, n_rows - 1) * ldx + d, xv[t]);
+#pragma unroll
+        for (int t = 0; t < RB; ++t)
+#pragma unroll
+            for (int j = 0; j < JB; ++j)
+#pragma unroll
+                for (int i = 0; i < 8; ++i) sum[t * JB + j] = fmaf(xv[t][i], wv[j][i], sum[t * JB + j]);
+    }
+#pragma unroll
+    for (int half = 8, off = 32; half >= 1; half >>= 1, off >>= 1) {
+        const bool upper = lane & off;
+#pragma unroll
+        for (int i = 0; i < half; ++i) {
+            const float keep = upper ? sum[i + half] : sum[i], give = upper ? sum[i] : sum[i + half];
+            sum[i] = keep + __shfl_xor(give, off, 64);
+        }
+    }
+    sum[0] += __shfl_xor(sum[0], 2, 64);
+    sum[0] += __shfl_xor(sum[0], 1, 64);
+    if ((lane & 3) == 0) part[wave][lane >> 2] = sum[0];          // (the lane's bits 5, 4, 3, 2 are the sum's number)
+    __syncthreads();
+    if (threadIdx.x >= RB * JB || t >= n_rows || j >= dim) return;
+    const float s = (part[0][e] + part[1][e]) + (part[2][e] + part[3][e]);
+    const float g = act == 1 ? 0.5f * s * (1.0f + tanhf(0.7978845608028654f * (s + 0.044715f * s * s * s))) : s / (1.0f + expf(-s));
+    store_f32(out + (size_t)t * ldo, j, g * column);
+}
+
+GI_API int gi_gate_token_columns_rows(const void* xv, int x_dtype, long ldx, const void* w, int w_dtype, long ldw, int width, const void* table, int table_dtype, long ldt, int first,
                                       const int* tokens, void* out, int out_dtype, long ldo, int n_rows, int dim, int act, int round_rows, hipStream_t stream) {
     GI_REQUIRE(n_rows > 0 && dim > 0 && width > 0 && ldx >= width && ldw >= width && ldo >= dim && first >= 0 && ldt >= first + dim && (act == 0 || act == 1),
                "gate_token_columns_rows: bad sizes (rows %d, width %d, dim %d, columns from %d of %ld)", n_rows, width, dim, first, ldt);
+    const bool low = x_dtype == GI_BF16;
+    if (w_dtype == GI_BF16 && table_dtype == GI_BF16 && out_dtype == GI_BF16 && round_rows && width % 8 == 0 && ldw % 8 == 0 && ldx % (low ? 8 : 4) == 0 &&
+        (((uintptr_t)xv | (uintptr_t)w) & 15) == 0) {
+        dim3 few((dim + 1) / 2, (n_rows + 7) / 8);
+        GI_REQUIRE(few.y <= 65535, "gate_token_columns_rows: too many rows");
+        if (low) gate_token_columns_few_kernel<bf16_t><<<few, 256, 0, stream>>>((const bf16_t*)xv, ldx, (const bf16_t*)w, ldw, width, (const bf16_t*)table, ldt, first, tokens, (bf16_t*)out,
+                                                                               ldo, n_rows, dim, act);
+        else gate_token_columns_few_kernel<float><<<few, 256, 0, stream>>>((const float*)xv, ldx, (const bf16_t*)w, ldw, width, (const bf16_t*)table, ldt, first, tokens, (bf16_t*)out, ldo,
+                                                                          n_rows, dim, act);
+        GI_CHECK_LAUNCH("gate_token_columns_rows");
+        return 0;
+    }
+    GI_REQUIRE(!low, "gate_token_columns_rows: rows in bfloat16 need bfloat16 weights, a width that is a multiple of 8 and rows that start at multiples of 16 bytes");
+    const float* x = (const float*)xv;
     dim3 grid(n_rows, (dim + 3) / 4);
     GI_REQUIRE(grid.y <= 65535, "gate_token_columns_rows: too many columns");
 #define LAUNCH(TW, TT, TO)                                                                                                                            \
@@ -833,71 +1047,37 @@ GI_API int gi_embed_positioned(const void* table, int table_dtype, const int* to
 
 // ------------------------------------------------- a norm on a sublayer's output, added on, and the sum as a product reads it
 // x[t] += w * norm(y[t]), and low[t] = bfloat16(x[t]): what a layer does whose norms follow its sublayers and whose next sublayer reads x
-// itself.  NV > 0: rows whose length is a multiple of 4 and at most 1024 NV, aligned: a thread asks for all its numbers at once and
-// keeps them.
-template <int NV, typename TW>
+// itself.  Rows whose length is a multiple of 4 and at most 8,192, aligned, take `rmsnorm_add_rows_kernel` above.
+template <typename TW>
 __global__ __launch_bounds__(256) void rmsnorm_add_store_kernel(const float* __restrict__ y, const TW* __restrict__ w, float* __restrict__ x, bf16_t* __restrict__ low,
                                                                int dim, float eps, size_t y_stride, size_t x_stride, size_t low_stride) {
     __shared__ float red[4];
     const float* yr = y + (size_t)blockIdx.x * y_stride;
     float* xr = x + (size_t)blockIdx.x * x_stride;
     bf16_t* lr = low + (size_t)blockIdx.x * low_stride;
-    if constexpr (NV > 0) {
-        float4 yv[NV], xv[NV], wv[NV];
-        float ss = 0.f;
-#pragma unroll
-        for (int i = 0; i < NV; ++i) {
-            const int d = min(4 * ((int)threadIdx.x + 256 * i), dim - 4);
-            yv[i] = load4(yr + d), xv[i] = load4(xr + d), wv[i] = load4(w + d);
-        }
-#pragma unroll
-        for (int i = 0; i < NV; ++i) {
-            const float s = (yv[i].x * yv[i].x + yv[i].y * yv[i].y) + (yv[i].z * yv[i].z + yv[i].w * yv[i].w);
-            ss += 4 * ((int)threadIdx.x + 256 * i) < dim ? s : 0.f;
-        }
-        const float r = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)dim + eps);
-#pragma unroll
-        for (int i = 0; i < NV; ++i) {
-            const int d = 4 * ((int)threadIdx.x + 256 * i);
-            if (d < dim) {
-                const float a = xv[i].x + wv[i].x * (r * yv[i].x), b = xv[i].y + wv[i].y * (r * yv[i].y);
-                const float c = xv[i].z + wv[i].z * (r * yv[i].z), e = xv[i].w + wv[i].w * (r * yv[i].w);
-                store4(xr + d, a, b, c, e);
-                store4(lr + d, a, b, c, e);
-            }
-        }
-    } else {
-        float ss = 0.f;
-        for (int d = threadIdx.x; d < dim; d += 256) ss = fmaf(yr[d], yr[d], ss);
-        const float r = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)dim + eps);
-        for (int d = threadIdx.x; d < dim; d += 256) {
-            const float v = xr[d] + load_f32(w, d) * (r * yr[d]);
-            xr[d] = v;
-            lr[d] = f32_to_bf16(v);
-        }
+    float ss = 0.f;
+    for (int d = threadIdx.x; d < dim; d += 256) ss = fmaf(yr[d], yr[d], ss);
+    const float r = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)dim + eps);
+    for (int d = threadIdx.x; d < dim; d += 256) {
+        const float v = xr[d] + load_f32(w, d) * (r * yr[d]);
+        xr[d] = v;
+        lr[d] = f32_to_bf16(v);
     }
 }
 
 GI_API int gi_rmsnorm_add_store(const float* y, const void* w, int w_dtype, float* x, void* low, int n_rows, int dim, float eps, long y_stride, long x_stride, long low_stride,
                                 hipStream_t stream) {
     GI_REQUIRE(n_rows > 0 && dim > 0 && y_stride >= dim && x_stride >= dim && low_stride >= dim && low != nullptr, "rmsnorm_add_store: bad sizes (rows %d, dim %d)", n_rows, dim);
-    const bool fast = dim % 4 == 0 && dim <= 8192 && y_stride % 4 == 0 && x_stride % 4 == 0 && low_stride % 4 == 0 &&
-                      (((uintptr_t)y | (uintptr_t)x | (uintptr_t)w | (uintptr_t)low) & 15) == 0;
-    const int nv = (dim + 1023) / 1024;
-#define GO(NV, TW) rmsnorm_add_store_kernel<NV, TW><<<n_rows, 256, 0, stream>>>(y, (const TW*)w, x, (bf16_t*)low, dim, eps, (size_t)y_stride, (size_t)x_stride, (size_t)low_stride)
-#define LAUNCH(TW)                         \
-    do {                                   \
-        if (!fast) GO(0, TW);              \
-        else if (nv <= 1) GO(1, TW);       \
-        else if (nv <= 2) GO(2, TW);       \
-        else if (nv <= 4) GO(4, TW);       \
-        else GO(8, TW);                    \
-    } while (0)
-    if (w_dtype == GI_F32) LAUNCH(float);
-    else if (w_dtype == GI_BF16) LAUNCH(bf16_t);
+    if (add_rows_takes(dim, y, y_stride, x, x_stride, w, nullptr, low, low_stride)) {
+        if (w_dtype == GI_F32) add_rows<ADD_STORE>(y, (const float*)w, (const float*)nullptr, x, (bf16_t*)low, n_rows, dim, eps, 0.f, y_stride, x_stride, low_stride, stream);
+        else if (w_dtype == GI_BF16) add_rows<ADD_STORE>(y, (const bf16_t*)w, (const bf16_t*)nullptr, x, (bf16_t*)low, n_rows, dim, eps, 0.f, y_stride, x_stride, low_stride, stream);
+        else return gi_fail("rmsnorm_add_store: unknown dtype %d", w_dtype);
+        GI_CHECK_LAUNCH("rmsnorm_add_store");
+        return 0;
+    }
+    if (w_dtype == GI_F32) rmsnorm_add_store_kernel<float><<<n_rows, 256, 0, stream>>>(y, (const float*)w, x, (bf16_t*)low, dim, eps, (size_t)y_stride, (size_t)x_stride, (size_t)low_stride);
+    else if (w_dtype == GI_BF16) rmsnorm_add_store_kernel<bf16_t><<<n_rows, 256, 0, stream>>>(y, (const bf16_t*)w, x, (bf16_t*)low, dim, eps, (size_t)y_stride, (size_t)x_stride, (size_t)low_stride);
     else return gi_fail("rmsnorm_add_store: unknown dtype %d", w_dtype);
-#undef LAUNCH
-#undef GO
     GI_CHECK_LAUNCH("rmsnorm_add_store");
     return 0;
 }

@@ -30,6 +30,7 @@ def compute_dtype(name) -> torch.dtype:
 class _Head:
     """The output head as the reader of the final norm: asked, like a part, whether it takes that norm half applied."""
     accepts_deferred_norm = True
+    takes_ready_rows = True                  # ... or wholly applied by whoever wrote the rows
 
     def __init__(self, weight: torch.Tensor, in_dtype: torch.dtype):
         self.weight, self.in_dtype = weight, in_dtype

@@ -45,7 +45,7 @@ _SIGNATURES = {
     "gi_add_weighted": [c_void_p, c_long, c_void_p, c_long, c_float, c_void_p, c_long, c_float, c_int, c_int, c_void_p],
     "gi_add_vector": [c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_void_p],
     "gi_gate_token_columns": [c_void_p, c_long, c_void_p, c_int, c_long, c_int, c_void_p, c_void_p, c_int, c_long, c_int, c_int, c_int, c_void_p],
-    "gi_gate_token_columns_rows": [c_void_p, c_long, c_void_p, c_int, c_long, c_int, c_void_p, c_int, c_long, c_int, c_void_p, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int,
+    "gi_gate_token_columns_rows": [c_void_p, c_int, c_long, c_void_p, c_int, c_long, c_int, c_void_p, c_int, c_long, c_int, c_void_p, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int,
                                    c_void_p],
     "gi_ssm_conv": [c_void_p, c_long, c_void_p, c_int, c_void_p, c_void_p, c_long, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
     "gi_ssm_tail": [c_void_p, c_long, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_long, c_int, c_int, c_void_p],
@@ -1613,20 +1613,31 @@ def gate_token_columns(u, table, first, tokens, out, activation="gelu_tanh"):
     return out
 
 
+def gate_token_columns_rows_takes(x, w) -> bool:
+    """Whether `gate_token_columns_rows` reads these bfloat16 rows."""
+    return (x.dtype == w.dtype == torch.bfloat16 and x.dim() == 2 and x.stride(1) == 1 and x.shape[1] % 8 == 0 and x.stride(0) % 8 == 0 and w.stride(0) % 8 == 0
+            and x.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0)
+
+
 def gate_token_columns_rows(x, w, table, first, tokens, out, activation="gelu_tanh"):
     """out[t, j] = act(w[j] . x[t]) * table[tokens[t], first + j] in one launch, for a few rows: x float32 [n, width], read as a product
-    reads rows (rounded to bfloat16 where w is bfloat16); w [dim, width]; out [n, dim] of w's dtype."""
+    reads rows (rounded to bfloat16 where w is bfloat16), or already so rounded (`gate_token_columns_rows_takes` says where that is
+    served); w [dim, width]; out [n, dim] of w's dtype."""
     _dev(x, w, table, tokens, out)
     n, width = x.shape
     dim = w.shape[0]
-    _f32_rows(x, "gate_token_columns_rows: x")
+    if x.dtype == torch.bfloat16:
+        if not gate_token_columns_rows_takes(x, w):
+            raise KernelError("gate_token_columns_rows: rows in bfloat16 need bfloat16 weights, a width that is a multiple of 8 and rows that start at multiples of 16 bytes")
+    else:
+        _f32_rows(x, "gate_token_columns_rows: x")
     if activation not in ACTIVATIONS:
         raise KernelError(f"gate_token_columns_rows: unknown activation {activation!r}; known: {', '.join(ACTIVATIONS)}")
     if not (w.shape == (dim, width) and w.stride(1) == 1 and table.dim() == 2 and table.stride(1) == 1 and 0 <= first and first + dim <= table.shape[1]
             and out.shape == (n, dim) and out.stride(1) == 1 and w.dtype == table.dtype == out.dtype):
         raise KernelError("gate_token_columns_rows: w [dim, width], a table that holds the columns asked for and out [n, dim], all of one dtype, are needed")
     _i32(tokens, "gate_token_columns_rows: tokens", n)
-    _call("gi_gate_token_columns_rows", x.data_ptr(), x.stride(0), w.data_ptr(), _code(w, "gate_token_columns_rows: w"), w.stride(0), width, table.data_ptr(),
+    _call("gi_gate_token_columns_rows", x.data_ptr(), _code(x, "gate_token_columns_rows: x"), x.stride(0), w.data_ptr(), _code(w, "gate_token_columns_rows: w"), w.stride(0), width, table.data_ptr(),
           _code(table, "gate_token_columns_rows: table"), table.stride(0), int(first), tokens.data_ptr(), out.data_ptr(), _code(out, "gate_token_columns_rows: out"),
           out.stride(0), n, dim, ACTIVATIONS[activation], 1 if w.dtype == torch.bfloat16 else 0, _stream())
     return out

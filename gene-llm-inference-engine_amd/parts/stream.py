@@ -54,6 +54,9 @@ class TokenSideInput(StreamPart):
         then, reads = reader if reader is not None else (None, None)
         if getattr(then, "is_identity", False) and hasattr(self.norm, "add_onto_and_store"):
             return self.norm.add_onto_and_store(y, x, then, getattr(reads, "in_dtype", ctx.dtype))
+        if (getattr(reads, "takes_ready_rows", False) and reads.in_dtype == torch.bfloat16 and type(then) is type(self.norm) and hasattr(self.norm, "add_onto_then")
+                and then.weight.dtype == self.norm.weight.dtype):          # (the model's last norm and its head, in bfloat16: float32 keeps one order of sums whatever is wanted)
+            return self.norm.add_onto_then(y, x, then, reads.in_dtype)
         self.norm.add_onto(y, x)
         return None
 
@@ -61,7 +64,8 @@ class TokenSideInput(StreamPart):
         s, T, dev = self.spec, ctx.n_rows, ctx.device
         if (T <= self.FEW_ROWS and self.in_dtype == torch.bfloat16 and self.w_gate.dtype == self.table.dtype == self.mid_dtype == torch.bfloat16):
             g = torch.empty((T, s.dim), dtype=torch.bfloat16, device=dev)
-            ops.gate_token_columns_rows(x, self.w_gate, self.table, s.first_column, ctx.tokens, g, s.activation)
+            rows = handed.materialize() if handed is not None and handed.norm is self.rows else x
+            ops.gate_token_columns_rows(rows if ops.gate_token_columns_rows_takes(rows, self.w_gate) else x, self.w_gate, self.table, s.first_column, ctx.tokens, g, s.activation)
             y = torch.empty((T, s.hidden_size), dtype=torch.float32, device=dev)
             linear(g, self.w_out, y)
             return self._join(y, x, ctx, next_reader)

@@ -216,12 +216,13 @@ def test_the_start_of_the_stream_and_a_sublayer_s_output_normed_and_added(dim, d
     assert relative_error(x, x0.double() + P.rms_norm(sub.double(), w.double(), 1e-4)) < 1e-6 and torch.equal(low, x.to(torch.bfloat16))
 
 
+@pytest.mark.parametrize("d", [24, 16, 32, 64, 128, 256])
 @pytest.mark.parametrize("every", [1, 2.5, 3, 64, 1000])
-def test_queries_that_grow_and_keys_that_serve_as_values(every):
-    """The kernel that norms and stores: queries at the positions around every step of their growth, keys normed, and the page's values
-    the keys before their norm."""
+def test_queries_that_grow_and_keys_that_serve_as_values(every, d):
+    """The kernels that norm and store (the one for heads of any size, the one for powers of two): queries at the positions around every
+    step of their growth, keys normed, and the page's values the keys before their norm."""
     from geneinfer_amd.kernels import ops
-    H, G, d, page, eps, coef = 4, 2, 24, 8, 1e-4, 0.8
+    H, G, page, eps, coef = 6, 3, 8, 1e-4, 0.8
     g = torch.Generator().manual_seed(int(every * 10))
     edges = sorted({max(0, int(n * every) + o) for n in (0, 1, 2, 3, 7) for o in (-2, -1, 0, 1)})
     T = len(edges)
@@ -243,6 +244,59 @@ def test_queries_that_grow_and_keys_that_serve_as_values(every):
         mine = cache[p // page].cpu().double()
         keys, values = mine[:G * page * d].reshape(G, page, d)[:, p % page], mine[G * page * d:].reshape(G, d, page)[:, :, p % page]
         assert relative_error(keys, P.rms_norm(kd[t], k_w.double(), eps)) < 2e-6 and torch.equal(values, kd[t])
+
+
+@pytest.mark.parametrize("H, G, d, page, T", [(4, 4, 16, 16, 5), (5, 1, 64, 16, 37), (32, 8, 64, 16, 70), (3, 3, 128, 32, 9), (2, 1, 256, 8, 3), (7, 7, 32, 5, 1)])
+def test_heads_normed_and_stored_without_a_rotation(H, G, d, page, T):
+    """Rows of two requests in bfloat16, values of their own with a weight on them, pages in falling order: against the plain statement, and
+    against the same kernel's general form (which a rotation by no angle makes it take)."""
+    from geneinfer_amd.kernels import ops
+    g = torch.Generator().manual_seed(H * d + T)
+    proj = torch.randn(T, (H + 2 * G) * d + 16, generator=g)
+    q_w, k_w = (1 + 0.2 * torch.randn(d, generator=g)).to(torch.bfloat16), (1 + 0.2 * torch.randn(d, generator=g)).to(torch.bfloat16)
+    slots = [i % 2 for i in range(T)]
+    where = [3 + i // 2 * 2 for i in range(T)]
+    pages = max(where) // page + 1
+    table = torch.arange(2 * pages - 1, -1, -1, dtype=torch.int32, device=DEV).reshape(2, pages).contiguous()
+    pd = proj.to(DEV)
+    q, k, v = pd[:, :H * d], pd[:, H * d:(H + G) * d], pd[:, (H + G) * d:(H + 2 * G) * d]
+    made = []
+    for cos, sin in ((None, None), (torch.ones(T, 2, device=DEV), torch.zeros(T, 2, device=DEV))):
+        cache, out = torch.zeros(2 * pages, G * page * 2 * d, dtype=torch.bfloat16, device=DEV), torch.empty(T, H * d, dtype=torch.bfloat16, device=DEV)
+        ops.norm_rope_store(q, k, v, q_w.to(DEV), k_w.to(DEV), 1e-5, cos, sin, 4 if cos is not None else 0, _ints(where), _ints(slots), table, out, cache, page, H, G, d, d,
+                            v_scale=0.7, query_growth=(0.5, 4))
+        made.append((out, cache))
+    grow = torch.tensor([P.query_growth(p, 0.5, 4) for p in where], dtype=F64)[:, None, None]
+    want = P.rms_norm(proj.double()[:, :H * d].reshape(T, H, d), q_w.double(), 1e-5) * grow
+    assert relative_error(made[0][0], want.reshape(T, H * d)) < 5e-3
+    assert relative_error(made[0][0], made[1][0]) < 5e-3 and relative_error(made[0][1], made[1][1]) < 5e-3
+    for t in (0, T - 1):
+        mine = made[0][1][int(table[slots[t], where[t] // page])].cpu().double()
+        keys, values = mine[:G * page * d].reshape(G, page, d)[:, where[t] % page], mine[G * page * d:].reshape(G, d, page)[:, :, where[t] % page]
+        assert relative_error(keys, P.rms_norm(proj.double()[t, H * d:(H + G) * d].reshape(G, d), k_w.double(), 1e-5)) < 5e-3
+        assert relative_error(values, 0.7 * proj.double()[t, (H + G) * d:(H + 2 * G) * d].reshape(G, d)) < 5e-3
+
+
+@pytest.mark.parametrize("rows, width, dim", [(1, 64, 10), (8, 2048, 256), (9, 128, 7), (16, 2056, 33), (3, 4096, 1)])
+@pytest.mark.parametrize("activation", ["gelu_tanh", "silu"])
+def test_the_gated_columns_of_a_few_rows(rows, width, dim, activation):
+    """Rounding, product, activation and the token's columns in one kernel, from 32-bit rows and from rows already rounded: the same bits."""
+    from geneinfer_amd.kernels import ops
+    g = torch.Generator().manual_seed(rows + width)
+    x, w = torch.randn(rows, width, generator=g), (torch.randn(dim, width, generator=g) * width ** -0.5).to(torch.bfloat16)
+    table, tokens = torch.randn(20, dim + 5, generator=g).to(torch.bfloat16), torch.randint(0, 20, (rows,), generator=g)
+    act = {"gelu_tanh": P.gelu_tanh, "silu": P.silu}[activation]
+    want = act(x.to(torch.bfloat16).double() @ w.double().T) * table.double()[tokens][:, 3:3 + dim]
+    outs = []
+    for rows_in in (x, x.to(torch.bfloat16)):
+        out = torch.empty(rows, dim, dtype=torch.bfloat16, device=DEV)
+        ops.gate_token_columns_rows(rows_in.to(DEV), w.to(DEV), table.to(DEV), 3, tokens.to(torch.int32).to(DEV), out, activation)
+        assert relative_error(out, want) < 5e-3
+        outs.append(out)
+    assert torch.equal(outs[0], outs[1])
+    odd = torch.randn(rows, width + 1, generator=g).to(torch.bfloat16).to(DEV)[:, 1:]
+    with pytest.raises(ops.KernelError):
+        ops.gate_token_columns_rows(odd, w.to(DEV), table.to(DEV), 3, tokens.to(torch.int32).to(DEV), outs[0], activation)
 
 
 def _pages(keys, values, page, hd, dtype, g):
