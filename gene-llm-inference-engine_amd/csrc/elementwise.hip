@@ -909,17 +909,27 @@ __global__ __launch_bounds__(256) void gate_token_columns_rows_kernel(const floa
 // The same for rows that allow loads of 16 bytes, x in bfloat16 or rounded to it on the way: a workgroup makes two outputs of up to eight rows,
 // so that a weight is read once for all of them; a thread takes eight neighbouring columns of everything at once, and the sixteen sums are
 // added over the lanes by halves (a lane keeps eight of them, then four, two, one) and over the four waves through LDS.
-__device__ __forceinline__ void load8(const bf16_t* p, float* v) {
-    const uint4 raw = *reinterpret_cast<const uint4*>(p);
-    v[0] = __uint_as_float(raw.x << 16), v[1] = __uint_as_float(raw.x & 0xffff0000u), v[2] = __uint_as_float(raw.y << 16), v[3] = __uint_as_float(raw.y & 0xffff0000u);
-    v[4] = __uint_as_float(raw.z << 16), v[5] = __uint_as_float(raw.z & 0xffff0000u), v[6] = __uint_as_float(raw.w << 16), v[7] = __uint_as_float(raw.w & 0xffff0000u);
-}
-__device__ __forceinline__ void load8(const float* p, float* v) {
-    const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
-    const float raw[8] = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
+template <typename T>
+struct Eight;                                                     // eight neighbouring numbers as they were loaded
+template <>
+struct Eight<bf16_t> {
+    uint4 raw;
+    __device__ __forceinline__ void load(const bf16_t* p) { raw = *reinterpret_cast<const uint4*>(p); }
+    __device__ __forceinline__ void rounded(float* v) const {
+        v[0] = __uint_as_float(raw.x << 16), v[1] = __uint_as_float(raw.x & 0xffff0000u), v[2] = __uint_as_float(raw.y << 16), v[3] = __uint_as_float(raw.y & 0xffff0000u);
+        v[4] = __uint_as_float(raw.z << 16), v[5] = __uint_as_float(raw.z & 0xffff0000u), v[6] = __uint_as_float(raw.w << 16), v[7] = __uint_as_float(raw.w & 0xffff0000u);
+    }
+};
+template <>
+struct Eight<float> {
+    float4 a, b;
+    __device__ __forceinline__ void load(const float* p) { a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4); }
+    __device__ __forceinline__ void rounded(float* v) const {
+        const float raw[8] = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
 #pragma unroll
-    for (int i = 0; i < 8; ++i) v[i] = bf16_to_f32(f32_to_bf16(raw[i]));
-}
+        for (int i = 0; i < 8; ++i) v[i] = bf16_to_f32(f32_to_bf16(raw[i]));
+    }
+};
 
 template <typename TX>
 __global__ __launch_bounds__(256) void gate_token_columns_few_kernel(const TX* __restrict__ x, long ldx, const bf16_t* __restrict__ w, long ldw, int width,
@@ -928,24 +938,43 @@ __global__ __launch_bounds__(256) void gate_token_columns_few_kernel(const TX* _
     constexpr int RB = 8, JB = 2;                                 // rows and outputs of a workgroup
     __shared__ float part[4][RB * JB];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, j0 = blockIdx.x * JB, t0 = blockIdx.y * RB;
-    // the sum this thread finishes at the end, if it is one of the first sixteen, and its number of the token's row, asked for first (two
-    // loads that depend on each other)
+    // the sum this thread finishes at the end, if it is one of the first sixteen; the number of the token's row that it needs then takes two
+    // loads that depend on each other: the token's number is asked for ahead of the first columns, the table's number behind them
     const int e = threadIdx.x % (RB * JB), t = t0 + e / JB, j = j0 + e % JB;
-    const float column = load_f32(table + (size_t)tokens[min(t, n_rows - 1)] * ldt + first, min(j, dim - 1));
+    const int token = tokens[min(t, n_rows - 1)];
+    Eight<TX> xv[2][RB];
+    Eight<bf16_t> wv[2][JB];
+    auto ask = [&](int b, int d) {                                // (columns behind the last are asked for as the last and weigh nothing)
+        const int dc = min(d, width - 8);
+#pragma unroll
+        for (int j = 0; j < JB; ++j) wv[b][j].load(w + (size_t)min(j0 + j, dim - 1) * ldw + dc);
+#pragma unroll
+        for (int t = 0; t < RB; ++t) xv[b][t].load(x + (size_t)min(t0 + t, n_rows - 1) * ldx + dc);
+    };
     float sum[RB * JB] = {};
-#pragma unroll 2
-    for (int d = threadIdx.x * 8; d < width; d += 2048) {
-        float wv[JB][8], xv[RB][8];
+    auto take = [&](int b, int d) {
+        if (d >= width) return;
+        float wf[JB][8];
 #pragma unroll
-        for (int j = 0; j < JB; ++j) load8(w + (size_t)min(j0 + j, dim - 1) * ldw + d, wv[j]);
+        for (int j = 0; j < JB; ++j) wv[b][j].rounded(wf[j]);
 #pragma unroll
-        for (int t = 0; t < RB; ++t) load8(x + (size_t)min(t0 + t, n_rows - 1) * ldx + d, xv[t]);
-#pragma unroll
-        for (int t = 0; t < RB; ++t)
+        for (int t = 0; t < RB; ++t) {
+            float xf[8];
+            xv[b][t].rounded(xf);
 #pragma unroll
             for (int j = 0; j < JB; ++j)
 #pragma unroll
-                for (int i = 0; i < 8; ++i) sum[t * JB + j] = fmaf(xv[t][i], wv[j][i], sum[t * JB + j]);
+                for (int i = 0; i < 8; ++i) sum[t * JB + j] = fmaf(xf[i], wf[j][i], sum[t * JB + j]);
+        }
+    };
+    int d = threadIdx.x * 8;
+    ask(0, d);
+    const float column = load_f32(table + (size_t)token * ldt + first, min(j, dim - 1));
+    for (int d0 = 0; d0 < width; d0 += 4096, d += 4096) {         // (every thread as often: no load is skipped)
+        ask(1, d + 2048);
+        take(0, d);
+        if (d0 + 4096 < width) ask(0, d + 4096);
+        take(1, d + 2048);
     }
 #pragma unroll
     for (int half = 8, off = 32; half >= 1; half >>= 1, off >>= 1) {
