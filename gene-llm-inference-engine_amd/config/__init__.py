@@ -1,7 +1,7 @@
 """Typed configurations, the architecture registry and the neutral model description."""
-from .spec import (AttentionSpec, DenseMlpSpec, GatedDeltaSpec, InterleavedRotarySpec, LatentAttentionSpec, LayerSpec, LearnedPositionsSpec, LightningSpec, MlstmSpec,
+from .spec import (AddRowsSpec, AttentionSpec, DenseMlpSpec, GatedDeltaSpec, InterleavedRotarySpec, LatentAttentionSpec, LayerNormSpec, LayerSpec, LearnedPositionsSpec, LightningSpec, MlstmSpec,
                    ModelSpec, NoNormSpec, PartialRotarySpec, RejoinSpec, RmsNormSpec, RotarySpec, RoutedExpertsSpec, RunEntry, ScaleSpec, SelectiveScanSpec, SideBySideSpec, SoftCapSpec,
-                   StreamAccessSpec, SwiGluSpec, TokenShiftSpec, TokenSideInputSpec)
+                   StreamAccessSpec, SwiGluSpec, TokenPairSpec, TokenShiftSpec, TokenSideInputSpec)
 from .errors import ConfigError
 from .registry import (config_class_for, parse_config, read_config, register_architecture,
                        registered_architectures)
@@ -11,3 +11,4 @@ from .rigalorn import RigalornConfig                   # registers itself
 from .zidevik import ZidevikConfig                     # registers itself
 from .mimitar import MimitarConfig                     # registers itself
 from .vubenex import VubenexConfig                     # registers itself
+from .puzorax import PuzoraxConfig                     # registers itself

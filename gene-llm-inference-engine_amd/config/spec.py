@@ -81,6 +81,16 @@ class RmsNormSpec:
 
 
 @dataclass(frozen=True)
+class LayerNormSpec:
+    """(x - mean) / sqrt(variance + eps) * weight + bias, with the variance the mean of the squared deviations."""
+    kind: ClassVar[str] = "layernorm"
+    size: int
+    eps: float
+    weight: str                      # tensor names
+    bias: str
+
+
+@dataclass(frozen=True)
 class NoNormSpec:
     """No norm: the rows as they are, for an arrangement that has a place for a norm where an architecture has none."""
     kind: ClassVar[str] = "none"
@@ -139,7 +149,8 @@ class LatentAttentionSpec:
     """Attention whose queries and keys/values pass through low-rank latents.  c_q = norm(W_dq x), q = W_uq c_q, per head
     [head_dim unrotated | rotary_dim rotated]; W_dkv x = [kv_rank | rotary_dim]: the first part, normed, is the latent c, the
     second one rotated key part for all heads; per head the unrotated key is W_uk c and the value W_uv c, so that only c and
-    the rotated part are cached.  score = (q_plain . k_plain + q_rot . k_rot) * scale; causal, optionally windowed."""
+    the rotated part are cached.  score = (q_plain . k_plain + q_rot . k_rot) * scale; causal, optionally windowed.
+    With `q_proj` the queries have no latent: q = W_q x (q_rank is then 0, and the three names of the query latent are empty)."""
     kind: ClassVar[str] = "latent_attention"
     hidden_size: int
     n_heads: int
@@ -158,9 +169,12 @@ class LatentAttentionSpec:
     uk_proj: str
     uv_proj: str
     o_proj: str
-    position: Optional[Any] = None   # a spec that gives cosines and sines for rotary_dim / 2 neighbouring pairs
+    position: Optional[Any] = None   # a spec that gives cosines and sines for rotary_dim / 2 pairs: neighbouring ones, or (i, i + rotary_dim/2)
     window: Optional[int] = None
     head_gate: Optional[str] = None  # tensor [heads, hidden]: head h's output is multiplied by sigmoid(row h of it . the mixer's input)
+    q_proj: Optional[str] = None     # tensor [heads*(head_dim + rotary_dim), hidden]: queries straight from the mixer's input
+    sinks: Optional[str] = None      # tensor [heads]: a learned score per head that joins the softmax's denominator and has no value
+    output_gate: Optional[str] = None    # tensor [heads*value_dim, hidden]: the heads' outputs times sigmoid(it . the mixer's input), channel by channel
 
 
 @dataclass(frozen=True)
@@ -211,7 +225,10 @@ class GatedDeltaSpec:
     the memory uses q/k head h // (n_heads / n_kv_heads)) and v pass a causal convolution of `conv_taps` taps per channel
     (tensors [channels, taps], the last tap the token's own) and SiLU; q and k are then divided by sqrt(sum of squares + 1e-6),
     q also by sqrt(key_dim).  Every head's y is divided by its root mean square (`norm_eps`), multiplied by `out_norm`
-    [value_dim], one for all heads, and by SiLU(gate(x)), and goes through `o_proj`."""
+    [value_dim], one for all heads, and by SiLU(gate(x)) (or `gate_activation` of it), and goes through `o_proj`.
+    With `channel_decay` every head and key channel has a decay of its own, which acts on the memory's row of that channel: a(x)
+    and dt_bias then have heads*key_dim numbers (a_log stays one per head).  a(x) and gate(x) may each pass a narrow middle:
+    a(x) = a_proj (a_down x) with a_down [a_rank, hidden], gate(x) = gate_proj (gate_down x) with gate_down [gate_rank, hidden]."""
     kind: ClassVar[str] = "gated_delta"
     hidden_size: int
     n_heads: int
@@ -233,6 +250,12 @@ class GatedDeltaSpec:
     gate_proj: str
     out_norm: str
     o_proj: str
+    channel_decay: bool = False
+    a_down: Optional[str] = None
+    a_rank: int = 0
+    gate_down: Optional[str] = None
+    gate_rank: int = 0
+    gate_activation: str = "silu"    # or "sigmoid"
 
 
 @dataclass(frozen=True)
@@ -309,7 +332,10 @@ class RoutedExpertsSpec:
     activations of `SwiGluSpec`, `activation_limit` with them).  `shared`, a feed-forward spec of any kind, serves every row and is
     added; with `shared_gate` [1, hidden] it is multiplied by sigmoid(shared_gate . h) first, one number a row.  With `n_groups` > 1 the
     experts form that many equal groups of neighbours, a group scores what its best expert scores, and only experts of the
-    `groups_kept` best groups can be chosen.  `renormalize_floor` is added to the sum the chosen scores are divided by."""
+    `groups_kept` best groups can be chosen.  `renormalize_floor` is added to the sum the chosen scores are divided by.
+    `correction` [experts + n_identity] is added to the scores for the choice; the weights come from the scores without it.  The
+    weights are multiplied by `weight_scale` at the end.  With `n_identity` > 0 the router (and the correction) has that many outputs
+    behind the experts'; one that is chosen stands for an expert that returns its input (no tensors)."""
     kind: ClassVar[str] = "routed_experts"
     hidden_size: int
     intermediate_size: int
@@ -329,12 +355,17 @@ class RoutedExpertsSpec:
     n_groups: int = 1
     groups_kept: int = 1
     renormalize_floor: float = 0.0
+    correction: Optional[str] = None
+    n_identity: int = 0
+    weight_scale: float = 1.0
 
     def __post_init__(self):
-        if not (len(self.gate_projs) == len(self.up_projs) == len(self.down_projs) == self.n_experts) or not 1 <= self.top <= self.n_experts:
+        if not (len(self.gate_projs) == len(self.up_projs) == len(self.down_projs) == self.n_experts) or not 1 <= self.top <= self.n_experts + self.n_identity:
             raise ValueError("routed experts: three matrices per expert, and 1 <= top <= experts")
+        if self.n_identity < 0 or (self.n_groups > 1 and (self.n_identity or self.correction is not None)):
+            raise ValueError("routed experts: experts in groups go without a correction and without experts that return their input")
         if (self.n_groups < 1 or self.n_experts % self.n_groups or not 1 <= self.groups_kept <= self.n_groups
-                or self.top > self.groups_kept * (self.n_experts // self.n_groups)):
+                or (self.n_groups > 1 and self.top > self.groups_kept * (self.n_experts // self.n_groups))):
             raise ValueError("routed experts: equal groups, of which 1 .. all are kept, with at least `top` experts in the kept ones")
         if self.shared_gate is not None and self.shared is None:
             raise ValueError("routed experts: a gate on the shared feed-forward needs a shared feed-forward")
@@ -370,6 +401,18 @@ class RejoinSpec:
     offsets: Optional[str] = None
     offsets_rows: int = 0
     row: int = 0
+
+
+@dataclass(frozen=True)
+class AddRowsSpec:
+    """Something added to the residual stream: row `row` of `offsets` [offsets_rows, hidden], and before it, with `token_rows`, the
+    token rows as the first layer got them."""
+    kind: ClassVar[str] = "add_rows"
+    hidden_size: int
+    offsets: str
+    offsets_rows: int
+    row: int
+    token_rows: bool = False
 
 
 @dataclass(frozen=True)
@@ -414,6 +457,19 @@ class LearnedPositionsSpec:
     kind: ClassVar[str] = "learned_positions"
     hidden_size: int
     positions: int
+    table: str
+
+
+@dataclass(frozen=True)
+class TokenPairSpec:
+    """A row of a second table added to the token's row (behind the token table): the row of the pair (the token before, the token),
+    number (before * mul_before + token * mul_token) mod `buckets` of `table` [buckets + 1, hidden]; a sequence's first token, which
+    has none before it, takes the last row.  A request's last token is kept beside its cache."""
+    kind: ClassVar[str] = "token_pairs"
+    hidden_size: int
+    buckets: int
+    mul_before: int
+    mul_token: int
     table: str
 
 

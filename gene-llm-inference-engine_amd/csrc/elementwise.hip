@@ -1110,3 +1110,170 @@ GI_API int gi_rmsnorm_add_store(const float* y, const void* w, int w_dtype, floa
     GI_CHECK_LAUNCH("rmsnorm_add_store");
     return 0;
 }
+
+// ------------------------------------------------- layer norm, and what may be added to a row before it
+// v = x[t] + add[t] + vec (either may be absent; with one of them the row is written back to x), then
+// out[t] = (v - mean(v)) / sqrt(mean((v - mean)^2) + eps) * w + b (w absent: no norm, the row is only added to).
+// One workgroup per row.  The sums are taken in 32-bit in an order that the row's length alone fixes: thread c % 256 takes the groups
+// of four neighbours c, c + 256, ... (single numbers where a row is not of whole groups), then the lanes, then the waves.
+template <typename TW, typename TO>
+__global__ __launch_bounds__(256) void layernorm_kernel(float* __restrict__ x, const int* __restrict__ rows, const float* __restrict__ add, const TW* __restrict__ vec,
+                                                       const TW* __restrict__ w, const TW* __restrict__ b, TO* __restrict__ out, int dim, float eps, size_t x_stride,
+                                                       size_t add_stride, size_t out_stride) {
+    __shared__ float red[4];
+    const size_t t = rows ? rows[blockIdx.x] : blockIdx.x;
+    float* xr = x + t * x_stride;
+    const bool joins = add != nullptr || vec != nullptr;
+    float sum = 0.f;
+    for (int d = threadIdx.x; d < dim; d += 256) {
+        float v = xr[d];
+        if (add) v += add[t * add_stride + d];
+        if (vec) v += load_f32(vec, d);
+        if (joins) xr[d] = v;
+        sum += v;
+    }
+    if (w == nullptr) return;                            // (the same for the whole workgroup)
+    const float mean = block_sum<256>(sum, red) / (float)dim;
+    float ss = 0.f;
+    for (int d = threadIdx.x; d < dim; d += 256) ss = fmaf(xr[d] - mean, xr[d] - mean, ss);      // (a thread reads back what it wrote itself)
+    const float r = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)dim + eps);
+    for (int d = threadIdx.x; d < dim; d += 256) store_f32(out, (size_t)blockIdx.x * out_stride + d, fmaf((xr[d] - mean) * r, load_f32(w, d), load_f32(b, d)));
+}
+
+// The same for aligned rows of whole groups of four, with the row in registers: PER groups a thread, all loads asked for at once.
+template <int PER, typename TW, typename TO>
+__global__ __launch_bounds__(256) void layernorm_rows_kernel(float* __restrict__ x, const int* __restrict__ rows, const float* __restrict__ add, const TW* __restrict__ vec,
+                                                            const TW* __restrict__ w, const TW* __restrict__ b, TO* __restrict__ out, int dim, float eps, size_t x_stride,
+                                                            size_t add_stride, size_t out_stride) {
+    __shared__ float red[4];
+    const size_t t = rows ? rows[blockIdx.x] : blockIdx.x;
+    float* xr = x + t * x_stride;
+    const bool joins = add != nullptr || vec != nullptr;
+    const int n4 = dim / 4;
+    float4 v[PER], wv[PER], bv[PER];
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        const int c = min((int)threadIdx.x + 256 * i, n4 - 1);
+        v[i] = load4(xr + 4 * c);
+        if (w) wv[i] = load4(w + 4 * c), bv[i] = load4(b + 4 * c);
+    }
+    if (add) {
+#pragma unroll
+        for (int i = 0; i < PER; ++i) {
+            const float4 a = load4(add + t * add_stride + 4 * min((int)threadIdx.x + 256 * i, n4 - 1));
+            v[i].x += a.x; v[i].y += a.y; v[i].z += a.z; v[i].w += a.w;
+        }
+    }
+    if (vec) {
+#pragma unroll
+        for (int i = 0; i < PER; ++i) {
+            const float4 a = load4(vec + 4 * min((int)threadIdx.x + 256 * i, n4 - 1));
+            v[i].x += a.x; v[i].y += a.y; v[i].z += a.z; v[i].w += a.w;
+        }
+    }
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        const int c = threadIdx.x + 256 * i;
+        if (c < n4) {
+            if (joins) store4(xr + 4 * c, v[i].x, v[i].y, v[i].z, v[i].w);
+            sum += (v[i].x + v[i].y) + (v[i].z + v[i].w);
+        }
+    }
+    if (w == nullptr) return;
+    const float mean = block_sum<256>(sum, red) / (float)dim;
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        v[i].x -= mean; v[i].y -= mean; v[i].z -= mean; v[i].w -= mean;
+        if ((int)threadIdx.x + 256 * i < n4) ss += (v[i].x * v[i].x + v[i].y * v[i].y) + (v[i].z * v[i].z + v[i].w * v[i].w);
+    }
+    const float r = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)dim + eps);
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        const int c = threadIdx.x + 256 * i;
+        if (c < n4) store4(out + (size_t)blockIdx.x * out_stride + 4 * c, fmaf(v[i].x * r, wv[i].x, bv[i].x), fmaf(v[i].y * r, wv[i].y, bv[i].y), fmaf(v[i].z * r, wv[i].z, bv[i].z),
+                           fmaf(v[i].w * r, wv[i].w, bv[i].w));
+    }
+}
+
+// rows: out[i] = norm of x[rows[i]] (add and vec must then be absent).  out_dtype says how the normed rows are stored; w and b nullptr: no norm.
+GI_API int gi_layernorm(float* x, const int* rows, const float* add, const void* vec, const void* w, const void* b, int w_dtype, void* out, int out_dtype, int n_rows, int dim,
+                        float eps, long x_stride, long add_stride, long out_stride, hipStream_t stream) {
+    GI_REQUIRE(n_rows > 0 && dim > 0 && x_stride >= dim && (add == nullptr || add_stride >= dim), "layernorm: bad sizes (rows %d, dim %d)", n_rows, dim);
+    GI_REQUIRE((w == nullptr) == (b == nullptr) && (w == nullptr || (out != nullptr && out_stride >= dim)) && (w != nullptr || add != nullptr || vec != nullptr),
+               "layernorm: weights come with biases and with room for the normed rows");
+    GI_REQUIRE(rows == nullptr || (add == nullptr && vec == nullptr), "layernorm: nothing can be added to a selection of rows");
+    const bool fast = dim % 4 == 0 && dim <= 8192 && x_stride % 4 == 0 && out_stride % 4 == 0 && add_stride % 4 == 0 && (((uintptr_t)x | (uintptr_t)add | (uintptr_t)vec |
+                      (uintptr_t)w | (uintptr_t)b | (uintptr_t)out) & 15) == 0;
+#define ARGS(TW, TO) x, rows, add, (const TW*)vec, (const TW*)w, (const TW*)b, (TO*)out, dim, eps, (size_t)x_stride, (size_t)add_stride, (size_t)out_stride
+#define LAUNCH(TW, TO)                                                                                                \
+    do {                                                                                                              \
+        if (fast && dim <= 1024) layernorm_rows_kernel<1, TW, TO><<<n_rows, 256, 0, stream>>>(ARGS(TW, TO));          \
+        else if (fast && dim <= 2048) layernorm_rows_kernel<2, TW, TO><<<n_rows, 256, 0, stream>>>(ARGS(TW, TO));     \
+        else if (fast && dim <= 4096) layernorm_rows_kernel<4, TW, TO><<<n_rows, 256, 0, stream>>>(ARGS(TW, TO));     \
+        else if (fast) layernorm_rows_kernel<8, TW, TO><<<n_rows, 256, 0, stream>>>(ARGS(TW, TO));                    \
+        else layernorm_kernel<TW, TO><<<n_rows, 256, 0, stream>>>(ARGS(TW, TO));                                      \
+    } while (0)
+    if (w_dtype == GI_F32 && out_dtype == GI_F32) LAUNCH(float, float);
+    else if (w_dtype == GI_F32 && out_dtype == GI_BF16) LAUNCH(float, bf16_t);
+    else if (w_dtype == GI_BF16 && out_dtype == GI_F32) LAUNCH(bf16_t, float);
+    else if (w_dtype == GI_BF16 && out_dtype == GI_BF16) LAUNCH(bf16_t, bf16_t);
+    else return gi_fail("layernorm: unknown dtypes %d, %d", w_dtype, out_dtype);
+#undef LAUNCH
+#undef ARGS
+    GI_CHECK_LAUNCH("layernorm");
+    return 0;
+}
+
+// ------------------------------------------------- the row of a pair of tokens added to the token's row
+// x[t] = table[token] + pairs[(before * mul_before + token * mul_token) mod buckets], with `before` the token of the request's row
+// before: the step's previous row, or, for a request's first row of the step, what `last` [slots] holds from the step before; at
+// position 0 there is none, and the row is pairs[buckets].  The workgroup of a request's first row of the step also leaves the
+// request's last token of the step in `last`, behind its own reading of it (no other workgroup touches that slot; rows that share the spare
+// slot all stand at position 0 and read nothing).  keep: the same rows once more, for a reader behind the layers (nullptr: none).
+template <typename TT>
+__global__ __launch_bounds__(256) void embed_pairs_kernel(const TT* __restrict__ table, const TT* __restrict__ pairs, const int* __restrict__ tokens, const int* __restrict__ pos,
+                                                         const int* __restrict__ slot, const int* __restrict__ seg_start, const int* __restrict__ seg_len, int n_segs, int n_rows,
+                                                         int* __restrict__ last, long last_stride, unsigned buckets, unsigned mul_before, unsigned mul_token,
+                                                         float* __restrict__ x, float* __restrict__ keep, int dim) {
+    __shared__ int end;                                  // the last row of the request whose first row this is
+    const int t = blockIdx.x, tid = threadIdx.x, p = pos[t], s = slot[t], token = tokens[t];
+    const bool first = t == 0 || slot[t - 1] != s || pos[t - 1] + 1 != p;
+    unsigned long long row = buckets;
+    if (p > 0) {
+        const unsigned long long before = (unsigned)(first ? last[(size_t)s * last_stride] : tokens[t - 1]);
+        row = (before * mul_before + (unsigned long long)(unsigned)token * mul_token) % buckets;
+    }
+    if (first) {                                         // (the same for the whole workgroup)
+        if (tid == 0) end = t;
+        __syncthreads();                                 // every thread has read the slot
+        for (int i = tid; i < n_segs; i += 256)
+            if (seg_start[i] == t && seg_len[i] > 0) end = min(t + seg_len[i], n_rows) - 1;
+        __syncthreads();
+        if (tid == 0) last[(size_t)s * last_stride] = tokens[end];
+    }
+    const TT* a = table + (size_t)token * dim;
+    const TT* b = pairs + (size_t)row * dim;
+    for (int d = tid; d < dim; d += 256) {
+        const float v = load_f32(a, d) + load_f32(b, d);
+        x[(size_t)t * dim + d] = v;
+        if (keep) keep[(size_t)t * dim + d] = v;
+    }
+}
+
+// mul_before and mul_token: reduced mod buckets by the caller (the row's number is the same), so that no product overflows 64 bits.
+GI_API int gi_embed_pairs(const void* table, const void* pairs, int dtype, const int* tokens, const int* pos, const int* slot, const int* seg_start, const int* seg_len, int n_segs,
+                          int* last, long last_stride, int buckets, int mul_before, int mul_token, float* x, float* keep, int n_rows, int dim, hipStream_t stream) {
+    GI_REQUIRE(n_rows > 0 && dim > 0 && n_segs > 0 && buckets > 0 && mul_before >= 0 && mul_before < buckets && mul_token >= 0 && mul_token < buckets && last_stride > 0,
+               "embed_pairs: bad sizes (rows %d, dim %d, requests %d, buckets %d, factors %d and %d)", n_rows, dim, n_segs, buckets, mul_before, mul_token);
+    if (dtype == GI_F32)
+        embed_pairs_kernel<float><<<n_rows, 256, 0, stream>>>((const float*)table, (const float*)pairs, tokens, pos, slot, seg_start, seg_len, n_segs, n_rows, last, last_stride,
+                                                              buckets, mul_before, mul_token, x, keep, dim);
+    else if (dtype == GI_BF16)
+        embed_pairs_kernel<bf16_t><<<n_rows, 256, 0, stream>>>((const bf16_t*)table, (const bf16_t*)pairs, tokens, pos, slot, seg_start, seg_len, n_segs, n_rows, last, last_stride,
+                                                               buckets, mul_before, mul_token, x, keep, dim);
+    else return gi_fail("embed_pairs: unknown dtype %d", dtype);
+    GI_CHECK_LAUNCH("embed_pairs");
+    return 0;
+}

@@ -19,7 +19,10 @@
 //   gi_experts_place     every item's place in that order (an expert's items keep their order), and every tile's expert
 //   gi_experts_gather    the rows of the items (times their score, where it weighs the input) at their places, as bfloat16
 //   gi_experts_combine   x[row] (+)= the sum over the row's choices of the results at their places (times the score, where it
-//                        weighs the output), the choices one after the other
+//                        weighs the output), the choices one after the other; and, in the same kernel, the layer norm of the new row
+//                        for whoever reads it next
+// A number from `n_experts` on stands for an expert that returns its input: it has no weights, no item of it takes a place, and the
+// kernels that add the choices up take the row itself for its result.
 // Nothing of this asks the host how the router chose: the launches' shapes depend on the number of items and experts alone.
 #include "common.h"
 
@@ -30,9 +33,12 @@ constexpr int ROUTE_PER_LANE = 16;      // experts a lane looks at: up to 1024 e
 // What the router makes of a row's logits (z: this lane's experts lane, lane + 64, ...; -inf beyond the last): the scores
 // (score_kind 0: sigmoid, 1: softmax over all experts), the `top` largest (the lower index wins a tie), optionally divided by
 // their sum + floor.  With n_groups > 1 the experts form that many equal groups of neighbours, a group scores what its best
-// expert scores, and only experts of the `keep` best groups can be chosen (the lower group wins a tie).
+// expert scores, and only experts of the `keep` best groups can be chosen (the lower group wins a tie).  With `correction`
+// [n_experts] the scores plus it choose (n_groups is then 1), and the weights are the scores without it.  All weights are multiplied
+// by `scale` at the end.
 __device__ __forceinline__ void choose_experts(float (&z)[ROUTE_PER_LANE], int lane, size_t t, int n_experts, int top, int score_kind, int renormalize, float floor,
-                                               int n_groups, int keep, int* __restrict__ ids, float* __restrict__ weights) {
+                                               int n_groups, int keep, const float* __restrict__ correction, float scale, int* __restrict__ ids,
+                                               float* __restrict__ weights) {
     float biggest = -INFINITY;
 #pragma unroll
     for (int i = 0; i < ROUTE_PER_LANE; ++i) biggest = fmaxf(biggest, z[i]);
@@ -73,6 +79,15 @@ __device__ __forceinline__ void choose_experts(float (&z)[ROUTE_PER_LANE], int l
     }
     float total = 0.f, mine = 0.f;
     int my_id = 0;
+    float score_of[ROUTE_PER_LANE];                     // what weighs, where it is not what chooses
+    if (correction != nullptr) {
+#pragma unroll
+        for (int i = 0; i < ROUTE_PER_LANE; ++i) {
+            const int e = lane + 64 * i;
+            score_of[i] = score_kind == 1 ? expf(z[i] - biggest) / denominator : 1.0f / (1.0f + expf(-z[i]));
+            z[i] = e < n_experts ? score_of[i] + correction[e] : -INFINITY;
+        }
+    }
     for (int k = 0; k < top; ++k) {
         float best = -INFINITY;
         int at = 0x7fffffff;
@@ -86,7 +101,15 @@ __device__ __forceinline__ void choose_experts(float (&z)[ROUTE_PER_LANE], int l
             const int oa = __shfl_xor(at, off, 64);
             if (ob > best || (ob == best && oa < at)) best = ob, at = oa;
         }
-        const float score = score_kind == 1 ? expf(best - biggest) / denominator : 1.0f / (1.0f + expf(-best));
+        float score;
+        if (correction != nullptr) {
+            float own = 0.f;
+#pragma unroll
+            for (int i = 0; i < ROUTE_PER_LANE; ++i) own = (at >> 6) == i ? score_of[i] : own;
+            score = __shfl(own, at & 63, 64);
+        } else {
+            score = score_kind == 1 ? expf(best - biggest) / denominator : 1.0f / (1.0f + expf(-best));
+        }
         total += score;
         if (lane == k) mine = score, my_id = at;
 #pragma unroll
@@ -96,13 +119,14 @@ __device__ __forceinline__ void choose_experts(float (&z)[ROUTE_PER_LANE], int l
     }
     if (lane < top) {
         ids[t * top + lane] = my_id;
-        weights[t * top + lane] = renormalize ? mine / (total + floor) : mine;
+        weights[t * top + lane] = (renormalize ? mine / (total + floor) : mine) * scale;
     }
 }
 
 // One wave per row.
 __global__ __launch_bounds__(64) void route_top_kernel(const float* __restrict__ logits, long ld, int n_experts, int top, int score_kind, int renormalize,
-                                                      float floor, int n_groups, int keep, int* __restrict__ ids, float* __restrict__ weights) {
+                                                      float floor, int n_groups, int keep, const float* __restrict__ correction, float scale, int* __restrict__ ids,
+                                                      float* __restrict__ weights) {
     const size_t t = blockIdx.x;
     const int lane = threadIdx.x;
     float z[ROUTE_PER_LANE];
@@ -111,19 +135,20 @@ __global__ __launch_bounds__(64) void route_top_kernel(const float* __restrict__
         const int e = lane + 64 * i;
         z[i] = e < n_experts ? logits[t * ld + e] : -INFINITY;
     }
-    choose_experts(z, lane, t, n_experts, top, score_kind, renormalize, floor, n_groups, keep, ids, weights);
+    choose_experts(z, lane, t, n_experts, top, score_kind, renormalize, floor, n_groups, keep, correction, scale, ids, weights);
 }
 
 // One wave per (row, choice, output j): both dot products over the row, the lanes' shares of k interleaved.
 template <typename TW, typename TA, typename TO>
 __global__ __launch_bounds__(256) void experts_gate_up_kernel(const TA* __restrict__ h, long ldh, const TW* __restrict__ w_gate, const TW* __restrict__ w_up,
                                                              const int* __restrict__ ids, const float* __restrict__ weights, int weigh_input,
-                                                             int top, TO* __restrict__ mid, long ldm, int width, int ff, int act, float limit, int group) {
+                                                             int top, TO* __restrict__ mid, long ldm, int width, int ff, int act, float limit, int group, int n_experts) {
     const size_t item = blockIdx.x;                     // (row * top + choice)
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int j = blockIdx.y * 4 + wave;
     if (j >= ff) return;
     const size_t row = item / top, e = ids[item];
+    if (e >= (size_t)n_experts) return;                  // (an expert that returns its input has nothing here)
     const float s = weigh_input ? weights[item] : 1.0f;
     const TA* a = h + row * ldh;
     // group > 0: one stack [experts][2 ff][width] of `group` gate rows, the `group` up rows of the same outputs, and so on
@@ -141,10 +166,10 @@ __global__ __launch_bounds__(256) void experts_gate_up_kernel(const TA* __restri
     if (lane == 0) store_f32(mid + item * ldm, j, gated_act(sg, su, act, limit));
 }
 
-template <typename TW, typename TM>
+template <typename TW, typename TM, typename TA>
 __global__ __launch_bounds__(256) void experts_down_kernel(const TM* __restrict__ mid, long ldm, const TW* __restrict__ w_down, const int* __restrict__ ids,
                                                           const float* __restrict__ weights, int weigh_output, int top, float* __restrict__ x, long ldx,
-                                                          int width, int ff, int accumulate) {
+                                                          int width, int ff, int accumulate, const TA* __restrict__ h, long ldh, int n_experts) {
     const size_t row = blockIdx.x;
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int c = blockIdx.y * 4 + wave;
@@ -152,6 +177,10 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const TM* __restrict_
     float total = 0.f;
     for (int k = 0; k < top; ++k) {
         const size_t item = row * top + k, e = ids[item];
+        if (e >= (size_t)n_experts) {                    // the input itself (weighed in either form)
+            total += weights[item] * load_f32(h, row * ldh + c);
+            continue;
+        }
         const TM* m = mid + item * ldm;
         const TW* w = w_down + (e * width + c) * (size_t)ff;
         float s = 0.f;
@@ -168,7 +197,8 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const TM* __restrict_
 constexpr int ROUTE_MAX_EXPERTS = 64 * ROUTE_PER_LANE;
 template <typename TA, typename TW>
 __global__ __launch_bounds__(256) void route_rows_kernel(const TA* __restrict__ h, long ldh, const TW* __restrict__ router, long ldr, int width, int n_experts, int top,
-                                                        int score_kind, int renormalize, float floor, int n_groups, int keep, int* __restrict__ ids, float* __restrict__ weights,
+                                                        int score_kind, int renormalize, float floor, int n_groups, int keep, const float* __restrict__ correction, float scale,
+                                                        int* __restrict__ ids, float* __restrict__ weights,
                                                         float* __restrict__ logits_out, long ldl, int n_extra, float* __restrict__ extra_out, long lde) {
     __shared__ float zs[ROUTE_MAX_EXPERTS];
     const size_t t = blockIdx.x;
@@ -205,7 +235,7 @@ __global__ __launch_bounds__(256) void route_rows_kernel(const TA* __restrict__ 
         const int e = lane + 64 * i;
         z[i] = e < n_experts ? zs[e] : -INFINITY;
     }
-    choose_experts(z, lane, t, n_experts, top, score_kind, renormalize, floor, n_groups, keep, ids, weights);
+    choose_experts(z, lane, t, n_experts, top, score_kind, renormalize, floor, n_groups, keep, correction, scale, ids, weights);
 }
 
 constexpr int EXPERT_TILE = 128;          // rows of a tile of the grouped product
@@ -250,9 +280,11 @@ __global__ __launch_bounds__(256) void experts_place_kernel(const int* __restric
 }
 
 // The row of every item at its place, times the item's score where that weighs the input, eight columns a thread.
-__global__ __launch_bounds__(256) void experts_gather_kernel(const bf16_t* __restrict__ h, long ldh, const int* __restrict__ place, const float* __restrict__ weights,
-                                                            int weigh_input, int top, bf16_t* __restrict__ out, long ldo, int width) {
+__global__ __launch_bounds__(256) void experts_gather_kernel(const bf16_t* __restrict__ h, long ldh, const int* __restrict__ ids, const int* __restrict__ place,
+                                                            const float* __restrict__ weights, int weigh_input, int top, bf16_t* __restrict__ out, long ldo, int width,
+                                                            int n_experts) {
     const size_t item = blockIdx.x;
+    if (ids[item] >= n_experts) return;
     const bf16_t* a = h + (item / top) * ldh;
     bf16_t* o = out + (size_t)place[item] * ldo;
     const float s = weigh_input ? weights[item] : 1.0f;
@@ -267,18 +299,86 @@ __global__ __launch_bounds__(256) void experts_gather_kernel(const bf16_t* __res
     }
 }
 
-__global__ __launch_bounds__(256) void experts_combine_kernel(const float* __restrict__ y, long ldy, const int* __restrict__ place, const float* __restrict__ weights,
-                                                             int weigh_output, int top, float* __restrict__ x, long ldx, int width, int accumulate) {
+__global__ __launch_bounds__(256) void experts_combine_kernel(const float* __restrict__ y, long ldy, const int* __restrict__ ids, const int* __restrict__ place,
+                                                             const float* __restrict__ weights, int weigh_output, int top, float* __restrict__ x, long ldx, int width, int accumulate,
+                                                             const bf16_t* __restrict__ h, long ldh, int n_experts) {
     const size_t row = blockIdx.x;
     const int c = blockIdx.y * 256 + threadIdx.x;
     if (c >= width) return;
     float total = 0.f;
     for (int k = 0; k < top; ++k) {
         const size_t item = row * top + k;
+        if (ids[item] >= n_experts) {
+            total += weights[item] * load_f32(h, row * ldh + c);
+            continue;
+        }
         const float v = y[(size_t)place[item] * ldy + c];
         total += weigh_output ? weights[item] * v : v;
     }
     x[row * ldx + c] = accumulate ? x[row * ldx + c] + total : total;
+}
+
+__device__ __forceinline__ float4 four(const float* p) { return *reinterpret_cast<const float4*>(p); }
+__device__ __forceinline__ float4 four(const bf16_t* p) {
+    const uint2 v = *reinterpret_cast<const uint2*>(p);
+    return float4{__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16), __uint_as_float(v.y & 0xffff0000u)};
+}
+
+// The same, a workgroup per row with the row in registers (PER groups of four columns a thread), and then the layer norm of the new row,
+// (v - mean) / sqrt(variance + eps) * w + b, as bfloat16 to `out`: the rows the next part reads.
+template <int PER, typename TW>
+__global__ __launch_bounds__(256) void experts_combine_norm_kernel(const float* __restrict__ y, long ldy, const int* __restrict__ ids, const int* __restrict__ place,
+                                                                  const float* __restrict__ weights, int weigh_output, int top, float* __restrict__ x, long ldx, int width,
+                                                                  int accumulate, const bf16_t* __restrict__ h, long ldh, int n_experts, const TW* __restrict__ w,
+                                                                  const TW* __restrict__ b, float eps, bf16_t* __restrict__ out, long ldo) {
+    __shared__ float red[4];
+    const size_t row = blockIdx.x;
+    const int n4 = width / 4;
+    float4 v[PER], wv[PER], bv[PER];
+    int at[PER];
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        at[i] = 4 * min((int)threadIdx.x + 256 * i, n4 - 1);
+        v[i] = accumulate ? four(x + row * ldx + at[i]) : float4{0.f, 0.f, 0.f, 0.f};
+        wv[i] = four(w + at[i]);
+        bv[i] = four(b + at[i]);
+    }
+    float4 total[PER];
+#pragma unroll
+    for (int i = 0; i < PER; ++i) total[i] = float4{0.f, 0.f, 0.f, 0.f};
+    for (int k = 0; k < top; ++k) {
+        const size_t item = row * top + k;
+        const bool itself = ids[item] >= n_experts;      // (the same for the whole workgroup)
+        const float s = itself || weigh_output ? weights[item] : 1.0f;
+#pragma unroll
+        for (int i = 0; i < PER; ++i) {
+            const float4 r = itself ? four(h + row * ldh + at[i]) : four(y + (size_t)place[item] * ldy + at[i]);
+            total[i].x += s * r.x; total[i].y += s * r.y; total[i].z += s * r.z; total[i].w += s * r.w;
+        }
+    }
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        v[i].x += total[i].x; v[i].y += total[i].y; v[i].z += total[i].z; v[i].w += total[i].w;
+        if ((int)threadIdx.x + 256 * i < n4) {
+            *reinterpret_cast<float4*>(x + row * ldx + at[i]) = v[i];
+            sum += (v[i].x + v[i].y) + (v[i].z + v[i].w);
+        }
+    }
+    const float mean = block_sum<256>(sum, red) / (float)width;
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        v[i].x -= mean; v[i].y -= mean; v[i].z -= mean; v[i].w -= mean;
+        if ((int)threadIdx.x + 256 * i < n4) ss += (v[i].x * v[i].x + v[i].y * v[i].y) + (v[i].z * v[i].z + v[i].w * v[i].w);
+    }
+    const float r = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)width + eps);
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        if ((int)threadIdx.x + 256 * i < n4)
+            *reinterpret_cast<uint2*>(out + row * ldo + at[i]) = uint2{f32x2_to_bf16x2(fmaf(v[i].x * r, wv[i].x, bv[i].x), fmaf(v[i].y * r, wv[i].y, bv[i].y)),
+                                                                      f32x2_to_bf16x2(fmaf(v[i].z * r, wv[i].z, bv[i].z), fmaf(v[i].w * r, wv[i].w, bv[i].w))};
+    }
 }
 
 }  // namespace
@@ -288,25 +388,26 @@ static int groups_fit(int n_experts, int top, int n_groups, int keep) {
 }
 
 GI_API int gi_route_top(const float* logits, long ld, int n_rows, int n_experts, int top, int score_kind, int renormalize, float floor, int n_groups, int keep,
-                        int* ids, float* weights, hipStream_t stream) {
+                        const float* correction, float scale, int* ids, float* weights, hipStream_t stream) {
+    GI_REQUIRE(correction == nullptr || n_groups == 1, "route_top: a correction of the scores and groups of experts do not go together");
     GI_REQUIRE(groups_fit(n_experts, top, n_groups, keep), "route_top: %d experts in %d groups of which %d are kept cannot give %d a row", n_experts, n_groups, keep, top);
     GI_REQUIRE(n_rows > 0 && n_experts > 0 && n_experts <= 64 * ROUTE_PER_LANE && top > 0 && top <= n_experts && top <= 64 && ld >= n_experts && (score_kind == 0 || score_kind == 1),
                "route_top: bad sizes (rows %d, experts %d, top %d)", n_rows, n_experts, top);
-    route_top_kernel<<<n_rows, 64, 0, stream>>>(logits, ld, n_experts, top, score_kind, renormalize, floor, n_groups, keep, ids, weights);
+    route_top_kernel<<<n_rows, 64, 0, stream>>>(logits, ld, n_experts, top, score_kind, renormalize, floor, n_groups, keep, correction, scale, ids, weights);
     GI_CHECK_LAUNCH("route_top");
     return 0;
 }
 
 GI_API int gi_experts_gate_up(const void* h, int h_dtype, long ldh, const void* w_gate, const void* w_up, int w_dtype, const int* ids, const float* weights,
-                              int weigh_input, void* mid, int mid_dtype, long ldm, int n_rows, int top, int width, int ff, int act, float limit, int group, hipStream_t stream) {
-    GI_REQUIRE(n_rows > 0 && top > 0 && top <= 65535 && width > 0 && ff > 0 && ldh >= width && ldm >= ff && act >= 0 && act < GI_N_ACTIVATIONS && (long)n_rows * top < (1l << 31)
+                              int weigh_input, void* mid, int mid_dtype, long ldm, int n_rows, int top, int width, int ff, int act, float limit, int group, int n_experts, hipStream_t stream) {
+    GI_REQUIRE(n_rows > 0 && n_experts > 0 && top > 0 && top <= 65535 && width > 0 && ff > 0 && ldh >= width && ldm >= ff && act >= 0 && act < GI_N_ACTIVATIONS && (long)n_rows * top < (1l << 31)
                && (group == 0 ? w_up != nullptr : group > 0 && ff % group == 0),
                "experts_gate_up: bad sizes (rows %d, top %d, width %d, ff %d)", n_rows, top, width, ff);
     dim3 grid(n_rows * top, (ff + 3) / 4);
     GI_REQUIRE(grid.y <= 65535, "experts_gate_up: experts too wide");
 #define LAUNCH(TW, TA, TO)                                                                                                                      \
     experts_gate_up_kernel<TW, TA, TO><<<grid, 256, 0, stream>>>((const TA*)h, ldh, (const TW*)w_gate, (const TW*)w_up, ids, weights, weigh_input, \
-                                                                 top, (TO*)mid, ldm, width, ff, act, limit, group)
+                                                                 top, (TO*)mid, ldm, width, ff, act, limit, group, n_experts)
     if (w_dtype == GI_BF16 && h_dtype == GI_BF16 && mid_dtype == GI_BF16) LAUNCH(bf16_t, bf16_t, bf16_t);
     else if (w_dtype == GI_F32 && h_dtype == GI_F32 && mid_dtype == GI_F32) LAUNCH(float, float, float);
     else if (w_dtype == GI_BF16 && h_dtype == GI_F32 && mid_dtype == GI_F32) LAUNCH(bf16_t, float, float);
@@ -317,29 +418,35 @@ GI_API int gi_experts_gate_up(const void* h, int h_dtype, long ldh, const void* 
 }
 
 GI_API int gi_experts_down(const void* mid, int mid_dtype, long ldm, const void* w_down, int w_dtype, const int* ids, const float* weights, int weigh_output,
-                           float* x, long ldx, int accumulate, int n_rows, int top, int width, int ff, hipStream_t stream) {
+                           float* x, long ldx, int accumulate, int n_rows, int top, int width, int ff, const void* h, int h_dtype, long ldh, int n_experts, hipStream_t stream) {
+    GI_REQUIRE(n_experts > 0 && h != nullptr && ldh >= width, "experts_down: the experts' inputs are missing or too short");
     GI_REQUIRE(n_rows > 0 && top > 0 && width > 0 && ff > 0 && ldx >= width && ldm >= ff, "experts_down: bad sizes (rows %d, top %d, width %d, ff %d)", n_rows, top, width, ff);
     dim3 grid(n_rows, (width + 3) / 4);
     GI_REQUIRE(grid.y <= 65535, "experts_down: rows too wide");
-#define LAUNCH(TW, TM) experts_down_kernel<TW, TM><<<grid, 256, 0, stream>>>((const TM*)mid, ldm, (const TW*)w_down, ids, weights, weigh_output, top, x, ldx, width, ff, accumulate)
-    if (w_dtype == GI_BF16 && mid_dtype == GI_BF16) LAUNCH(bf16_t, bf16_t);
-    else if (w_dtype == GI_F32 && mid_dtype == GI_F32) LAUNCH(float, float);
-    else if (w_dtype == GI_BF16 && mid_dtype == GI_F32) LAUNCH(bf16_t, float);
-    else return gi_fail("experts_down: dtypes (%d, %d) are not served", w_dtype, mid_dtype);
+#define LAUNCH(TW, TM, TA)                                                                                                                                                        \
+    experts_down_kernel<TW, TM, TA><<<grid, 256, 0, stream>>>((const TM*)mid, ldm, (const TW*)w_down, ids, weights, weigh_output, top, x, ldx, width, ff, accumulate, (const TA*)h, ldh, \
+                                                              n_experts)
+    if (w_dtype == GI_BF16 && mid_dtype == GI_BF16 && h_dtype == GI_BF16) LAUNCH(bf16_t, bf16_t, bf16_t);
+    else if (w_dtype == GI_F32 && mid_dtype == GI_F32 && h_dtype == GI_F32) LAUNCH(float, float, float);
+    else if (w_dtype == GI_BF16 && mid_dtype == GI_F32 && h_dtype == GI_F32) LAUNCH(bf16_t, float, float);
+    else if (w_dtype == GI_BF16 && mid_dtype == GI_BF16 && h_dtype == GI_F32) LAUNCH(bf16_t, bf16_t, float);
+    else if (w_dtype == GI_F32 && mid_dtype == GI_F32 && h_dtype == GI_BF16) LAUNCH(float, float, bf16_t);
+    else return gi_fail("experts_down: dtypes (%d, %d, %d) are not served", w_dtype, mid_dtype, h_dtype);
 #undef LAUNCH
     GI_CHECK_LAUNCH("experts_down");
     return 0;
 }
 
 GI_API int gi_route_rows(const void* h, int h_dtype, long ldh, const void* router, int r_dtype, long ldr, int n_rows, int width, int n_experts, int top, int score_kind,
-                         int renormalize, float floor, int n_groups, int keep, int* ids, float* weights, float* logits, long ldl, int n_extra, float* extra, long lde,
-                         hipStream_t stream) {
+                         int renormalize, float floor, int n_groups, int keep, const float* correction, float scale, int* ids, float* weights, float* logits, long ldl, int n_extra,
+                         float* extra, long lde, hipStream_t stream) {
+    GI_REQUIRE(correction == nullptr || n_groups == 1, "route_rows: a correction of the scores and groups of experts do not go together");
     GI_REQUIRE(n_extra >= 0 && (n_extra == 0 || (extra != nullptr && lde >= n_extra)), "route_rows: %d rows behind the experts' need room for their products", n_extra);
     GI_REQUIRE(groups_fit(n_experts, top, n_groups, keep), "route_rows: %d experts in %d groups of which %d are kept cannot give %d a row", n_experts, n_groups, keep, top);
     GI_REQUIRE(n_rows > 0 && width > 0 && n_experts > 0 && n_experts <= ROUTE_MAX_EXPERTS && top > 0 && top <= n_experts && top <= 64 && ldh >= width && ldr >= width
                && (score_kind == 0 || score_kind == 1) && (logits == nullptr || ldl >= n_experts),
                "route_rows: bad sizes (rows %d, width %d, experts %d, top %d)", n_rows, width, n_experts, top);
-#define LAUNCH(TA, TW) route_rows_kernel<TA, TW><<<n_rows, 256, 0, stream>>>((const TA*)h, ldh, (const TW*)router, ldr, width, n_experts, top, score_kind, renormalize, floor, n_groups, keep, ids, weights, logits, ldl, n_extra, extra, lde)
+#define LAUNCH(TA, TW) route_rows_kernel<TA, TW><<<n_rows, 256, 0, stream>>>((const TA*)h, ldh, (const TW*)router, ldr, width, n_experts, top, score_kind, renormalize, floor, n_groups, keep, correction, scale, ids, weights, logits, ldl, n_extra, extra, lde)
     if (h_dtype == GI_BF16 && r_dtype == GI_BF16) LAUNCH(bf16_t, bf16_t);
     else if (h_dtype == GI_F32 && r_dtype == GI_F32) LAUNCH(float, float);
     else if (h_dtype == GI_F32 && r_dtype == GI_BF16) LAUNCH(float, bf16_t);
@@ -363,21 +470,45 @@ GI_API int gi_experts_place(const int* ids, int n_items, int n_experts, int* cou
     return 0;
 }
 
-GI_API int gi_experts_gather(const void* h, long ldh, const int* place, const float* weights, int weigh_input, int n_rows, int top, void* out, long ldo, int width,
-                             hipStream_t stream) {
+GI_API int gi_experts_gather(const void* h, long ldh, const int* ids, const int* place, const float* weights, int weigh_input, int n_rows, int top, void* out, long ldo, int width,
+                             int n_experts, hipStream_t stream) {
     GI_REQUIRE(n_rows > 0 && top > 0 && width > 0 && width % 8 == 0 && ldh % 8 == 0 && ldo % 8 == 0 && ldh >= width && ldo >= width && (long)n_rows * top < (1l << 31)
                && ((uintptr_t)h & 15) == 0 && ((uintptr_t)out & 15) == 0, "experts_gather: bad sizes (rows %d, top %d, width %d)", n_rows, top, width);
-    experts_gather_kernel<<<n_rows * top, 256, 0, stream>>>((const bf16_t*)h, ldh, place, weights, weigh_input, top, (bf16_t*)out, ldo, width);
+    experts_gather_kernel<<<n_rows * top, 256, 0, stream>>>((const bf16_t*)h, ldh, ids, place, weights, weigh_input, top, (bf16_t*)out, ldo, width, n_experts);
     GI_CHECK_LAUNCH("experts_gather");
     return 0;
 }
 
-GI_API int gi_experts_combine(const float* y, long ldy, const int* place, const float* weights, int weigh_output, int n_rows, int top, float* x, long ldx, int width,
-                              int accumulate, hipStream_t stream) {
-    GI_REQUIRE(n_rows > 0 && top > 0 && width > 0 && ldy >= width && ldx >= width, "experts_combine: bad sizes (rows %d, top %d, width %d)", n_rows, top, width);
+// norm_w, norm_b, out: also the layer norm of the new rows as bfloat16 (nullptr: none); widths gi_experts_combine_norm_takes names, rows at multiples of 16 bytes.
+GI_API int gi_experts_combine_norm_takes(int width) { return width > 0 && width % 4 == 0 && width <= 8192; }
+
+GI_API int gi_experts_combine(const float* y, long ldy, const int* ids, const int* place, const float* weights, int weigh_output, int n_rows, int top, float* x, long ldx, int width,
+                              int accumulate, const void* h, long ldh, int n_experts, const void* norm_w, const void* norm_b, int norm_dtype, float eps, void* out, long ldo,
+                              hipStream_t stream) {
+    GI_REQUIRE(n_rows > 0 && top > 0 && width > 0 && ldy >= width && ldx >= width && n_experts > 0 && h != nullptr && ldh >= width, "experts_combine: bad sizes (rows %d, top %d, width %d)",
+               n_rows, top, width);
+    if (out != nullptr) {
+        GI_REQUIRE(gi_experts_combine_norm_takes(width) && norm_w != nullptr && norm_b != nullptr && ldo >= width && ldy % 4 == 0 && ldx % 4 == 0 && ldh % 4 == 0 && ldo % 4 == 0 &&
+                   (((uintptr_t)y | (uintptr_t)x | (uintptr_t)h | (uintptr_t)norm_w | (uintptr_t)norm_b | (uintptr_t)out) & 15) == 0,
+                   "experts_combine: rows of %d columns, or their alignment, are not taken with a norm behind", width);
+#define LAUNCH_NORM(PER, TW)                                                                                                                                              \
+    experts_combine_norm_kernel<PER, TW><<<n_rows, 256, 0, stream>>>(y, ldy, ids, place, weights, weigh_output, top, x, ldx, width, accumulate, (const bf16_t*)h, ldh, n_experts, \
+                                                                     (const TW*)norm_w, (const TW*)norm_b, eps, (bf16_t*)out, ldo)
+#define BY_WIDTH(TW)                                                                                                                                                      \
+    do {                                                                                                                                                                  \
+        if (width <= 1024) LAUNCH_NORM(1, TW); else if (width <= 2048) LAUNCH_NORM(2, TW); else if (width <= 4096) LAUNCH_NORM(4, TW); else LAUNCH_NORM(8, TW);           \
+    } while (0)
+        if (norm_dtype == GI_F32) BY_WIDTH(float);
+        else if (norm_dtype == GI_BF16) BY_WIDTH(bf16_t);
+        else return gi_fail("experts_combine: unknown dtype %d", norm_dtype);
+#undef BY_WIDTH
+#undef LAUNCH_NORM
+        GI_CHECK_LAUNCH("experts_combine (with a norm)");
+        return 0;
+    }
     dim3 grid(n_rows, (width + 255) / 256);
     GI_REQUIRE(grid.y <= 65535, "experts_combine: rows too wide");
-    experts_combine_kernel<<<grid, 256, 0, stream>>>(y, ldy, place, weights, weigh_output, top, x, ldx, width, accumulate);
+    experts_combine_kernel<<<grid, 256, 0, stream>>>(y, ldy, ids, place, weights, weigh_output, top, x, ldx, width, accumulate, (const bf16_t*)h, ldh, n_experts);
     GI_CHECK_LAUNCH("experts_combine");
     return 0;
 }

@@ -8,14 +8,15 @@
 // A page holds its places' keys [place][kv_rank + rot] and, behind them, the latent once more with the places innermost
 // [kv_rank][place]: the layout of a layer with one key/value head whose values are shorter than its keys, which every attention
 // kernel reads, and both operands of the matrix instructions come out of memory as they lie.
-// The rotation here turns neighbouring channels, the pair (2i, 2i + 1) by pos * f_i.
+// The rotation turns neighbouring channels, the pair (2i, 2i + 1), or the pair (i, i + rot/2), by pos * f_i.
 //
 //   latent_prepare   one wave per (row, which): the query latent normed into the rows the up projection reads; the key/value
 //                    latent normed and the rotated part turned, both written to the row's place in its page
 //   latent_queries   one wave per (row, head): a head's unrotated channels into the rows the folding product reads, its
 //                    rotated channels turned and written behind the place where that product puts q'
+//   latent_direct    both of these in one launch, where the queries have no latent and so stand in the same rows as the key/value latent
 //   heads_product    out[t, h, :] = a[t, h, :] W_h^T for every head in one launch (the folding of W_uk into the queries and the
-//                    product with W_uv behind the attention), on the matrix cores
+//                    product with W_uv behind the attention, whose results a gate per channel may multiply on the way), on the matrix cores
 //   latent_attention one wave per (row, 16 heads, share of the context): all heads read the same keys, so 16 of them are the
 //                    columns of one matrix instruction even for a single decoded row; for the rows of prompts a workgroup takes a
 //                    few consecutive rows with all their heads and stages the keys they see once in LDS
@@ -23,56 +24,88 @@
 
 namespace {
 
+// A row's rot channels at src, turned, to dst: pairs of neighbours, or (half_split) the pairs (i, i + rot/2).
+template <typename TC>
+__device__ __forceinline__ void turn_pairs(const float* __restrict__ src, const float* __restrict__ cos_t, const float* __restrict__ sin_t, size_t t, int rot, int half_split,
+                                           int lane, TC* __restrict__ dst) {
+    for (int i = lane; i < rot / 2; i += 64) {
+        const int a = half_split ? i : 2 * i, b = half_split ? i + rot / 2 : 2 * i + 1;
+        const float u = src[a], v = src[b];
+        const float c = cos_t[t * (rot / 2) + i], s = sin_t[t * (rot / 2) + i];
+        store_f32(dst, a, u * c - v * s);
+        store_f32(dst, b, v * c + u * s);
+    }
+}
+
+// The key/value latent at src normed, and the rotated part behind it turned, to the row's place of its page: one wave.
+template <typename TW, typename TC>
+__device__ __forceinline__ void store_latent(const float* __restrict__ src, size_t t, int kv_rank, int rot, int half_split, const TW* __restrict__ w, float eps,
+                                             const float* __restrict__ cos_t, const float* __restrict__ sin_t, int p, long page, TC* __restrict__ cache, long page_stride,
+                                             int page_size, int lane) {
+    float ss = 0.f;
+    for (int d = lane; d < kv_rank; d += 64) ss = fmaf(src[d], src[d], ss);
+    const float r = 1.0f / sqrtf(wave_sum(ss) / (float)kv_rank + eps);
+    TC* dst = cache + page * page_stride + (size_t)(p % page_size) * (kv_rank + rot);
+    TC* as_value = cache + page * page_stride + (size_t)page_size * (kv_rank + rot) + p % page_size;      // [kv_rank][place]
+    for (int d = lane; d < kv_rank; d += 64) {
+        const float c = load_f32(w, d) * (r * src[d]);
+        store_f32(dst, d, c);
+        store_f32(as_value, (size_t)d * page_size, c);
+    }
+    turn_pairs(src + kv_rank, cos_t, sin_t, t, rot, half_split, lane, dst + kv_rank);
+}
+
+// A head's query at src parted: its unrotated channels to `plain`, the turned ones to `turned`: one wave.
+template <typename TA, typename TC>
+__device__ __forceinline__ void part_query(const float* __restrict__ src, size_t t, int dim, int rot, int half_split, const float* __restrict__ cos_t, const float* __restrict__ sin_t,
+                                           int lane, TA* __restrict__ plain, TC* __restrict__ turned) {
+    for (int d = lane; d < dim; d += 64) store_f32(plain, d, src[d]);
+    turn_pairs(src + dim, cos_t, sin_t, t, rot, half_split, lane, turned);
+}
+
 template <typename TW, typename TA, typename TC>
 __global__ __launch_bounds__(64) void latent_prepare_kernel(const float* __restrict__ proj, long ld, int q_rank, int kv_rank, int rot,
                                                            const TW* __restrict__ q_norm, const TW* __restrict__ kv_norm, float eps,
                                                            const float* __restrict__ cos_t, const float* __restrict__ sin_t,
                                                            const int* __restrict__ pos, const int* __restrict__ slot, const int* __restrict__ table,
                                                            int table_stride, TA* __restrict__ cq, long ldcq, TC* __restrict__ cache, long page_stride,
-                                                           int page_size) {
+                                                           int page_size, int half_split) {
     const int t = blockIdx.x, lane = threadIdx.x;
-    const bool query = blockIdx.y == 0;
-    const float* src = proj + (size_t)t * ld + (query ? 0 : q_rank);
-    const int n = query ? q_rank : kv_rank;
-    const TW* w = query ? q_norm : kv_norm;
-    float ss = 0.f;
-    for (int d = lane; d < n; d += 64) ss = fmaf(src[d], src[d], ss);
-    const float r = 1.0f / sqrtf(wave_sum(ss) / (float)n + eps);
-    if (query) {
-        for (int d = lane; d < n; d += 64) store_f32(cq, (size_t)t * ldcq + d, load_f32(w, d) * (r * src[d]));
+    const float* src = proj + (size_t)t * ld;
+    if (blockIdx.y == 0) {
+        float ss = 0.f;
+        for (int d = lane; d < q_rank; d += 64) ss = fmaf(src[d], src[d], ss);
+        const float r = 1.0f / sqrtf(wave_sum(ss) / (float)q_rank + eps);
+        for (int d = lane; d < q_rank; d += 64) store_f32(cq, (size_t)t * ldcq + d, load_f32(q_norm, d) * (r * src[d]));
         return;
     }
     const int p = pos[t];
-    const long page = table[(size_t)slot[t] * table_stride + p / page_size];
-    TC* dst = cache + page * page_stride + (size_t)(p % page_size) * (kv_rank + rot);
-    TC* as_value = cache + page * page_stride + (size_t)page_size * (kv_rank + rot) + p % page_size;      // [kv_rank][place]
-    for (int d = lane; d < n; d += 64) {
-        const float c = load_f32(w, d) * (r * src[d]);
-        store_f32(dst, d, c);
-        store_f32(as_value, (size_t)d * page_size, c);
-    }
-    for (int i = lane; i < rot / 2; i += 64) {
-        const float u = src[kv_rank + 2 * i], v = src[kv_rank + 2 * i + 1];
-        const float c = cos_t[(size_t)t * (rot / 2) + i], s = sin_t[(size_t)t * (rot / 2) + i];
-        store_f32(dst, kv_rank + 2 * i, u * c - v * s);
-        store_f32(dst, kv_rank + 2 * i + 1, v * c + u * s);
-    }
+    store_latent(src + q_rank, t, kv_rank, rot, half_split, kv_norm, eps, cos_t, sin_t, p, (long)table[(size_t)slot[t] * table_stride + p / page_size], cache, page_stride, page_size, lane);
 }
 
 template <typename TA, typename TC>
 __global__ __launch_bounds__(64) void latent_queries_kernel(const float* __restrict__ q, long ldq, const float* __restrict__ cos_t,
                                                            const float* __restrict__ sin_t, TA* __restrict__ plain, long ld_plain,
-                                                           TC* __restrict__ folded, long ld_folded, int n_heads, int dim, int rot, int kv_rank) {
-    const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
-    const float* src = q + (size_t)t * ldq + (size_t)h * (dim + rot);
-    for (int d = lane; d < dim; d += 64) store_f32(plain, (size_t)t * ld_plain + (size_t)h * dim + d, src[d]);
-    TC* dst = folded + (size_t)t * ld_folded + (size_t)h * (kv_rank + rot) + kv_rank;
-    for (int i = lane; i < rot / 2; i += 64) {
-        const float u = src[dim + 2 * i], v = src[dim + 2 * i + 1];
-        const float c = cos_t[(size_t)t * (rot / 2) + i], s = sin_t[(size_t)t * (rot / 2) + i];
-        store_f32(dst, 2 * i, u * c - v * s);
-        store_f32(dst, 2 * i + 1, v * c + u * s);
+                                                           TC* __restrict__ folded, long ld_folded, int dim, int rot, int kv_rank, int half_split) {
+    const size_t t = blockIdx.x, h = blockIdx.y;
+    part_query(q + t * ldq + h * (dim + rot), t, dim, rot, half_split, cos_t, sin_t, threadIdx.x, plain + t * ld_plain + h * dim, folded + t * ld_folded + h * (kv_rank + rot) + kv_rank);
+}
+
+// item 0: the row's key/value latent into its page; items 1 ..: the heads' queries.
+template <typename TW, typename TA, typename TC>
+__global__ __launch_bounds__(64) void latent_direct_kernel(const float* __restrict__ q, long ldq, const float* __restrict__ kv, long ldkv, const TW* __restrict__ kv_norm, float eps,
+                                                          const float* __restrict__ cos_t, const float* __restrict__ sin_t, const int* __restrict__ pos, const int* __restrict__ slot,
+                                                          const int* __restrict__ table, int table_stride, TA* __restrict__ plain, long ld_plain, TC* __restrict__ folded,
+                                                          long ld_folded, TC* __restrict__ cache, long page_stride, int page_size, int dim, int rot, int kv_rank, int half_split) {
+    const size_t t = blockIdx.x;
+    if (blockIdx.y == 0) {
+        const int p = pos[t];
+        store_latent(kv + t * ldkv, t, kv_rank, rot, half_split, kv_norm, eps, cos_t, sin_t, p, (long)table[(size_t)slot[t] * table_stride + p / page_size], cache, page_stride, page_size,
+                     (int)threadIdx.x);
+        return;
     }
+    const size_t h = blockIdx.y - 1;
+    part_query(q + t * ldq + h * (dim + rot), t, dim, rot, half_split, cos_t, sin_t, threadIdx.x, plain + t * ld_plain + h * dim, folded + t * ld_folded + h * (kv_rank + rot) + kv_rank);
 }
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
@@ -80,12 +113,14 @@ typedef float floatx4 __attribute__((ext_vector_type(4)));
 typedef unsigned int uintx4 __attribute__((ext_vector_type(4)));
 __device__ __forceinline__ bf16x8 as_bf16x8(uint4 v) { return __builtin_bit_cast(bf16x8, v); }
 __device__ __forceinline__ float exp2_fast(float x) { return __builtin_amdgcn_exp2f(x); }
+constexpr float LOG2E = 1.4426950408889634f;
 
 // out[t, h*n_out + n] = sum_k a[t, h*k_dim + k] * w[h][n][k], bfloat16 operands, 32-bit sums.  One wave per (16 rows, head, 64
-// columns): the operands of the 16x16x32 matrix instruction are 16-byte pieces of a's and w's rows as they lie in memory.
+// columns): the operands of the 16x16x32 matrix instruction are 16-byte pieces of a's and w's rows as they lie in memory.  With `gate`
+// (float32 [n_rows, ldg], head h's channels from h*n_out on) every result is multiplied by sigmoid(gate).
 template <typename TO>
 __global__ __launch_bounds__(64) void heads_product_kernel(const bf16_t* __restrict__ a, long lda, const bf16_t* __restrict__ w, TO* __restrict__ out, long ldo,
-                                                          long out_head_stride, int n_rows, int k_dim, int n_out) {
+                                                          long out_head_stride, int n_rows, int k_dim, int n_out, const float* __restrict__ gate, long ldg) {
     const int lane = threadIdx.x, r = lane & 15, q4 = lane >> 4;
     const int row0 = blockIdx.x * 16, h = blockIdx.y, col0 = blockIdx.z * 64;
     const int row = min(row0 + r, n_rows - 1);
@@ -112,7 +147,10 @@ __global__ __launch_bounds__(64) void heads_product_kernel(const bf16_t* __restr
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
             const int t = row0 + 4 * q4 + v;
-            if (t < n_rows && col < n_out) store_f32(out, (size_t)t * ldo + (size_t)h * out_head_stride + col, acc[j][v]);
+            if (t < n_rows && col < n_out) {
+                const float y = gate ? acc[j][v] / (1.0f + expf(-gate[(size_t)t * ldg + (size_t)h * n_out + col])) : acc[j][v];
+                store_f32(out, (size_t)t * ldo + (size_t)h * out_head_stride + col, y);
+            }
         }
     }
 }
@@ -123,11 +161,13 @@ __global__ __launch_bounds__(64) void heads_product_kernel(const bf16_t* __restr
 // the second operand of O^T = V^T P^T.  KS = key channels / 32 (rounded up: pieces beyond the key are zeros), DT = value channels / 16.
 // Shares of one row meet in `part` ([row][head][share]{m, l, o[vd]}, 32-bit) and `latent_merge_kernel` adds them; with one share
 // the wave writes the heads' outputs itself.  `rows`: the step's rows that this launch serves (nullptr: all, in order).
+// `sinks` [heads], where given: a score per head that joins the softmax's sum and has no value; the row's first share starts from it.
 template <int KS, int DT>
 __global__ __launch_bounds__(64) void latent_attention_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ cache, bf16_t* __restrict__ out,
                                                              float* __restrict__ part, const int* __restrict__ rows, const int* __restrict__ pos,
                                                              const int* __restrict__ slot, const int* __restrict__ table, int table_stride, long page_stride,
-                                                             int page_size, int n_heads, int kd, int vd, int window, float scale2, int n_splits) {
+                                                             int page_size, int n_heads, int kd, int vd, int window, float scale2, int n_splits,
+                                                             const float* __restrict__ sinks) {
     const int lane = threadIdx.x, r = lane & 15, q4 = lane >> 4;
     const int t = rows ? rows[blockIdx.x] : blockIdx.x, hg = blockIdx.y, sp = blockIdx.z;
     const int head = hg * 16 + r;
@@ -153,6 +193,7 @@ __global__ __launch_bounds__(64) void latent_attention_kernel(const bf16_t* __re
 #pragma unroll
     for (int i = 0; i < DT; ++i) o[i] = floatx4{};
     float m = -INFINITY, l = 0.f;
+    if (sinks && sp == 0) m = sinks[head_ok ? head : 0] * LOG2E, l = 1.f;
 
     for (int tile = tile0; tile < tile1; ++tile) {
         const int kv0 = tile << 5;
@@ -283,7 +324,7 @@ template <int KS, int DT, bool AHEAD>
 __global__ __launch_bounds__(512) void latent_attention_tiles_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ cache, bf16_t* __restrict__ out,
                                                                     const int4* __restrict__ tiles, int pieces_per_tile, int TR, int HG,
                                                                     const int* __restrict__ table, int table_stride, long page_stride, int page_size,
-                                                                    int n_heads, int kd, int vd, int window, float scale2) {
+                                                                    int n_heads, int kd, int vd, int window, float scale2, const float* __restrict__ sinks) {
     extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
     constexpr int KP = KS * 32 + 8, VP = 40;
     bf16_t* Ks = reinterpret_cast<bf16_t*>(lds);         // [32][KP]
@@ -317,6 +358,7 @@ __global__ __launch_bounds__(512) void latent_attention_tiles_kernel(const bf16_
 #pragma unroll
     for (int i = 0; i < DT; ++i) o[i] = floatx4{};
     float m = -INFINITY, l = 0.f;
+    if (sinks) m = sinks[head < n_heads ? head : 0] * LOG2E, l = 1.f;
     const int k_pieces = kd >> 3;
     // A tile on its way: every position's key in 16-byte pieces, every value channel's 32 places in four.  With AHEAD the next
     // tile is asked for into registers before this one is worked on (workgroups have 320 threads or more: a thread brings at most
@@ -438,7 +480,7 @@ __global__ __launch_bounds__(512) void latent_attention_tiles_kernel(const bf16_
 // [n_rows, rot/2]; cq: [n_rows, ldcq] gets the normed query latent; the cache's pages hold [place][kv_rank + rot], then [kv_rank][place].
 GI_API int gi_latent_prepare(const float* proj, long ld, int q_rank, int kv_rank, int rot, const void* q_norm, const void* kv_norm, int norm_dtype,
                              float eps, const float* cos_t, const float* sin_t, const int* pos, const int* slot, const int* table, int table_stride,
-                             void* cq, int cq_dtype, long ldcq, void* cache, int cache_dtype, long page_stride, int page_size, int n_rows,
+                             void* cq, int cq_dtype, long ldcq, void* cache, int cache_dtype, long page_stride, int page_size, int half_split, int n_rows,
                              hipStream_t stream) {
     GI_REQUIRE(n_rows > 0 && q_rank > 0 && kv_rank > 0 && rot >= 0 && rot % 2 == 0, "latent_prepare: bad sizes (rows %d, latents %d and %d, %d rotated channels)",
                n_rows, q_rank, kv_rank, rot);
@@ -448,7 +490,7 @@ GI_API int gi_latent_prepare(const float* proj, long ld, int q_rank, int kv_rank
     dim3 grid(n_rows, 2);
 #define GO(TW, TA, TC)                                                                                                                        \
     latent_prepare_kernel<TW, TA, TC><<<grid, 64, 0, stream>>>(proj, ld, q_rank, kv_rank, rot, (const TW*)q_norm, (const TW*)kv_norm, eps, cos_t, sin_t, pos, \
-                                                               slot, table, table_stride, (TA*)cq, ldcq, (TC*)cache, page_stride, page_size)
+                                                               slot, table, table_stride, (TA*)cq, ldcq, (TC*)cache, page_stride, page_size, half_split)
     if (norm_dtype == GI_F32 && cq_dtype == GI_F32 && cache_dtype == GI_F32) GO(float, float, float);
     else if (norm_dtype == GI_BF16 && cq_dtype == GI_BF16 && cache_dtype == GI_BF16) GO(bf16_t, bf16_t, bf16_t);
     else if (norm_dtype == GI_F32 && cq_dtype == GI_BF16 && cache_dtype == GI_BF16) GO(float, bf16_t, bf16_t);
@@ -463,13 +505,13 @@ GI_API int gi_latent_prepare(const float* proj, long ld, int q_rank, int kv_rank
 // q: float32 [n_rows, ldq], per head [dim unrotated | rot rotated]; plain: [n_rows, ld_plain] gets the heads' unrotated channels
 // [n_heads][dim]; folded: [n_rows, ld_folded], per head [kv_rank + rot], gets the turned channels behind each head's first kv_rank.
 GI_API int gi_latent_queries(const float* q, long ldq, const float* cos_t, const float* sin_t, void* plain, int plain_dtype, long ld_plain, void* folded,
-                             int folded_dtype, long ld_folded, int n_rows, int n_heads, int dim, int rot, int kv_rank, hipStream_t stream) {
+                             int folded_dtype, long ld_folded, int n_rows, int n_heads, int dim, int rot, int kv_rank, int half_split, hipStream_t stream) {
     GI_REQUIRE(n_rows > 0 && n_heads > 0 && n_heads <= 65535 && dim > 0 && rot >= 0 && rot % 2 == 0 && kv_rank > 0, "latent_queries: bad sizes (rows %d, heads %d, %d + %d channels)",
                n_rows, n_heads, dim, rot);
     GI_REQUIRE(ldq >= (long)n_heads * (dim + rot) && ld_plain >= (long)n_heads * dim && ld_folded >= (long)n_heads * (kv_rank + rot), "latent_queries: rows too short");
     GI_REQUIRE(rot == 0 || (cos_t != nullptr && sin_t != nullptr), "latent_queries: a rotation needs its cosines and sines");
     dim3 grid(n_rows, n_heads);
-#define GO(TA, TC) latent_queries_kernel<TA, TC><<<grid, 64, 0, stream>>>(q, ldq, cos_t, sin_t, (TA*)plain, ld_plain, (TC*)folded, ld_folded, n_heads, dim, rot, kv_rank)
+#define GO(TA, TC) latent_queries_kernel<TA, TC><<<grid, 64, 0, stream>>>(q, ldq, cos_t, sin_t, (TA*)plain, ld_plain, (TC*)folded, ld_folded, dim, rot, kv_rank, half_split)
     if (plain_dtype == GI_F32 && folded_dtype == GI_F32) GO(float, float);
     else if (plain_dtype == GI_BF16 && folded_dtype == GI_BF16) GO(bf16_t, bf16_t);
     else if (plain_dtype == GI_F32 && folded_dtype == GI_BF16) GO(float, bf16_t);
@@ -479,20 +521,47 @@ GI_API int gi_latent_queries(const float* q, long ldq, const float* cos_t, const
     return 0;
 }
 
+// q: float32 [n_rows, ldq], per head [dim unrotated | rot rotated]; kv: float32 [n_rows, ldkv] = [key/value latent (kv_rank) | rotated key
+// part (rot)]; plain, folded and the cache as the two above fill them.
+GI_API int gi_latent_direct(const float* q, long ldq, const float* kv, long ldkv, const void* kv_norm, int norm_dtype, float eps, const float* cos_t, const float* sin_t,
+                            const int* pos, const int* slot, const int* table, int table_stride, void* plain, int plain_dtype, long ld_plain, void* folded, long ld_folded,
+                            void* cache, int cache_dtype, long page_stride, int page_size, int half_split, int n_rows, int n_heads, int dim, int rot, int kv_rank,
+                            hipStream_t stream) {
+    GI_REQUIRE(n_rows > 0 && n_heads > 0 && n_heads < 65535 && dim > 0 && rot >= 0 && rot % 2 == 0 && kv_rank > 0, "latent_direct: bad sizes (rows %d, heads %d, %d + %d channels, latent %d)",
+               n_rows, n_heads, dim, rot, kv_rank);
+    GI_REQUIRE(ldq >= (long)n_heads * (dim + rot) && ldkv >= (long)kv_rank + rot && ld_plain >= (long)n_heads * dim && ld_folded >= (long)n_heads * (kv_rank + rot) && page_size > 0 &&
+               page_stride >= (long)page_size * (2L * kv_rank + rot), "latent_direct: rows or pages too short");
+    GI_REQUIRE(rot == 0 || (cos_t != nullptr && sin_t != nullptr), "latent_direct: a rotation needs its cosines and sines");
+    dim3 grid(n_rows, n_heads + 1);
+#define GO(TW, TA, TC)                                                                                                                                   \
+    latent_direct_kernel<TW, TA, TC><<<grid, 64, 0, stream>>>(q, ldq, kv, ldkv, (const TW*)kv_norm, eps, cos_t, sin_t, pos, slot, table, table_stride, (TA*)plain, ld_plain, \
+                                                              (TC*)folded, ld_folded, (TC*)cache, page_stride, page_size, dim, rot, kv_rank, half_split)
+    if (norm_dtype == GI_F32 && plain_dtype == GI_F32 && cache_dtype == GI_F32) GO(float, float, float);
+    else if (norm_dtype == GI_BF16 && plain_dtype == GI_BF16 && cache_dtype == GI_BF16) GO(bf16_t, bf16_t, bf16_t);
+    else if (norm_dtype == GI_F32 && plain_dtype == GI_BF16 && cache_dtype == GI_BF16) GO(float, bf16_t, bf16_t);
+    else if (norm_dtype == GI_F32 && plain_dtype == GI_F32 && cache_dtype == GI_BF16) GO(float, float, bf16_t);
+    else if (norm_dtype == GI_BF16 && plain_dtype == GI_F32 && cache_dtype == GI_BF16) GO(bf16_t, float, bf16_t);
+    else return gi_fail("latent_direct: dtypes (%d, %d, %d) are not served", norm_dtype, plain_dtype, cache_dtype);
+#undef GO
+    GI_CHECK_LAUNCH("latent_direct");
+    return 0;
+}
+
 // a: bfloat16 [n_rows, lda], head h's operand in columns [h*k_dim, (h+1)*k_dim); w: bfloat16 [n_heads][n_out][k_dim]; out: [n_rows, ldo],
 // head h's result in columns [h*out_head_stride, h*out_head_stride + n_out).
 GI_API int gi_heads_product_supports(int k_dim, int n_out) { return k_dim > 0 && n_out > 0 && k_dim % 8 == 0; }
 
 GI_API int gi_heads_product(const void* a, long lda, const void* w, void* out, int out_dtype, long ldo, long out_head_stride, int n_rows, int n_heads, int k_dim,
-                            int n_out, hipStream_t stream) {
+                            int n_out, const float* gate, long ldg, hipStream_t stream) {
+    GI_REQUIRE(gate == nullptr || ldg >= (long)n_heads * n_out, "heads_product: the gates' rows are too short");
     GI_REQUIRE(n_rows > 0 && n_heads > 0 && n_heads <= 65535 && gi_heads_product_supports(k_dim, n_out), "heads_product: bad sizes (rows %d, heads %d, k %d, n %d; k a multiple of 8)",
                n_rows, n_heads, k_dim, n_out);
     GI_REQUIRE(lda % 8 == 0 && lda >= (long)n_heads * k_dim && ((uintptr_t)a & 15) == 0 && ((uintptr_t)w & 15) == 0 && out_head_stride >= n_out &&
                ldo >= (long)(n_heads - 1) * out_head_stride + n_out, "heads_product: operands must be 16-byte aligned with row strides that are multiples of 8, and rows long enough");
     GI_REQUIRE((n_out + 63) / 64 <= 65535, "heads_product: too many columns");
     dim3 grid((n_rows + 15) / 16, n_heads, (n_out + 63) / 64);
-    if (out_dtype == GI_F32) heads_product_kernel<float><<<grid, 64, 0, stream>>>((const bf16_t*)a, lda, (const bf16_t*)w, (float*)out, ldo, out_head_stride, n_rows, k_dim, n_out);
-    else if (out_dtype == GI_BF16) heads_product_kernel<bf16_t><<<grid, 64, 0, stream>>>((const bf16_t*)a, lda, (const bf16_t*)w, (bf16_t*)out, ldo, out_head_stride, n_rows, k_dim, n_out);
+    if (out_dtype == GI_F32) heads_product_kernel<float><<<grid, 64, 0, stream>>>((const bf16_t*)a, lda, (const bf16_t*)w, (float*)out, ldo, out_head_stride, n_rows, k_dim, n_out, gate, ldg);
+    else if (out_dtype == GI_BF16) heads_product_kernel<bf16_t><<<grid, 64, 0, stream>>>((const bf16_t*)a, lda, (const bf16_t*)w, (bf16_t*)out, ldo, out_head_stride, n_rows, k_dim, n_out, gate, ldg);
     else return gi_fail("heads_product: unknown output dtype %d", out_dtype);
     GI_CHECK_LAUNCH("heads_product");
     return 0;
@@ -510,7 +579,7 @@ GI_API long gi_latent_attention_scratch_floats(int n_rows, int n_heads, int vd, 
 // rows: the n_rows rows of the step to serve (nullptr: rows 0 .. n_rows - 1).
 GI_API int gi_latent_attention_bf16(const void* q, const void* cache, void* out, float* part, long part_floats, const int* rows, const int* pos, const int* slot,
                                     const int* table, int table_stride, long page_stride, int page_size, int n_rows, int n_heads, int kd, int vd, int window,
-                                    float scale, int n_splits, hipStream_t stream) {
+                                    float scale, int n_splits, const float* sinks, hipStream_t stream) {
     GI_REQUIRE(n_rows > 0 && n_heads > 0 && gi_latent_attention_supports(kd, vd, page_size), "latent_attention: sizes (rows %d, heads %d, keys %d, values %d, pages of %d) are not taken",
                n_rows, n_heads, kd, vd, page_size);
     GI_REQUIRE(window >= 0 && n_splits >= 1 && n_splits <= 64 && page_stride >= (long)page_size * (kd + vd) && page_stride % 8 == 0 && ((uintptr_t)cache & 15) == 0 &&
@@ -522,7 +591,7 @@ GI_API int gi_latent_attention_bf16(const void* q, const void* cache, void* out,
     const float scale2 = scale * 1.4426950408889634f;
 #define GO(KS, DT)                                                                                                                                      \
     latent_attention_kernel<KS, DT><<<grid, 64, 0, stream>>>((const bf16_t*)q, (const bf16_t*)cache, (bf16_t*)out, part, rows, pos, slot, table, table_stride, \
-                                                             page_stride, page_size, n_heads, kd, vd, window, scale2, n_splits)
+                                                             page_stride, page_size, n_heads, kd, vd, window, scale2, n_splits, sinks)
     if (kd <= 96 && vd <= 64) GO(3, 4);
     else if (kd <= 160 && vd <= 128) GO(5, 8);
     else if (kd <= 288 && vd <= 256) GO(9, 16);
@@ -565,18 +634,19 @@ GI_API int gi_latent_attention_tiles_prepare() {
 
 template <int KS, int DT>
 static int launch_latent_tiles(const void* q, const void* cache, void* out, const void* tiles, int n_tiles, int tile_rows, const int* table, int table_stride,
-                               long page_stride, int page_size, int n_heads, int kd, int vd, int window, float scale2, hipStream_t stream) {
+                               long page_stride, int page_size, int n_heads, int kd, int vd, int window, float scale2, const float* sinks, hipStream_t stream) {
     const int HG = (n_heads + 15) / 16, TR = 8 / HG > 0 ? 8 / HG : 1;
     const int pieces = (tile_rows + TR - 1) / TR;
     const size_t lds_bytes = (size_t)(32 * (KS * 32 + 8) + DT * 16 * 40) * 2;
     if (int rc = allow_latent_tiles_lds<KS, DT>()) return rc;
     latent_attention_tiles_kernel<KS, DT, (KS <= 9)><<<(unsigned)(n_tiles * pieces), 64 * TR * HG, lds_bytes, stream>>>(
-        (const bf16_t*)q, (const bf16_t*)cache, (bf16_t*)out, (const int4*)tiles, pieces, TR, HG, table, table_stride, page_stride, page_size, n_heads, kd, vd, window, scale2);
+        (const bf16_t*)q, (const bf16_t*)cache, (bf16_t*)out, (const int4*)tiles, pieces, TR, HG, table, table_stride, page_stride, page_size, n_heads, kd, vd, window, scale2,
+        sinks);
     return 0;
 }
 
 GI_API int gi_latent_attention_tiles_bf16(const void* q, const void* cache, void* out, const void* tiles, int n_tiles, int tile_rows, const int* table, int table_stride,
-                                          long page_stride, int page_size, int n_heads, int kd, int vd, int window, float scale, hipStream_t stream) {
+                                          long page_stride, int page_size, int n_heads, int kd, int vd, int window, float scale, const float* sinks, hipStream_t stream) {
     GI_REQUIRE(n_tiles > 0 && tile_rows > 0 && n_heads > 0 && gi_latent_attention_tiles_supports(n_heads, kd, vd, page_size),
                "latent_attention (tiles): sizes (%d tiles of %d rows, heads %d, keys %d, values %d, pages of %d) are not taken", n_tiles, tile_rows, n_heads, kd, vd, page_size);
     GI_REQUIRE(window >= 0 && page_stride >= (long)page_size * (kd + vd) && page_stride % 8 == 0 && ((uintptr_t)cache & 15) == 0 && ((uintptr_t)q & 15) == 0 &&
@@ -584,7 +654,7 @@ GI_API int gi_latent_attention_tiles_bf16(const void* q, const void* cache, void
     GI_REQUIRE((long)n_tiles * tile_rows < 2147483647L, "latent_attention (tiles): too many rows");
     const float scale2 = scale * 1.4426950408889634f;
     int rc;
-#define GO(KS, DT) rc = launch_latent_tiles<KS, DT>(q, cache, out, tiles, n_tiles, tile_rows, table, table_stride, page_stride, page_size, n_heads, kd, vd, window, scale2, stream)
+#define GO(KS, DT) rc = launch_latent_tiles<KS, DT>(q, cache, out, tiles, n_tiles, tile_rows, table, table_stride, page_stride, page_size, n_heads, kd, vd, window, scale2, sinks, stream)
     if (kd <= 96 && vd <= 64) GO(3, 4);
     else if (kd <= 160 && vd <= 128) GO(5, 8);
     else if (kd <= 288 && vd <= 256) GO(9, 16);

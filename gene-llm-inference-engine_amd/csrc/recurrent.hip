@@ -28,7 +28,7 @@
 // two sums over the key's rows, which the kernel takes in one pass over the memory as it was before the token.  Before the rule,
 // q, k and v pass a short causal convolution over the request's rows (the last taps - 1 rows before a step are part of the
 // request's state) and SiLU, and q and k are made unit vectors; after it, a head's output is divided by its root mean square, as
-// the matrix memory's.
+// the matrix memory's.  The decay is one number per head, or one per head and key channel, which then scales the memory's row of that channel.
 #include "common.h"
 
 namespace {
@@ -207,10 +207,13 @@ __global__ __launch_bounds__(64) void mlstm_scan_kernel(const float* __restrict_
 // y[t, h*dv + d] = w[h*dv + d] * o[t, h, d] * rsqrt(mean_d(o[t, h, :]^2) + eps) * sigmoid(g[t, h*dv + d]): one wave per (row, head).
 // With `den` [rows, heads], o is what the rows hold divided by den[t, h] (the matrix memory's sums and their divisor).
 // w_head_stride: dv where every head has weights of its own, 0 where all heads share one [dv]; gate_act 0: sigmoid(g), 1: SiLU, g sigmoid(g).
+// With `low` (float32 rows of stride ldg, `rank` numbers each) g is made here, g[t, i] = w_up[i] . low[t], the numbers rounded to bfloat16 as a
+// product's rows are: the form for a few rows.
 template <typename TW, typename TO>
 __global__ __launch_bounds__(64) void head_norm_gate_kernel(const float* __restrict__ o, long ldo, const float* __restrict__ den,
                                                            const float* __restrict__ g, long ldg, const TW* __restrict__ w,
-                                                           TO* __restrict__ y, long ldy, int n_heads, int dv, float eps, int w_head_stride, int gate_act) {
+                                                           TO* __restrict__ y, long ldy, int n_heads, int dv, float eps, int w_head_stride, int gate_act,
+                                                           const float* __restrict__ low, int rank, const bf16_t* __restrict__ w_up) {
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const float* orow = o + (size_t)t * ldo + (size_t)h * dv;
     const float by = den ? den[(size_t)t * n_heads + h] : 1.0f;
@@ -222,7 +225,16 @@ __global__ __launch_bounds__(64) void head_norm_gate_kernel(const float* __restr
     const float r = 1.0f / sqrtf(wave_sum(ss) / (float)dv + eps);
     for (int d = lane; d < dv; d += 64) {
         const float v = den ? orow[d] / by : orow[d];
-        const float z = g[(size_t)t * ldg + (size_t)h * dv + d];
+        float z;
+        if (low) {
+            const float* l = low + (size_t)t * ldg;
+            const bf16_t* wz = w_up + ((size_t)h * dv + d) * rank;
+            z = 0.f;
+#pragma unroll 8
+            for (int i = 0; i < rank; ++i) z = fmaf(bf16_to_f32(f32_to_bf16(l[i])), bf16_to_f32(wz[i]), z);
+        } else {
+            z = g[(size_t)t * ldg + (size_t)h * dv + d];
+        }
         const float gate = (gate_act ? z : 1.0f) / (1.0f + expf(-z));
         store_f32(y, (size_t)t * ldy + (size_t)h * dv + d, load_f32(w, (size_t)h * w_head_stride + d) * (v * r) * gate);
     }
@@ -248,21 +260,36 @@ __device__ __forceinline__ int rows_before(const int* __restrict__ slot, const i
 //   items 2 n_kv .. + n_heads a value head: convolution, SiLU
 //   the last item             per head the decay exp(-exp(a_log) softplus(pre_a + dt_bias)) and the step size sigmoid(pre_b)
 // qkv: float32 [rows, n_conv] in the columns' order; gates: float32 [rows, 2 n_heads], decays then step sizes.
+// With decays per channel (dn = dk numbers a head, else 1) there are n_heads last items, one per head, and gates is [rows, n_heads dk +
+// n_heads].  pre_a [rows, lda] holds the heads' dn numbers; or, with `low` (bfloat16 weights w_up [n_heads dn][rank] on the numbers
+// low [rows, rank], which are rounded to bfloat16 as a product's rows are), pre_a is made here: the form for a few rows.
 // move_tail: every row of the step is its request's only one (a decode step); the thread that has read a channel's tail then also
 // moves it on by the row's own input, and no other kernel needs to (with several rows of a request in a step, rows read the tail
 // that others would be writing: `delta_tail_kernel` does it behind this one).
-__global__ __launch_bounds__(64) void delta_prepare_kernel(const float* __restrict__ proj, long ld, int conv_off, int a_off, int b_off,
+__global__ __launch_bounds__(64) void delta_prepare_kernel(const float* __restrict__ proj, long ld, int conv_off, const float* __restrict__ pre_a, long lda, int b_off,
                                                           const float* __restrict__ taps, int n_taps, float* __restrict__ tail, long tail_stride, int move_tail,
                                                           const float* __restrict__ a_log, const float* __restrict__ dt_bias,
                                                           const int* __restrict__ slot, const int* __restrict__ pos, float* __restrict__ qkv,
-                                                          float* __restrict__ gates, int n_heads, int n_kv, int dk, int dv, float q_scale) {
+                                                          float* __restrict__ gates, int n_heads, int n_kv, int dk, int dv, float q_scale, int dn,
+                                                          const float* __restrict__ low, int rank, const bf16_t* __restrict__ w_up) {
     const int t = blockIdx.x, item = blockIdx.y, lane = threadIdx.x;
-    if (item == 2 * n_kv + n_heads) {
-        for (int h = lane; h < n_heads; h += 64) {
-            const float pre_a = proj[(size_t)t * ld + a_off + h], pre_b = proj[(size_t)t * ld + b_off + h];
-            gates[(size_t)t * 2 * n_heads + h] = expf(-expf(a_log[h]) * softplus_f(pre_a + dt_bias[h]));
-            gates[(size_t)t * 2 * n_heads + n_heads + h] = 1.0f / (1.0f + expf(-pre_b));
+    if (item >= 2 * n_kv + n_heads) {
+        const int h0 = dn > 1 ? item - 2 * n_kv - n_heads : 0, h1 = dn > 1 ? h0 + 1 : n_heads;
+        float* out = gates + (size_t)t * n_heads * (dn + 1);
+        for (int i = h0 * dn + lane; i < h1 * dn; i += 64) {
+            float a;
+            if (low) {
+                a = 0.f;
+                const float* l = low + (size_t)t * ld;
+                const bf16_t* w = w_up + (size_t)i * rank;
+#pragma unroll 8
+                for (int r = 0; r < rank; ++r) a = fmaf(bf16_to_f32(f32_to_bf16(l[r])), bf16_to_f32(w[r]), a);
+            } else {
+                a = pre_a[(size_t)t * lda + i];
+            }
+            out[i] = expf(-expf(a_log[i / dn]) * softplus_f(a + dt_bias[i]));
         }
+        for (int h = h0 + lane; h < h1; h += 64) out[n_heads * dn + h] = 1.0f / (1.0f + expf(-proj[(size_t)t * ld + b_off + h]));
         return;
     }
     const int n_conv = 2 * n_kv * dk + n_heads * dv;
@@ -325,7 +352,48 @@ __global__ __launch_bounds__(256) void delta_tail_kernel(const float* __restrict
 // updated behind them, and a token's chain of dependent steps is one pass and one reduction, not two of each.  Every sum over the
 // key's rows is the lanes' own shares in a fixed order, then the 16 groups by lane moves: the bits do not depend on the cut.
 // Key and query of a block of tokens wait in LDS; the block after it is asked for while this one is worked on.
-template <int ROWS>
+// CHANNEL: the decay is a number per key channel, so the sums are taken over D M, whose rows the decays have scaled already:
+//     e = s (v - (D M)^T k),   y = (D M)^T q + e (k . q).
+// A row of a token in LDS is then {k, q, d, k q} (two such numbers, {k, q}, otherwise).
+template <bool CHANNEL>
+struct DeltaItem { typedef float2 type; };
+template <>
+struct DeltaItem<true> { typedef float4 type; };
+__device__ __forceinline__ float2 delta_item(float2*, float k, float q, float) { return float2{k, q}; }
+__device__ __forceinline__ float4 delta_item(float4*, float k, float q, float d) { return float4{k, q, d, k * q}; }
+
+// One token for one lane's rows of a column: the memory moves on, the column's read-out comes back (in every lane of the column).
+template <int ROWS, bool CHANNEL>
+__device__ __forceinline__ float delta_token(float (&S)[ROWS], const typename DeltaItem<CHANNEL>::type (&x)[ROWS], float v, float decay, float step) {
+    float sk = 0.f, sq = 0.f, kq = 0.f;
+#pragma unroll
+    for (int rr = 0; rr < ROWS; ++rr) {
+        if constexpr (CHANNEL) {
+            S[rr] *= x[rr].z;
+            kq += x[rr].w;
+        } else {
+            kq = fmaf(x[rr].x, x[rr].y, kq);
+        }
+        sk = fmaf(S[rr], x[rr].x, sk);
+        sq = fmaf(S[rr], x[rr].y, sq);
+    }
+    sk = group_sum<16>(sk);
+    sq = group_sum<16>(sq);
+    kq = group_sum<16>(kq);
+    if constexpr (CHANNEL) {
+        const float w = step * (v - sk);
+#pragma unroll
+        for (int rr = 0; rr < ROWS; ++rr) S[rr] = fmaf(x[rr].x, w, S[rr]);
+        return fmaf(w, kq, sq);
+    } else {
+        const float w = step * (v - decay * sk);               // s (v - d M^T k)
+#pragma unroll
+        for (int rr = 0; rr < ROWS; ++rr) S[rr] = fmaf(decay, S[rr], x[rr].x * w);
+        return fmaf(decay, sq, w * kq);
+    }
+}
+
+template <int ROWS, bool CHANNEL>
 __global__ __launch_bounds__(64) void delta_scan_kernel(const float* __restrict__ qkv, long ld, const float* __restrict__ gates,
                                                        const int* __restrict__ seg_start, const int* __restrict__ seg_len,
                                                        const int* __restrict__ row_slot, float* __restrict__ state, long state_stride,
@@ -334,7 +402,8 @@ __global__ __launch_bounds__(64) void delta_scan_kernel(const float* __restrict_
     constexpr int TB = (1024 / KQ) < 16 ? (1024 / KQ) : 16;      // tokens staged at a time
     constexpr int PER = TB * KQ / 64;            // (k, q) pairs a lane brings per block
     static_assert(TB >= 2 && TB * C <= 64, "a block of 2 to 16 tokens; a lane brings one value and one pair of gates");
-    __shared__ float2 kq_s[2][TB][KQ];
+    typedef typename DeltaItem<CHANNEL>::type item_t;
+    __shared__ item_t kq_s[2][TB][KQ];
     __shared__ float v_s[2][TB][C];
     __shared__ float2 gb_s[2][TB];
     const int seg = blockIdx.x, h = blockIdx.y, vt = blockIdx.z, n_tiles = gridDim.z;
@@ -354,21 +423,25 @@ __global__ __launch_bounds__(64) void delta_scan_kernel(const float* __restrict_
         S[rr] = i < dk ? st[(size_t)i * C + c] : 0.f;
     }
     // A block of TB tokens from `first` on (rows beyond the request's last are read as its last: finite, and never used).
-    float2 kq_reg[PER], gb_reg;
+    const int dn = CHANNEL ? dk : 1;             // decays a head
+    const size_t ldg = (size_t)n_heads * (dn + 1);
+    item_t kq_reg[PER];
+    float2 gb_reg;
     float v_reg;
     auto fetch = [&](int first) {
 #pragma unroll
         for (int e = 0; e < PER; ++e) {
             const int idx = lane + 64 * e, u = idx / KQ, i = idx % KQ;
-            const float* row = qkv + (size_t)(t0 + min(first + u, n - 1)) * ld;
+            const size_t t = t0 + min(first + u, n - 1);
+            const float* row = qkv + t * ld;
             const int ic = min(i, dk - 1);
-            const float kk = row[k_at + ic], qq = row[q_at + ic];
-            kq_reg[e] = i < dk ? float2{kk, qq} : float2{0.f, 0.f};
+            const float kk = row[k_at + ic], qq = row[q_at + ic], dd = CHANNEL ? gates[t * ldg + h * dk + ic] : 0.f;
+            kq_reg[e] = i < dk ? delta_item((item_t*)nullptr, kk, qq, dd) : item_t{};
         }
         const int u = min(lane / C, TB - 1), cc = min(vt * C + lane % C, dv - 1);
         v_reg = qkv[(size_t)(t0 + min(first + u, n - 1)) * ld + v_at + cc];
-        const float* g = gates + (size_t)(t0 + min(first + min(lane, TB - 1), n - 1)) * 2 * n_heads;
-        gb_reg = float2{g[h], g[n_heads + h]};
+        const float* g = gates + (size_t)(t0 + min(first + min(lane, TB - 1), n - 1)) * ldg;
+        gb_reg = float2{CHANNEL ? 0.f : g[h], g[n_heads * dn + h]};
     };
     auto stash = [&](int buf) {
 #pragma unroll
@@ -389,27 +462,51 @@ __global__ __launch_bounds__(64) void delta_scan_kernel(const float* __restrict_
         if (more) fetch(b0 + TB);
         for (int u = 0; u < here; ++u) {
             const float2 gb = gb_s[buf][u];
-            float kx[ROWS];
-            float sk = 0.f, sq = 0.f, kq = 0.f;
+            item_t x[ROWS];
 #pragma unroll
-            for (int rr = 0; rr < ROWS; ++rr) {
-                const float2 pair = kq_s[buf][u][rr * RG + rg];
-                kx[rr] = pair.x;
-                sk = fmaf(S[rr], pair.x, sk);
-                sq = fmaf(S[rr], pair.y, sq);
-                kq = fmaf(pair.x, pair.y, kq);
-            }
-            sk = group_sum<RG>(sk);
-            sq = group_sum<RG>(sq);
-            kq = group_sum<RG>(kq);
-            const float w = gb.y * (v_s[buf][u][c] - gb.x * sk);       // s (v - d M^T k)
-#pragma unroll
-            for (int rr = 0; rr < ROWS; ++rr) S[rr] = fmaf(gb.x, S[rr], kx[rr] * w);
-            if (rg == 0 && live) out[(size_t)(t0 + b0 + u) * ldo + h * dv + col] = fmaf(gb.x, sq, w * kq);
+            for (int rr = 0; rr < ROWS; ++rr) x[rr] = kq_s[buf][u][rr * RG + rg];
+            const float y = delta_token<ROWS, CHANNEL>(S, x, v_s[buf][u][c], gb.x, gb.y);
+            if (rg == 0 && live) out[(size_t)(t0 + b0 + u) * ldo + h * dv + col] = y;
         }
         if (more) stash(buf ^ 1);                // (the buffer the block before this one was read from)
         barrier_lds();
     }
+#pragma unroll
+    for (int rr = 0; rr < ROWS; ++rr) {
+        const int i = rr * RG + rg;
+        if (i < dk) st[(size_t)i * C + c] = S[rr];
+    }
+}
+
+// The same for steps in which every request brings one row: nothing is staged, a wave takes its row's numbers as they lie, and a
+// workgroup is four waves (tiles).  Every sum in the scan's order: the same bits.
+template <int ROWS, bool CHANNEL>
+__global__ __launch_bounds__(256) void delta_single_kernel(const float* __restrict__ qkv, long ld, const float* __restrict__ gates,
+                                                          const int* __restrict__ seg_start, const int* __restrict__ seg_len,
+                                                          const int* __restrict__ row_slot, float* __restrict__ state, long state_stride,
+                                                          float* __restrict__ out, long ldo, int n_heads, int n_kv, int dk, int dv) {
+    constexpr int C = 4, RG = 16;
+    typedef typename DeltaItem<CHANNEL>::type item_t;
+    const int seg = blockIdx.x, h = blockIdx.y, vt = blockIdx.z * 4 + (threadIdx.x >> 6), n_tiles = (dv + C - 1) / C;
+    const int lane = threadIdx.x & 63, c = lane / RG, rg = lane % RG;
+    if (vt >= n_tiles || seg_len[seg] <= 0) return;
+    const size_t t = seg_start[seg];
+    const int col = vt * C + c, kvh = h / (n_heads / n_kv), dn = CHANNEL ? dk : 1;
+    float* st = state + (size_t)row_slot[t] * state_stride + ((size_t)h * n_tiles + vt) * ((size_t)dk * C);
+    const float* row = qkv + t * ld;
+    const float* g = gates + t * n_heads * (dn + 1);
+    float S[ROWS];
+    item_t x[ROWS];
+#pragma unroll
+    for (int rr = 0; rr < ROWS; ++rr) {
+        const int i = rr * RG + rg, ic = min(i, dk - 1);
+        const float s = st[(size_t)ic * C + c], k = row[(n_kv + kvh) * dk + ic], q = row[kvh * dk + ic], d = CHANNEL ? g[h * dk + ic] : 0.f;
+        S[rr] = i < dk ? s : 0.f;
+        x[rr] = i < dk ? delta_item((item_t*)nullptr, k, q, d) : item_t{};
+    }
+    const float v = row[2 * n_kv * dk + h * dv + min(col, dv - 1)];
+    const float y = delta_token<ROWS, CHANNEL>(S, x, v, CHANNEL ? 0.f : g[h], g[n_heads * dn + h]);
+    if (rg == 0 && col < dv) out[t * ldo + h * dv + col] = y;
 #pragma unroll
     for (int rr = 0; rr < ROWS; ++rr) {
         const int i = rr * RG + rg;
@@ -463,19 +560,23 @@ GI_API int gi_delta_max_key_dim() { return 512; }
 GI_API int gi_delta_max_taps() { return DELTA_MAX_TAPS; }
 
 // proj: float32 [n_rows, ld]; see delta_prepare_kernel.  state: [slots, state_stride], a slot's memories then its tail.
-GI_API int gi_delta_prepare(const float* proj, long ld, int conv_off, int a_off, int b_off, const float* taps, int n_taps, const float* a_log,
+// pre_a: float32 [n_rows, lda], the decays' pre-activations, one a head, or (channel != 0) one a head and key channel; or low: float32 rows
+// of proj's stride with `rank` numbers each, and w_up bfloat16 [heads or heads*dk][rank], from which they are made here.
+GI_API int gi_delta_prepare(const float* proj, long ld, int conv_off, const float* pre_a, long lda, int b_off, const float* taps, int n_taps, const float* a_log,
                             const float* dt_bias, const int* slot, const int* pos, float* state, long state_stride, float* qkv, float* gates,
-                            int n_rows, int n_heads, int n_kv, int dk, int dv, float q_scale, int move_tail, hipStream_t stream) {
+                            int n_rows, int n_heads, int n_kv, int dk, int dv, float q_scale, int move_tail, int channel, const float* low, int rank, const void* w_up,
+                            hipStream_t stream) {
+    const int dn = channel ? dk : 1;
     GI_REQUIRE(n_rows > 0 && n_heads > 0 && n_kv > 0 && n_heads % n_kv == 0 && dk > 0 && dv > 0, "delta_prepare: bad sizes (rows %d, heads %d, kv heads %d, dk %d, dv %d)",
                n_rows, n_heads, n_kv, dk, dv);
     GI_REQUIRE(n_taps >= 1 && n_taps <= DELTA_MAX_TAPS, "delta_prepare: %d taps, 1 to %d are served", n_taps, DELTA_MAX_TAPS);
     const long n_conv = 2L * n_kv * dk + (long)n_heads * dv;
-    GI_REQUIRE(conv_off >= 0 && a_off >= 0 && b_off >= 0 && ld >= conv_off + n_conv && ld >= a_off + n_heads && ld >= b_off + n_heads,
-               "delta_prepare: the columns named lie outside the rows");
-    GI_REQUIRE(state_stride >= gi_delta_state_floats(n_heads, n_kv, dk, dv, n_taps) && 2 * n_kv + n_heads + 1 <= 65535, "delta_prepare: state stride %ld too small, or too many heads", state_stride);
-    dim3 grid(n_rows, 2 * n_kv + n_heads + 1);
-    delta_prepare_kernel<<<grid, 64, 0, stream>>>(proj, ld, conv_off, a_off, b_off, taps, n_taps, state + gi_delta_memory_floats(n_heads, dk, dv), state_stride, move_tail,
-                                                  a_log, dt_bias, slot, pos, qkv, gates, n_heads, n_kv, dk, dv, q_scale);
+    GI_REQUIRE(conv_off >= 0 && b_off >= 0 && ld >= conv_off + n_conv && ld >= b_off + n_heads, "delta_prepare: the columns named lie outside the rows");
+    GI_REQUIRE(low != nullptr ? (rank > 0 && w_up != nullptr) : (pre_a != nullptr && lda >= (long)n_heads * dn), "delta_prepare: the decays' inputs are missing or too short");
+    GI_REQUIRE(state_stride >= gi_delta_state_floats(n_heads, n_kv, dk, dv, n_taps) && 2 * n_kv + 2 * n_heads <= 65535, "delta_prepare: state stride %ld too small, or too many heads", state_stride);
+    dim3 grid(n_rows, 2 * n_kv + n_heads + (dn > 1 ? n_heads : 1));
+    delta_prepare_kernel<<<grid, 64, 0, stream>>>(proj, ld, conv_off, pre_a, lda, b_off, taps, n_taps, state + gi_delta_memory_floats(n_heads, dk, dv), state_stride, move_tail,
+                                                  a_log, dt_bias, slot, pos, qkv, gates, n_heads, n_kv, dk, dv, q_scale, dn, low, rank, (const bf16_t*)w_up);
     GI_CHECK_LAUNCH("delta_prepare");
     return 0;
 }
@@ -491,30 +592,40 @@ GI_API int gi_delta_tail(const float* proj, long ld, int conv_off, int n_taps, c
     return 0;
 }
 
-// qkv: float32 [n_rows, ld], a row's unit queries [n_kv][dk], unit keys [n_kv][dk], values [n_heads][dv]; gates: float32 [n_rows, 2 n_heads];
+// qkv: float32 [n_rows, ld], a row's unit queries [n_kv][dk], unit keys [n_kv][dk], values [n_heads][dv]; gates: float32 [n_rows, 2 n_heads],
+// or [n_rows, n_heads dk + n_heads] with a decay per head and key channel (channel != 0);
 // out: float32 [n_rows, ldo] gets the heads' read-outs [n_heads][dv].
 GI_API int gi_delta_scan(const float* qkv, long ld, const float* gates, const int* seg_start, const int* seg_len, int n_segs, const int* row_slot,
-                         float* state, long state_stride, float* out, long ldo, int n_heads, int n_kv, int dk, int dv, hipStream_t stream) {
+                         float* state, long state_stride, float* out, long ldo, int n_heads, int n_kv, int dk, int dv, int channel, int single, hipStream_t stream) {
     GI_REQUIRE(n_segs > 0 && n_heads > 0 && n_kv > 0 && n_heads % n_kv == 0 && dk > 0 && dk <= 512 && dv > 0, "delta_scan: bad sizes (runs %d, heads %d, kv heads %d, dk %d, dv %d; dk at most 512)",
                n_segs, n_heads, n_kv, dk, dv);
     GI_REQUIRE(ld >= 2L * n_kv * dk + (long)n_heads * dv && ldo >= (long)n_heads * dv && state_stride >= gi_delta_memory_floats(n_heads, dk, dv), "delta_scan: row or state strides too small");
     const int tiles = (dv + 3) / 4;
     GI_REQUIRE(n_heads <= 65535 && tiles <= 65535, "delta_scan: too many heads or value channels");
     dim3 grid(n_segs, n_heads, tiles);
-#define GO(R) delta_scan_kernel<R><<<grid, 64, 0, stream>>>(qkv, ld, gates, seg_start, seg_len, row_slot, state, state_stride, out, ldo, n_heads, n_kv, dk, dv)
+#define ARGS qkv, ld, gates, seg_start, seg_len, row_slot, state, state_stride, out, ldo, n_heads, n_kv, dk, dv
+#define GO(R)                                                                                                \
+    do {                                                                                                     \
+        if (single && channel) delta_single_kernel<R, true><<<dim3(n_segs, n_heads, (tiles + 3) / 4), 256, 0, stream>>>(ARGS);       \
+        else if (single) delta_single_kernel<R, false><<<dim3(n_segs, n_heads, (tiles + 3) / 4), 256, 0, stream>>>(ARGS);            \
+        else if (channel) delta_scan_kernel<R, true><<<grid, 64, 0, stream>>>(ARGS);                         \
+        else delta_scan_kernel<R, false><<<grid, 64, 0, stream>>>(ARGS);                                     \
+    } while (0)
     if (dk <= 32) GO(2); else if (dk <= 64) GO(4); else if (dk <= 128) GO(8); else if (dk <= 256) GO(16); else GO(32);
 #undef GO
+#undef ARGS
     GI_CHECK_LAUNCH("delta_scan");
     return 0;
 }
 
 GI_API int gi_head_norm_gate(const float* o, long ldo, const float* den, const float* g, long ldg, const void* w, int w_dtype, void* y, int y_dtype, long ldy, int n_rows,
-                             int n_heads, int dv, float eps, int shared_weight, int gate_act, hipStream_t stream) {
+                             int n_heads, int dv, float eps, int shared_weight, int gate_act, const float* low, int rank, const void* w_up, hipStream_t stream) {
+    GI_REQUIRE(low != nullptr ? (rank > 0 && w_up != nullptr && ldg >= rank) : g != nullptr, "head_norm_gate: the gates' inputs are missing");
     GI_REQUIRE(n_rows > 0 && n_heads > 0 && n_heads <= 65535 && dv > 0, "head_norm_gate: bad sizes (rows %d, heads %d, dv %d)", n_rows, n_heads, dv);
     GI_REQUIRE(gate_act == 0 || gate_act == 1, "head_norm_gate: the gate is a sigmoid (0) or SiLU (1)");
     dim3 grid(n_rows, n_heads);
     const int w_head_stride = shared_weight ? 0 : dv;
-#define GO(TW, TO) head_norm_gate_kernel<TW, TO><<<grid, 64, 0, stream>>>(o, ldo, den, g, ldg, (const TW*)w, (TO*)y, ldy, n_heads, dv, eps, w_head_stride, gate_act)
+#define GO(TW, TO) head_norm_gate_kernel<TW, TO><<<grid, 64, 0, stream>>>(o, ldo, den, g, ldg, (const TW*)w, (TO*)y, ldy, n_heads, dv, eps, w_head_stride, gate_act, low, rank, (const bf16_t*)w_up)
     if (w_dtype == GI_F32 && y_dtype == GI_F32) GO(float, float);
     else if (w_dtype == GI_F32 && y_dtype == GI_BF16) GO(float, bf16_t);
     else if (w_dtype == GI_BF16 && y_dtype == GI_BF16) GO(bf16_t, bf16_t);

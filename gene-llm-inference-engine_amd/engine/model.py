@@ -57,6 +57,13 @@ class DecoderModel:
         self.head = _Head(self.lm_head, self.head_in_dtype)
         self.after_embedding = [row_transform_class(t)(t, tensors, dtype, device) for t in spec.after_embedding]
         self.after_head = [row_transform_class(t)(t, tensors, dtype, device) for t in spec.after_head]
+        if any(t.fetches_token_rows for t in self.after_embedding[1:]):
+            raise ValueError("a transform that fetches the token rows itself must be the first one behind the token table")
+        # those of them that keep a state per request: theirs follows the run order's in the list of cache needs
+        self.transform_entry = {}
+        for t in spec.after_embedding:
+            if row_transform_class(t).cache_need(t) is not None:
+                self.transform_entry[t] = len(spec.run_order) + len(self.transform_entry)
         # the longest sequence the parts behind the token table allow (a table of positions ends somewhere), or None
         self.position_limit = min((t.position_limit for t in self.after_embedding if getattr(t, "position_limit", None) is not None), default=None)
         self.run_order = spec.run_order
@@ -75,9 +82,11 @@ class DecoderModel:
 
     # ----------------------------------------------------------------------------- what it needs
     def cache_needs(self):
-        """Per run-order entry: its cache need, and the entry whose cache it reads (or None)."""
+        """Per run-order entry: its cache need, and the entry whose cache it reads (or None); then the needs of what keeps a state behind
+        the token table."""
         needs = [block_class(self.spec.layers[e.layer].block).cache_need(self.spec.layers[e.layer]) for e in self.run_order]
-        return needs, [e.cache_of for e in self.run_order]
+        needs += [row_transform_class(t).cache_need(t) for t in self.transform_entry]
+        return needs, [e.cache_of for e in self.run_order] + [None] * len(self.transform_entry)
 
     def weight_bytes_read_per_step(self) -> int:
         """Bytes of weights one step reads when it uses every matrix once: what every part of the run order holds (a
@@ -92,19 +101,23 @@ class DecoderModel:
         [n_logit_rows, vocab] of the rows listed in `logit_rows`, or None if there are none."""
         x = torch.empty((ctx.n_rows, self.spec.hidden_size), dtype=torch.float32, device=self.device)
         trace = self.trace
-        handed = self._embed(ctx, x)      # the next block's first norm, where whoever wrote x could leave it half applied
+        handed = self._embed(ctx, x, cache)      # the next block's first norm, where whoever wrote x could leave it half applied
         if trace is not None:
             trace("embedding", -1, x)
-        if self.keeps_token_rows:
+        if self.keeps_token_rows and "token_rows" not in ctx.memo:
             ctx.memo["token_rows"] = x.clone()
         if self.n_streams > 1:            # every copy starts as the token rows
             x = ops.streams_spread(x, torch.empty((ctx.n_rows, self.n_streams * self.spec.hidden_size), dtype=torch.float32, device=self.device), self.n_streams)
         for i, entry in enumerate(self.run_order):
             ctx.trace = None if trace is None else (lambda tag, rows, i=i: trace(tag, i, rows))
             layer, extras = self.layers[entry.layer], self.after_layer[entry.layer]
-            if self.before_entry[i] is not None:          # (it changes x: a norm handed on by whoever wrote x last is void)
-                self.before_entry[i].forward(x, ctx)
-                handed = None
+            before = self.before_entry[i]
+            if before is not None:                        # (it changes x: a norm handed on by whoever wrote x last is void)
+                if getattr(before, "hands_norm_on", False):
+                    handed = before.forward(x, ctx, handed=None, next_reader=self._first_reader(layer))
+                else:
+                    before.forward(x, ctx)
+                    handed = None
             if i + 1 == len(self.run_order):              # the head reads every row of the final norm, or a selection, which is not handed on
                 behind = (self.final_norm, self.head) if ctx.every_row_wanted and trace is None else None
             elif self.before_entry[i + 1] is not None:    # (x changes again before anybody reads it)
@@ -147,7 +160,7 @@ class DecoderModel:
     def _first_reader(stage):
         return stage.first_reader() if getattr(stage, "hands_norm_on", False) else None
 
-    def _embed(self, ctx: StepContext, x: torch.Tensor):
+    def _embed(self, ctx: StepContext, x: torch.Tensor, cache):
         """The rows of the token table into x.  Where the first block's first norm can be taken half applied (`HandedRows`: a few
         single rows of decoding requests in bfloat16, a norm of the form g * x * rsqrt(mean square + eps), a reader whose product
         finishes it), the kernel that fetches the rows does the norm's first half too and the `HandedRows` are returned; None otherwise."""
@@ -171,7 +184,14 @@ class DecoderModel:
                 low = torch.empty(x.shape, dtype=torch.bfloat16, device=self.device)
             ops.embed_positioned(self.embedding, ctx.tokens, math.prod(float(t.spec.factor) for t in transforms[:-1]), transforms[-1].table, ctx.row_pos, x, low)
             return None if low is None else ReadyRows(norm, x, low)
-        ops.embed(self.embedding, ctx.tokens, x)
+        if transforms and transforms[0].fetches_token_rows:
+            entry = self.transform_entry.get(transforms[0].spec)
+            if self.keeps_token_rows and len(transforms) == 1:
+                ctx.memo["token_rows"] = torch.empty_like(x)          # (the same kernel writes both)
+            transforms[0].fetch(self.embedding, x, ctx, None if entry is None else cache.layer_cache(entry), ctx.memo.get("token_rows"))
+            transforms = transforms[1:]
+        else:
+            ops.embed(self.embedding, ctx.tokens, x)
         for transform in transforms:
             if transform.needs_context:
                 transform(x, ctx)

@@ -51,27 +51,32 @@ _SIGNATURES = {
     "gi_ssm_tail": [c_void_p, c_long, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_long, c_int, c_int, c_void_p],
     "gi_ssm_scan": [c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_long, c_int, c_int, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p,
                     c_void_p, c_long, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_float, c_void_p, c_long, c_int, c_int, c_int, c_void_p],
-    "gi_route_top": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_void_p, c_void_p],
-    "gi_experts_gate_up": [c_void_p, c_int, c_long, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p],
-    "gi_route_rows": [c_void_p, c_int, c_long, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_void_p, c_void_p, c_long, c_int, c_void_p, c_long,
+    "gi_route_top": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p],
+    "gi_experts_gate_up": [c_void_p, c_int, c_long, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p],
+    "gi_route_rows": [c_void_p, c_int, c_long, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_long, c_int, c_void_p, c_long,
                       c_void_p],
     "gi_experts_place": [c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p],
-    "gi_experts_gather": [c_void_p, c_long, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_long, c_int, c_void_p],
-    "gi_experts_combine": [c_void_p, c_long, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_long, c_int, c_int, c_void_p],
+    "gi_experts_gather": [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_long, c_int, c_int, c_void_p],
+    "gi_experts_combine": [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_long, c_int, c_int, c_void_p, c_long, c_int, c_void_p, c_void_p, c_int, c_float,
+                           c_void_p, c_long, c_void_p],
+    "gi_layernorm": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_float, c_long, c_long, c_long, c_void_p],
+    "gi_embed_pairs": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_long, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p],
+    "gi_latent_direct": [c_void_p, c_long, c_void_p, c_long, c_void_p, c_int, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_long, c_void_p, c_long,
+                         c_void_p, c_int, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "gi_gemm_bf16_grouped": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_float, c_int, c_int, c_int, c_long, c_long, c_long, c_void_p, c_long, c_void_p],
-    "gi_experts_down": [c_void_p, c_int, c_long, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p],
+    "gi_experts_down": [c_void_p, c_int, c_long, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int, c_long, c_int, c_void_p],
     "gi_xielu": [c_void_p, c_long, c_void_p, c_int, c_long, c_int, c_int, c_void_p, c_void_p],
-    "gi_delta_prepare": [c_void_p, c_long, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p,
-                         c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p],
+    "gi_delta_prepare": [c_void_p, c_long, c_int, c_void_p, c_long, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p,
+                         c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p],
     "gi_delta_tail": [c_void_p, c_long, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_long, c_int, c_int, c_int, c_int, c_void_p],
-    "gi_delta_scan": [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_long, c_void_p, c_long, c_int, c_int, c_int, c_int, c_void_p],
+    "gi_delta_scan": [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_long, c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "gi_latent_prepare": [c_void_p, c_long, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
-                          c_void_p, c_int, c_long, c_void_p, c_int, c_long, c_int, c_int, c_void_p],
-    "gi_heads_product": [c_void_p, c_long, c_void_p, c_void_p, c_int, c_long, c_long, c_int, c_int, c_int, c_int, c_void_p],
+                          c_void_p, c_int, c_long, c_void_p, c_int, c_long, c_int, c_int, c_int, c_void_p],
+    "gi_heads_product": [c_void_p, c_long, c_void_p, c_void_p, c_int, c_long, c_long, c_int, c_int, c_int, c_int, c_void_p, c_long, c_void_p],
     "gi_latent_attention_bf16": [c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int, c_int, c_int,
-                                 c_float, c_int, c_void_p],
-    "gi_latent_attention_tiles_bf16": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p],
-    "gi_latent_queries": [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_long, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p],
+                                 c_float, c_int, c_void_p, c_void_p],
+    "gi_latent_attention_tiles_bf16": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p, c_void_p],
+    "gi_latent_queries": [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_long, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "gi_act_mul": [c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_float, c_void_p],
     "gi_streams_spread": [c_void_p, c_long, c_void_p, c_long, c_int, c_int, c_int, c_void_p],
     "gi_streams_norm_shift": [c_void_p, c_long, c_int, c_int, c_void_p, c_void_p, c_int, c_float, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_long,
@@ -89,7 +94,7 @@ _SIGNATURES = {
     "gi_segments": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p],
     "gi_mlstm_scan": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_float, c_float, c_void_p, c_void_p, c_int, c_void_p,
                       c_void_p, c_long, c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_void_p],
-    "gi_head_norm_gate": [c_void_p, c_long, c_void_p, c_void_p, c_long, c_void_p, c_int, c_void_p, c_int, c_long, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p],
+    "gi_head_norm_gate": [c_void_p, c_long, c_void_p, c_void_p, c_long, c_void_p, c_int, c_void_p, c_int, c_long, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p],
     "gi_gemm_bf16": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_int, c_int, c_int, c_long, c_long, c_long, c_void_p, c_long, c_void_p],
     "gi_attention_prompt_bf16": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int, c_int,
                                  c_float, c_int, c_void_p, c_void_p, c_int, c_void_p, c_long, c_int, c_void_p, c_void_p, c_long, c_int, c_float, c_void_p],
@@ -153,6 +158,8 @@ def lib():
         l.gi_latent_attention_tiles_prepare.restype = c_int
         l.gi_streams_write_norm_takes.argtypes = [c_int, c_int]
         l.gi_streams_write_norm_takes.restype = c_int
+        l.gi_experts_combine_norm_takes.argtypes = [c_int]
+        l.gi_experts_combine_norm_takes.restype = c_int
         l.gi_streams_max.argtypes = []
         l.gi_streams_max.restype = c_int
         l.gi_probe_mfma_flops.argtypes = [c_int, c_int]
@@ -326,6 +333,54 @@ def embed_positioned(table, tokens, scale, where, positions, x, low=None):
     _call("gi_embed_positioned", _ptr(table), _code(table, "embed_positioned: table") if table is not None else F32, _ptr(tokens), float(scale), where.data_ptr(),
           _code(where, "embed_positioned: positions"), where.shape[0], positions.data_ptr(), x.data_ptr(), _ptr(low), n, dim, _stream())
     return x
+
+
+def embed_pairs(table, pairs, tokens, positions, slots, segments, last, mul_before, mul_token, x, keep=None):
+    """x[t] = table[token] + pairs[(before * mul_before + token * mul_token) mod buckets] with pairs [buckets + 1, dim] and `before` the
+    token of the request's row before (the step's previous row, or what `last` int32 [slots, 1] holds of the request); a row at position
+    0 takes pairs' last row.  `last` gets every request's last token of the step.  segments: (first row, rows) of the step's requests
+    (`segments(ctx)`).  keep: float32 [n, dim] that gets the same rows, or None."""
+    _dev(table, pairs, tokens, positions, slots, *segments, last, x, keep)
+    n, dim = x.shape
+    if not (table.dim() == 2 and table.shape[1] == dim and table.is_contiguous() and pairs.dim() == 2 and pairs.shape[1] == dim and pairs.shape[0] >= 2 and pairs.is_contiguous()
+            and pairs.dtype == table.dtype):
+        raise KernelError("embed_pairs: the tables must be [entries, dim], contiguous, of one dtype")
+    if not all(t is None or (t.dtype == torch.float32 and t.shape == (n, dim) and t.is_contiguous()) for t in (x, keep)):
+        raise KernelError("embed_pairs: the rows must be float32 [n, dim], contiguous")
+    if not (last.dtype == torch.int32 and last.dim() == 2 and last.shape[1] >= 1):
+        raise KernelError("embed_pairs: the requests' last tokens must be int32 [slots, 1]")
+    for t, what in ((tokens, "tokens"), (positions, "positions"), (slots, "slots")):
+        _i32(t, f"embed_pairs: {what}", n)
+    seg_start, seg_len = segments
+    n_segs, buckets = seg_start.numel(), pairs.shape[0] - 1
+    _i32(seg_start, "embed_pairs: seg_start", n_segs)
+    _i32(seg_len, "embed_pairs: seg_len", n_segs)
+    _call("gi_embed_pairs", table.data_ptr(), pairs.data_ptr(), _code(table, "embed_pairs: table"), tokens.data_ptr(), positions.data_ptr(), slots.data_ptr(), seg_start.data_ptr(),
+          seg_len.data_ptr(), n_segs, last.data_ptr(), last.stride(0), buckets, int(mul_before) % buckets, int(mul_token) % buckets, x.data_ptr(), _ptr(keep), n, dim, _stream())
+    return x
+
+
+def layernorm(x, weight, bias, eps, out, rows=None, add=None, vector=None):
+    """out = (v - mean) / sqrt(mean((v - mean)^2) + eps) * weight + bias per row of v = x (+ add) (+ vector), which is also written back to
+    x where something is added.  x float32 [n, dim]; add float32 [n, dim] and vector [dim] (of weight's dtype) or None; rows: int32
+    indices, out[i] = norm(x[rows[i]]).  weight, bias and out None: nothing but the sum."""
+    _dev(x, weight, bias, out, rows, add, vector)
+    dim = x.shape[1]
+    n = x.shape[0] if rows is None else rows.numel()
+    _f32_rows(x, "layernorm: x")
+    _f32_rows(add, "layernorm: the rows added", n, dim)
+    one = [v for v in (weight, bias, vector) if v is not None]
+    if not all(v.shape == (dim,) and v.is_contiguous() and v.dtype == one[0].dtype for v in one) or (weight is None) != (bias is None):
+        raise KernelError("layernorm: weight, bias and vector must be [dim], contiguous and of one dtype")
+    if weight is None:
+        out = None
+    elif not (out is not None and out.shape == (n, dim) and out.stride(1) == 1):
+        raise KernelError("layernorm: out must be [n, dim] with unit inner stride")
+    if rows is not None:
+        _i32(rows, "layernorm: rows", n)
+    _call("gi_layernorm", x.data_ptr(), _ptr(rows), _ptr(add), _ptr(vector), _ptr(weight), _ptr(bias), _code(one[0], "layernorm: weight") if one else F32, _ptr(out),
+          _code(out, "layernorm: out") if out is not None else F32, n, dim, float(eps), x.stride(0), add.stride(0) if add is not None else 0, out.stride(0) if out is not None else 0, _stream())
+    return out
 
 
 def add_position_rows(x, where, positions):
@@ -737,25 +792,41 @@ def mlstm_scan(proj, offsets, i_bias, f_bias, cap, q_scale, seg_start, seg_len, 
 GATES = {"sigmoid": 0, "silu": 1}
 
 
-def head_norm_gate(o, gate, weight, eps, out, n_heads, dv, den=None, gate_activation="sigmoid"):
+def _few_row_up(what, up, n_out):
+    """Of `up` = (low, w): float32 [n, rank] and bfloat16 [n_out, rank]: what a kernel that multiplies a few rows itself is told."""
+    if up is None:
+        return None, 0, 0, None
+    low, w = up
+    _dev(low, w)
+    _f32_rows(low, f"{what}: the narrow rows")
+    if not (w.dtype == torch.bfloat16 and w.shape == (n_out, low.shape[1]) and w.is_contiguous()):
+        raise KernelError(f"{what}: the product from the narrow rows needs bfloat16 [{n_out}, rank]")
+    return low.data_ptr(), low.stride(0), low.shape[1], w.data_ptr()
+
+
+def head_norm_gate(o, gate, weight, eps, out, n_heads, dv, den=None, gate_activation="sigmoid", gate_up=None):
     """out[t, h*dv + d] = weight[h*dv + d] * o[t, h, d] * rsqrt(mean over d of o[t, h, :]^2 + eps) * sigmoid(gate[t, h*dv + d]);
     o and gate float32 [n, heads*dv] (unit inner stride: columns of a wider product are fine).  den: float32 [n, heads]; o is
     then what the rows hold divided by den[t, h].  weight may be [dv] instead: one for all heads.  gate_activation "silu": the
-    last factor is gate * sigmoid(gate)."""
+    last factor is gate * sigmoid(gate).  gate None with gate_up = (low, w): gate = w low, made here (a few rows: low float32 [n, rank],
+    rounded to bfloat16 as a product's rows are, w bfloat16 [heads*dv, rank])."""
     _dev(o, gate, weight, out, den)
     n = o.shape[0]
     if den is not None and not (den.dtype == torch.float32 and den.shape == (n, n_heads) and den.is_contiguous()):
         raise KernelError("head_norm_gate: den must be float32 [n, heads], contiguous")
+    if (gate is None) == (gate_up is None):
+        raise KernelError("head_norm_gate: the gates, or what they are made of, must be given")
     for t, name in ((o, "o"), (gate, "gate")):
-        if not (t.dtype == torch.float32 and t.shape == (n, n_heads * dv) and t.stride(1) == 1):
+        if t is not None and not (t.dtype == torch.float32 and t.shape == (n, n_heads * dv) and t.stride(1) == 1):
             raise KernelError(f"head_norm_gate: {name} must be float32 [n, heads*dv]")
+    low, ld_low, rank, w_up = _few_row_up("head_norm_gate", gate_up, n_heads * dv)
     shared = weight.numel() == dv and n_heads > 1
     if not (weight.numel() in (n_heads * dv, dv) and weight.is_contiguous() and out.shape == (n, n_heads * dv) and out.stride(1) == 1):
         raise KernelError("head_norm_gate: weight must be [heads*dv] or [dv], and out [n, heads*dv]")
     if gate_activation not in GATES:
         raise KernelError(f"head_norm_gate: unknown gate {gate_activation!r}; known: {', '.join(GATES)}")
-    _call("gi_head_norm_gate", o.data_ptr(), o.stride(0), _ptr(den), gate.data_ptr(), gate.stride(0), weight.data_ptr(), _code(weight, "head_norm_gate: weight"),
-          out.data_ptr(), _code(out, "head_norm_gate: out"), out.stride(0), n, n_heads, dv, float(eps), 1 if shared else 0, GATES[gate_activation], _stream())
+    _call("gi_head_norm_gate", o.data_ptr(), o.stride(0), _ptr(den), _ptr(gate), gate.stride(0) if gate is not None else ld_low, weight.data_ptr(), _code(weight, "head_norm_gate: weight"),
+          out.data_ptr(), _code(out, "head_norm_gate: out"), out.stride(0), n, n_heads, dv, float(eps), 1 if shared else 0, GATES[gate_activation], low, rank, w_up, _stream())
     return out
 
 
@@ -843,32 +914,48 @@ def _delta_checks(what, proj, state, n_heads, n_kv, dk, dv, n_taps):
         raise KernelError(f"{what}: keys of 1 to {DELTA_MAX_KEY_DIM} channels, 1 to {DELTA_MAX_TAPS} taps and heads in whole groups are served")
 
 
-def delta_prepare(proj, conv_off, a_off, b_off, taps, a_log, dt_bias, ctx_slots, ctx_positions, state, qkv, gates, n_heads, n_kv, dk, dv, q_scale,
-                  single_rows=False):
+def delta_prepare(proj, conv_off, a, b_off, taps, a_log, dt_bias, ctx_slots, ctx_positions, state, qkv, gates, n_heads, n_kv, dk, dv, q_scale,
+                  single_rows=False, channel=False, a_up=None):
     """What the gated delta rule needs of every row (csrc/recurrent.hip: delta_prepare_kernel): the columns [conv_off, conv_off +
     2 n_kv dk + n_heads dv) of proj (queries, keys, values) through their short convolutions (taps float32 [channels, n_taps]; a
     request's rows before this step come from its state) and SiLU, queries and keys made unit vectors per head (queries times
-    q_scale), into qkv float32 [n, channels]; and gates float32 [n, 2 heads]: the decays exp(-exp(a_log) softplus(proj[a_off + h] +
-    dt_bias)), then the step sizes sigmoid(proj[b_off + h]).  single_rows: every row is its request's only row of the step; the
-    kernel then also moves every request's tail on by its row, and `delta_tail` is not needed."""
+    q_scale), into qkv float32 [n, channels]; and gates float32 [n, 2 heads]: the decays exp(-exp(a_log) softplus(a + dt_bias)), then
+    the step sizes sigmoid(proj[b_off + h]).  a: the column of proj at which the heads' numbers begin, or float32 [n, heads] rows of
+    their own.  single_rows: every row is its request's only row of the step; the kernel then also moves every request's tail on by its
+    row, and `delta_tail` is not needed.  channel: a decay per head and key channel; a and dt_bias are [.., heads*dk] and gates
+    [n, heads*dk + heads].  a None with a_up = (columns of proj [n, rank], w bfloat16 [heads or heads*dk, rank]): a = w x those columns
+    (rounded to bfloat16 as a product's rows are), made here: the form for a few rows."""
     _dev(proj, taps, a_log, dt_bias, ctx_slots, ctx_positions, state, qkv, gates)
     n, n_conv = proj.shape[0], 2 * n_kv * dk + n_heads * dv
     n_taps = taps.shape[1]
     _delta_checks("delta_prepare", proj, state, n_heads, n_kv, dk, dv, n_taps)
     if not (taps.dtype == torch.float32 and taps.shape == (n_conv, n_taps) and taps.is_contiguous()):
         raise KernelError("delta_prepare: taps must be float32 [2 kv_heads dk + heads dv, n_taps]")
-    for t, name in ((a_log, "a_log"), (dt_bias, "dt_bias")):
-        if not (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == n_heads):
-            raise KernelError(f"delta_prepare: {name} must be float32 [heads]")
-    if not (qkv.dtype == torch.float32 and qkv.shape == (n, n_conv) and qkv.is_contiguous() and gates.dtype == torch.float32 and gates.shape == (n, 2 * n_heads) and gates.is_contiguous()):
-        raise KernelError("delta_prepare: qkv must be float32 [n, channels] and gates float32 [n, 2 heads], contiguous")
-    if min(conv_off, a_off, b_off) < 0 or max(conv_off + n_conv, a_off + n_heads, b_off + n_heads) > proj.shape[1]:
+    n_decays = n_heads * dk if channel else n_heads
+    for t, name, size in ((a_log, "a_log", n_heads), (dt_bias, "dt_bias", n_decays)):
+        if not (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == size):
+            raise KernelError(f"delta_prepare: {name} must be float32 [{size}]")
+    if not (qkv.dtype == torch.float32 and qkv.shape == (n, n_conv) and qkv.is_contiguous() and gates.dtype == torch.float32 and gates.shape == (n, n_decays + n_heads)
+            and gates.is_contiguous()):
+        raise KernelError("delta_prepare: qkv must be float32 [n, channels] and gates float32 [n, decays + heads], contiguous")
+    if min(conv_off, b_off) < 0 or max(conv_off + n_conv, b_off + n_heads) > proj.shape[1]:
         raise KernelError("delta_prepare: the columns named lie outside proj")
+    if isinstance(a, int):
+        if not 0 <= a <= proj.shape[1] - n_decays:
+            raise KernelError("delta_prepare: the columns named lie outside proj")
+        a = proj[:, a:a + n_decays]
+    if (a is None) == (a_up is None):
+        raise KernelError("delta_prepare: the decays' inputs, or what they are made of, must be given")
+    _f32_rows(a, "delta_prepare: the decays' inputs", n, n_decays)
+    _dev(a)
+    low, ld_low, rank, w_up = _few_row_up("delta_prepare", a_up, n_decays)
+    if a_up is not None and (ld_low != proj.stride(0) or a_up[0].shape[0] != n):
+        raise KernelError("delta_prepare: the narrow rows must be columns of proj")
     _i32(ctx_slots, "delta_prepare: slots", n)
     _i32(ctx_positions, "delta_prepare: positions", n)
-    _call("gi_delta_prepare", proj.data_ptr(), proj.stride(0), int(conv_off), int(a_off), int(b_off), taps.data_ptr(), n_taps, a_log.data_ptr(), dt_bias.data_ptr(),
+    _call("gi_delta_prepare", proj.data_ptr(), proj.stride(0), int(conv_off), _ptr(a), a.stride(0) if a is not None else 0, int(b_off), taps.data_ptr(), n_taps, a_log.data_ptr(), dt_bias.data_ptr(),
           ctx_slots.data_ptr(), ctx_positions.data_ptr(), state.data_ptr(), state.stride(0), qkv.data_ptr(), gates.data_ptr(), n, n_heads, n_kv, dk, dv,
-          float(q_scale), 1 if single_rows else 0, _stream())
+          float(q_scale), 1 if single_rows else 0, 1 if channel else 0, low, rank, w_up, _stream())
 
 
 def delta_tail(proj, conv_off, n_taps, seg_start, seg_len, row_slot, state, n_heads, n_kv, dk, dv):
@@ -885,15 +972,17 @@ def delta_tail(proj, conv_off, n_taps, seg_start, seg_len, row_slot, state, n_he
           state.data_ptr(), state.stride(0), n_heads, n_kv, dk, dv, _stream())
 
 
-def delta_scan(qkv, gates, seg_start, seg_len, row_slot, state, out, n_heads, n_kv, dk, dv):
+def delta_scan(qkv, gates, seg_start, seg_len, row_slot, state, out, n_heads, n_kv, dk, dv, channel=False, single_rows=False):
     """The gated delta rule over every request's rows of the step, in order (csrc/recurrent.hip states it): qkv and gates as
     `delta_prepare` leaves them, out float32 [n, heads*dv] gets the read-outs M^T q; the memories come from the request's state
-    slot and go back into it."""
+    slot and go back into it.  channel: the decays are one per head and key channel.  single_rows: every request of the step has one row
+    (a kernel without staging; the same bits)."""
     _dev(qkv, gates, seg_start, seg_len, row_slot, state, out)
     n = qkv.shape[0]
     if not (qkv.dtype == torch.float32 and qkv.dim() == 2 and qkv.stride(1) == 1 and qkv.shape[1] >= 2 * n_kv * dk + n_heads * dv and gates.dtype == torch.float32
-            and gates.shape == (n, 2 * n_heads) and gates.is_contiguous() and out.dtype == torch.float32 and out.shape == (n, n_heads * dv) and out.stride(1) == 1):
-        raise KernelError("delta_scan: qkv must be float32 [n, channels], gates float32 [n, 2 heads], out float32 [n, heads*dv]")
+            and gates.shape == (n, n_heads * (dk + 1 if channel else 2)) and gates.is_contiguous() and out.dtype == torch.float32 and out.shape == (n, n_heads * dv)
+            and out.stride(1) == 1):
+        raise KernelError("delta_scan: qkv must be float32 [n, channels], gates float32 [n, decays + heads], out float32 [n, heads*dv]")
     if not (state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1 and state.shape[1] >= delta_memory_floats(n_heads, dk, dv)):
         raise KernelError("delta_scan: state must be float32 [slots, at least delta_memory_floats]")
     if not (0 < dk <= DELTA_MAX_KEY_DIM and n_heads % n_kv == 0):
@@ -903,16 +992,17 @@ def delta_scan(qkv, gates, seg_start, seg_len, row_slot, state, out, n_heads, n_
     _i32(seg_len, "delta_scan: seg_len", n_segs)
     _i32(row_slot, "delta_scan: slots", n)
     _call("gi_delta_scan", qkv.data_ptr(), qkv.stride(0), gates.data_ptr(), seg_start.data_ptr(), seg_len.data_ptr(), n_segs, row_slot.data_ptr(), state.data_ptr(),
-          state.stride(0), out.data_ptr(), out.stride(0), n_heads, n_kv, dk, dv, _stream())
+          state.stride(0), out.data_ptr(), out.stride(0), n_heads, n_kv, dk, dv, 1 if channel else 0, 1 if single_rows else 0, _stream())
     return out
 
 
 # --------------------------------------------------------------------------------------------- attention through latents
-def latent_prepare(proj, q_rank, kv_rank, rot, q_norm, kv_norm, eps, cos, sin, positions, slots, table, cq, cache, page_size):
+def latent_prepare(proj, q_rank, kv_rank, rot, q_norm, kv_norm, eps, cos, sin, positions, slots, table, cq, cache, page_size, half_split=False):
     """proj float32 [n, q_rank + kv_rank + rot]: the query latent, RMS-normed with q_norm, into cq [n, q_rank]; the key/value latent,
     RMS-normed with kv_norm, and the last rot channels turned in neighbouring pairs (cos, sin float32 [n, rot/2]), into the row's
     place of its page: the keys [place][kv_rank + rot], and the latent once more behind them with the places innermost, [kv_rank][place]
-    (a layer of one key/value head with keys of kv_rank + rot and values of kv_rank channels)."""
+    (a layer of one key/value head with keys of kv_rank + rot and values of kv_rank channels).  half_split: the pairs turned are
+    (i, i + rot/2)."""
     _dev(proj, q_norm, kv_norm, cos, sin, positions, slots, table, cq, cache)
     n = proj.shape[0]
     if not (proj.dtype == torch.float32 and proj.dim() == 2 and proj.stride(1) == 1 and proj.shape[1] >= q_rank + kv_rank + rot):
@@ -932,12 +1022,12 @@ def latent_prepare(proj, q_rank, kv_rank, rot, q_norm, kv_norm, eps, cos, sin, p
     _i32(slots, "latent_prepare: slots", n)
     _call("gi_latent_prepare", proj.data_ptr(), proj.stride(0), q_rank, kv_rank, rot, q_norm.data_ptr(), kv_norm.data_ptr(), _code(q_norm, "latent_prepare: norm"),
           float(eps), _ptr(cos), _ptr(sin), positions.data_ptr(), slots.data_ptr(), table.data_ptr(), table.stride(0), cq.data_ptr(), _code(cq, "latent_prepare: cq"),
-          cq.stride(0), cache.data_ptr(), _code(cache, "latent_prepare: cache"), cache.stride(0), int(page_size), n, _stream())
+          cq.stride(0), cache.data_ptr(), _code(cache, "latent_prepare: cache"), cache.stride(0), int(page_size), 1 if half_split else 0, n, _stream())
 
 
-def latent_queries(q, cos, sin, plain, folded, n_heads, dim, rot, kv_rank):
+def latent_queries(q, cos, sin, plain, folded, n_heads, dim, rot, kv_rank, half_split=False):
     """q float32 [n, heads*(dim + rot)]: every head's first dim channels into plain [n, heads*dim]; its last rot channels, turned in
-    neighbouring pairs, into folded [n, heads*(kv_rank + rot)] behind the head's first kv_rank places."""
+    neighbouring pairs (half_split: the pairs (i, i + rot/2)), into folded [n, heads*(kv_rank + rot)] behind the head's first kv_rank places."""
     _dev(q, cos, sin, plain, folded)
     n = q.shape[0]
     if not (q.dtype == torch.float32 and q.shape == (n, n_heads * (dim + rot)) and q.stride(1) == 1 and plain.shape == (n, n_heads * dim) and plain.stride(1) == 1
@@ -948,7 +1038,31 @@ def latent_queries(q, cos, sin, plain, folded, n_heads, dim, rot, kv_rank):
             if not (t.dtype == torch.float32 and t.shape == (n, rot // 2) and t.is_contiguous()):
                 raise KernelError("latent_queries: cos/sin must be float32 [n, rot/2]")
     _call("gi_latent_queries", q.data_ptr(), q.stride(0), _ptr(cos), _ptr(sin), plain.data_ptr(), _code(plain, "latent_queries: plain"), plain.stride(0),
-          folded.data_ptr(), _code(folded, "latent_queries: folded"), folded.stride(0), n, n_heads, dim, rot, kv_rank, _stream())
+          folded.data_ptr(), _code(folded, "latent_queries: folded"), folded.stride(0), n, n_heads, dim, rot, kv_rank, 1 if half_split else 0, _stream())
+
+
+def latent_direct(q, kv, kv_norm, eps, cos, sin, positions, slots, table, plain, folded, cache, page_size, n_heads, dim, rot, kv_rank, half_split=False):
+    """What `latent_prepare` does for the key/value latent and `latent_queries` for the queries, in one launch, for queries that have no
+    latent: q float32 [n, heads*(dim + rot)] and kv float32 [n, kv_rank + rot] (columns of one wider product are fine)."""
+    _dev(q, kv, kv_norm, cos, sin, positions, slots, table, plain, folded, cache)
+    n = q.shape[0]
+    _f32_rows(q, "latent_direct: q", n, n_heads * (dim + rot))
+    _f32_rows(kv, "latent_direct: kv", n, kv_rank + rot)
+    if not (kv_norm.shape == (kv_rank,) and kv_norm.is_contiguous() and plain.shape == (n, n_heads * dim) and plain.stride(1) == 1 and folded.shape == (n, n_heads * (kv_rank + rot))
+            and folded.stride(1) == 1 and folded.dtype == cache.dtype):
+        raise KernelError("latent_direct: the norm's weights [kv_rank], plain [n, heads*dim] and folded [n, heads*(kv_rank+rot)] of the cache's dtype are needed")
+    if rot:
+        for t in (cos, sin):
+            if not (t.dtype == torch.float32 and t.shape == (n, rot // 2) and t.is_contiguous()):
+                raise KernelError("latent_direct: cos/sin must be float32 [n, rot/2]")
+    _check_paged(cache, table, "latent_direct")
+    if cache.stride(0) < page_size * (2 * kv_rank + rot):
+        raise KernelError("latent_direct: the pages are too small for these latents")
+    _i32(positions, "latent_direct: positions", n)
+    _i32(slots, "latent_direct: slots", n)
+    _call("gi_latent_direct", q.data_ptr(), q.stride(0), kv.data_ptr(), kv.stride(0), kv_norm.data_ptr(), _code(kv_norm, "latent_direct: norm"), float(eps), _ptr(cos), _ptr(sin),
+          positions.data_ptr(), slots.data_ptr(), table.data_ptr(), table.stride(0), plain.data_ptr(), _code(plain, "latent_direct: plain"), plain.stride(0), folded.data_ptr(),
+          folded.stride(0), cache.data_ptr(), _code(cache, "latent_direct: cache"), cache.stride(0), int(page_size), 1 if half_split else 0, n, n_heads, dim, rot, kv_rank, _stream())
 
 
 class AttentionPlan:
@@ -1491,11 +1605,13 @@ def measured_mfma_rate(device="cuda:0", iters: int = 20000, repeats: int = 5) ->
     return lib().gi_probe_mfma_flops(iters, n_blocks) / (ms * 1e-3) / 1e12
 
 
-def heads_product(a, w, out, n_heads, out_head_stride=None):
+def heads_product(a, w, out, n_heads, out_head_stride=None, channel_gate=None):
     """out[t, h*stride + n] = sum_k a[t, h*k_dim + k] * w[h, n, k] for every head in one launch, on the matrix cores: a bfloat16
     [rows, heads*k_dim], w bfloat16 [heads, n_out, k_dim] contiguous, out [rows, >= heads*stride] bfloat16 or float32 (stride: n_out
-    if not given).  False, and nothing done, where the kernel does not take the operands (the caller then multiplies head by head)."""
-    _dev(a, w, out)
+    if not given).  channel_gate: float32 [rows, heads*n_out], every result is multiplied by its sigmoid.  False, and nothing done, where
+    the kernel does not take the operands (the caller then multiplies head by head)."""
+    _dev(a, w, out, channel_gate)
+    _f32_rows(channel_gate, "heads_product: the gates", a.shape[0], n_heads * w.shape[1])
     rows, k_dim, n_out = a.shape[0], w.shape[2], w.shape[1]
     stride = int(out_head_stride or n_out)
     if not (a.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and w.is_contiguous() and w.shape[0] == n_heads and a.shape[1] == n_heads * k_dim and a.stride(1) == 1
@@ -1504,7 +1620,8 @@ def heads_product(a, w, out, n_heads, out_head_stride=None):
         return False
     if _profile is not None:
         _profile.note = (f"{n_heads}x{n_out}x{k_dim}", w.numel() * w.element_size())
-    _call("gi_heads_product", a.data_ptr(), a.stride(0), w.data_ptr(), out.data_ptr(), _code(out, "heads_product: out"), out.stride(0), stride, rows, n_heads, k_dim, n_out, _stream())
+    _call("gi_heads_product", a.data_ptr(), a.stride(0), w.data_ptr(), out.data_ptr(), _code(out, "heads_product: out"), out.stride(0), stride, rows, n_heads, k_dim, n_out,
+          _ptr(channel_gate), channel_gate.stride(0) if channel_gate is not None else 0, _stream())
     return True
 
 
@@ -1519,13 +1636,15 @@ def latent_attention_prepare():
         raise KernelError(lib().gi_last_error().decode())
 
 
-def latent_attention_bf16(q, cache, out, ctx, table, n_heads, kd, vd, page_size, window=None, scale=1.0):
+def latent_attention_bf16(q, cache, out, ctx, table, n_heads, kd, vd, page_size, window=None, scale=1.0, sinks=None):
     """Attention of a step's rows over latent pages (one key/value head for all query heads: keys [place][kd], then the values
     [vd][place]) on the matrix cores; q bfloat16 [n, heads*kd], out bfloat16 [n, heads*vd].  The rows of prompts go by the attention
     plan's tiles: a workgroup takes a few consecutive rows with all their heads and stages the keys they see once in LDS.  Single
     rows, and the rows of short portions, are a wave per 16 heads and share of their context each; with few of them the context is
-    shared out further and a second kernel adds the shares."""
-    _dev(q, cache, out, table)
+    shared out further and a second kernel adds the shares.  sinks: float32 [heads], a score per head that joins the softmax's denominator only."""
+    _dev(q, cache, out, table, sinks)
+    if sinks is not None and not (sinks.dtype == torch.float32 and sinks.is_contiguous() and sinks.numel() == n_heads):
+        raise KernelError("latent_attention: sinks must be float32 [heads]")
     n = q.shape[0]
     if not (q.dtype == torch.bfloat16 and cache.dtype == torch.bfloat16 and out.dtype == torch.bfloat16 and q.shape == (n, n_heads * kd) and q.is_contiguous()
             and out.shape == (n, n_heads * vd) and out.is_contiguous()):
@@ -1537,7 +1656,7 @@ def latent_attention_bf16(q, cache, out, ctx, table, n_heads, kd, vd, page_size,
     by_tiles = plan.n_tiles > 0 and bool(lib().gi_latent_attention_tiles_supports(n_heads, kd, vd, int(page_size)))
     if by_tiles:
         _call("gi_latent_attention_tiles_bf16", q.data_ptr(), cache.data_ptr(), out.data_ptr(), plan.tiles.data_ptr(), plan.n_tiles, plan.tile, table.data_ptr(),
-              table.stride(0), cache.stride(0), int(page_size), n_heads, kd, vd, int(window or 0), float(scale), _stream())
+              table.stride(0), cache.stride(0), int(page_size), n_heads, kd, vd, int(window or 0), float(scale), _ptr(sinks), _stream())
         if not plan.n_decode:
             return out
         n_single, rows, span = plan.n_decode, plan.decode_rows, plan.max_decode_context
@@ -1550,7 +1669,8 @@ def latent_attention_bf16(q, cache, out, ctx, table, n_heads, kd, vd, page_size,
     n_part = n_single * n_heads * n_splits * (vd + 2) if n_splits > 1 else 0
     part = torch.empty(n_part, dtype=torch.float32, device=out.device) if n_part else None
     _call("gi_latent_attention_bf16", q.data_ptr(), cache.data_ptr(), out.data_ptr(), _ptr(part), n_part, _ptr(rows), ctx.row_pos.data_ptr(), ctx.row_slot.data_ptr(),
-          table.data_ptr(), table.stride(0), cache.stride(0), int(page_size), n_single, n_heads, kd, vd, int(window or 0), float(scale), n_splits, _stream())
+          table.data_ptr(), table.stride(0), cache.stride(0), int(page_size), n_single, n_heads, kd, vd, int(window or 0), float(scale), n_splits, _ptr(sinks),
+          _stream())
     return out
 
 
@@ -1757,10 +1877,19 @@ def _router_groups(what, n_experts, top, groups):
     return n_groups, keep
 
 
-def route_top(logits, top, ids, weights, score="sigmoid", renormalize=False, groups=None, floor=0.0):
+def _router_correction(what, correction, n_experts, groups):
+    if correction is not None:
+        _dev(correction)
+        if not (correction.dtype == torch.float32 and correction.is_contiguous() and correction.numel() == n_experts) or groups is not None:
+            raise KernelError(f"{what}: the correction must be float32 [experts], and the experts in one group")
+    return _ptr(correction)
+
+
+def route_top(logits, top, ids, weights, score="sigmoid", renormalize=False, groups=None, floor=0.0, correction=None, scale=1.0):
     """ids int32 [n, top], weights float32 [n, top]: per row the `top` experts with the largest scores (the lower index wins a tie)
     and their scores, divided by their sum + `floor` if `renormalize`.  groups = (count, keep): the experts form `count` equal groups
-    of neighbours, a group scores what its best expert scores, and only experts of the `keep` best groups can be chosen."""
+    of neighbours, a group scores what its best expert scores, and only experts of the `keep` best groups can be chosen.  correction:
+    float32 [experts], added to the scores for the choice (the weights come from the scores without it).  The weights are multiplied by `scale`."""
     _dev(logits, ids, weights)
     n, n_experts = logits.shape
     _f32_rows(logits, "route_top: logits")
@@ -1771,7 +1900,7 @@ def route_top(logits, top, ids, weights, score="sigmoid", renormalize=False, gro
     if not (ids.dtype == torch.int32 and ids.shape == (n, top) and ids.is_contiguous() and weights.dtype == torch.float32 and weights.shape == (n, top) and weights.is_contiguous()):
         raise KernelError("route_top: ids must be int32 [n, top] and weights float32 [n, top], contiguous")
     _call("gi_route_top", logits.data_ptr(), logits.stride(0), n, n_experts, top, ROUTER_SCORES[score], 1 if renormalize else 0, float(floor),
-          *_router_groups("route_top", n_experts, top, groups), ids.data_ptr(), weights.data_ptr(), _stream())
+          *_router_groups("route_top", n_experts, top, groups), _router_correction("route_top", correction, n_experts, groups), float(scale), ids.data_ptr(), weights.data_ptr(), _stream())
 
 
 def _expert_stack(w, rows, cols, what):
@@ -1782,7 +1911,8 @@ def _expert_stack(w, rows, cols, what):
 def experts_gate_up(h, w_gate, w_up, ids, weights, mid, weigh_input=True, activation="silu", limit=0.0):
     """mid[(row, choice)] = act(W_gate[e] a) * (W_up[e] a), a = the row of h (times the choice's weight if `weigh_input`, stored as
     h's dtype), e = ids[row, choice]; one wave per output, for the few rows of decoding steps.  w_up None: w_gate is one stack
-    [experts, 2 ff, width] of 16 gate rows, the 16 up rows of the same outputs, and so on (`interleave_gate_up` per expert)."""
+    [experts, 2 ff, width] of 16 gate rows, the 16 up rows of the same outputs, and so on (`interleave_gate_up` per expert).  A number from
+    `experts` on in ids has no matrices; its rows of mid are left as they are."""
     _dev(h, w_gate, w_up, ids, weights, mid)
     n, width = h.shape
     top = ids.shape[1]
@@ -1798,13 +1928,17 @@ def experts_gate_up(h, w_gate, w_up, ids, weights, mid, weigh_input=True, activa
         raise KernelError("experts_gate_up: h [n, width], mid [n * top, ff], ids int32 and weights float32 [n, top] are needed")
     _call("gi_experts_gate_up", h.data_ptr(), _code(h, "experts_gate_up: h"), h.stride(0), w_gate.data_ptr(), _ptr(w_up), _code(w_gate, "experts_gate_up: weights"),
           ids.data_ptr(), weights.data_ptr(), 1 if weigh_input else 0, mid.data_ptr(), _code(mid, "experts_gate_up: mid"), mid.stride(0), n, top, width, ff,
-          ACTIVATIONS[activation], float(limit), group, _stream())
+          ACTIVATIONS[activation], float(limit), group, w_gate.shape[0], _stream())
     return mid
 
 
-def experts_down(mid, w_down, ids, weights, x, accumulate=True, weigh_output=False):
-    """x[row] (+)= sum over the row's choices of W_down[e] mid[(row, choice)] (times the choice's weight if `weigh_output`)."""
-    _dev(mid, w_down, ids, weights, x)
+def experts_down(mid, w_down, ids, weights, x, accumulate=True, weigh_output=False, h=None):
+    """x[row] (+)= sum over the row's choices of W_down[e] mid[(row, choice)] (times the choice's weight if `weigh_output`).  A number from
+    `experts` on in ids stands for an expert that returns its input: the choice's weight times the row of h."""
+    _dev(mid, w_down, ids, weights, x, h)
+    h = x if h is None else h
+    if not (h.shape == x.shape and h.stride(1) == 1):
+        raise KernelError("experts_down: the experts' inputs must be [n, width]")
     n, width = x.shape
     top, ff = ids.shape[1], w_down.shape[2]
     _expert_stack(w_down, width, ff, "experts_down: the down products")
@@ -1813,13 +1947,14 @@ def experts_down(mid, w_down, ids, weights, x, accumulate=True, weigh_output=Fal
             and weights.dtype == torch.float32 and weights.shape == (n, top) and weights.is_contiguous()):
         raise KernelError("experts_down: mid [n * top, ff], ids int32 and weights float32 [n, top] are needed")
     _call("gi_experts_down", mid.data_ptr(), _code(mid, "experts_down: mid"), mid.stride(0), w_down.data_ptr(), _code(w_down, "experts_down: weights"), ids.data_ptr(),
-          weights.data_ptr(), 1 if weigh_output else 0, x.data_ptr(), x.stride(0), 1 if accumulate else 0, n, top, width, ff, _stream())
+          weights.data_ptr(), 1 if weigh_output else 0, x.data_ptr(), x.stride(0), 1 if accumulate else 0, n, top, width, ff, h.data_ptr(), _code(h, "experts_down: h"), h.stride(0),
+          w_down.shape[0], _stream())
     return x
 
 
-def route_rows(h, router, top, ids, weights, score="sigmoid", renormalize=False, logits=None, groups=None, floor=0.0, extra=None):
+def route_rows(h, router, top, ids, weights, score="sigmoid", renormalize=False, logits=None, groups=None, floor=0.0, extra=None, correction=None, scale=1.0):
     """The router's product and its choice in one launch: logits = h @ router.T with 32-bit sums in an order that the width alone
-    fixes, then as `route_top` (with its `groups` and `floor`).  logits: float32 [n, experts] to keep them in, or None.  extra:
+    fixes, then as `route_top` (with its `groups`, `floor`, `correction` and `scale`).  logits: float32 [n, experts] to keep them in, or None.  extra:
     float32 [n, k]: the router's matrix has k more rows behind the experts', whose products with the rows go there (no expert's
     logits: they take no part in the choice)."""
     _dev(h, router, ids, weights, logits, extra)
@@ -1838,7 +1973,8 @@ def route_rows(h, router, top, ids, weights, score="sigmoid", renormalize=False,
     if logits is not None:
         _f32_rows(logits, "route_rows: logits", n, n_experts)
     _call("gi_route_rows", h.data_ptr(), _code(h, "route_rows: h"), h.stride(0), router.data_ptr(), _code(router, "route_rows: the router"), router.stride(0), n, width,
-          n_experts, top, ROUTER_SCORES[score], 1 if renormalize else 0, float(floor), *_router_groups("route_rows", n_experts, top, groups), ids.data_ptr(), weights.data_ptr(),
+          n_experts, top, ROUTER_SCORES[score], 1 if renormalize else 0, float(floor), *_router_groups("route_rows", n_experts, top, groups),
+          _router_correction("route_rows", correction, n_experts, groups), float(scale), ids.data_ptr(), weights.data_ptr(),
           _ptr(logits), logits.stride(0) if logits is not None else 0, n_extra, _ptr(extra), extra.stride(0) if extra is not None else 0, _stream())
 
 
@@ -1872,11 +2008,19 @@ def experts_grouped_supported(h, w_gate, w_up, w_down) -> bool:
     return width % 64 == 0 and ff % 64 == 0 and width >= 128 and 2 * ff >= 128 and h.stride(0) % 8 == 0 and h.data_ptr() % 16 == 0
 
 
-def routed_experts(h, w_gate, w_up, w_down, ids, weights, x, accumulate=True, weigh="input", activation="silu", limit=0.0):
+def experts_combine_norm_takes(x, h) -> bool:
+    """Whether the kernel that adds the experts' results onto these rows also takes a layer norm behind it."""
+    return (bool(lib().gi_experts_combine_norm_takes(x.shape[1])) and x.stride(0) % 4 == 0 and h.stride(0) % 4 == 0 and x.data_ptr() % 16 == 0 and h.data_ptr() % 16 == 0)
+
+
+def routed_experts(h, w_gate, w_up, w_down, ids, weights, x, accumulate=True, weigh="input", activation="silu", limit=0.0, then=None):
     """x[row] (+)= sum over the row's choices of expert(a): the whole mixture behind the router's choice.  weigh "input": a = weight * h[row]
     (stored as h's dtype); "output": a = h[row] and the weight multiplies the expert's result.  w_up None: w_gate holds both (see
     `experts_gate_up`).  Few items, or 32-bit operands: every item walks its expert's matrices.  Many in bfloat16: the items' rows are
-    put in the order of their experts and all experts' products are two launches on the matrix cores."""
+    put in the order of their experts and all experts' products are two launches on the matrix cores.  A number from `experts` on in ids
+    stands for an expert that returns its input (times the choice's weight, whichever `weigh` is).
+    then = (weight, bias, eps), the layer norm that reads x next: where the kernel that adds the results up makes its rows on the way
+    (bfloat16 [n, width]), they are returned; None otherwise."""
     if weigh not in ("input", "output"):
         raise KernelError(f"routed_experts: the weights weigh an expert's 'input' or its 'output', not {weigh!r}")
     n, top = ids.shape
@@ -1895,20 +2039,28 @@ def routed_experts(h, w_gate, w_up, w_down, ids, weights, x, accumulate=True, we
         count, place, tile_expert = book[:n_experts], book[n_experts:n_experts + n * top], book[n_experts + n * top:]
         _call("gi_experts_place", ids.data_ptr(), n * top, n_experts, count.data_ptr(), place.data_ptr(), tile_expert.data_ptr(), n_tiles, _stream())
         rows = torch.empty((n_tiles * tile, width), dtype=torch.bfloat16, device=dev)
-        _call("gi_experts_gather", h.data_ptr(), h.stride(0), place.data_ptr(), weights.data_ptr(), 1 if weigh == "input" else 0, n, top, rows.data_ptr(), rows.stride(0),
-              width, _stream())
+        _call("gi_experts_gather", h.data_ptr(), h.stride(0), ids.data_ptr(), place.data_ptr(), weights.data_ptr(), 1 if weigh == "input" else 0, n, top, rows.data_ptr(),
+              rows.stride(0), width, n_experts, _stream())
         mid = torch.empty((n_tiles * tile, ff), dtype=torch.bfloat16, device=dev)
         gemm_bf16_grouped(rows, w_gate, mid, tile_expert, gated=True if activation == "silu" else activation, gate_limit=limit)
         y = torch.empty((n_tiles * tile, width), dtype=torch.float32, device=dev)
         gemm_bf16_grouped(mid, w_down, y, tile_expert)
-        _call("gi_experts_combine", y.data_ptr(), y.stride(0), place.data_ptr(), weights.data_ptr(), 1 if weigh == "output" else 0, n, top, x.data_ptr(), x.stride(0),
-              width, 1 if accumulate else 0, _stream())
-        return x
+        norm_w, norm_b, eps, low = None, None, 0.0, None
+        if then is not None and experts_combine_norm_takes(x, h):
+            norm_w, norm_b, eps = then
+            if not (norm_w.shape == norm_b.shape == (width,) and norm_w.is_contiguous() and norm_b.is_contiguous() and norm_w.dtype == norm_b.dtype
+                    and norm_w.data_ptr() % 16 == 0 and norm_b.data_ptr() % 16 == 0):
+                raise KernelError("routed_experts: the norm behind needs weight and bias [width] of one dtype, aligned")
+            low = torch.empty((n, width), dtype=torch.bfloat16, device=dev)
+        _call("gi_experts_combine", y.data_ptr(), y.stride(0), ids.data_ptr(), place.data_ptr(), weights.data_ptr(), 1 if weigh == "output" else 0, n, top, x.data_ptr(), x.stride(0),
+              width, 1 if accumulate else 0, h.data_ptr(), h.stride(0), n_experts, _ptr(norm_w), _ptr(norm_b), _code(norm_w, "routed_experts: norm") if low is not None else F32, float(eps),
+              _ptr(low), low.stride(0) if low is not None else 0, _stream())
+        return low
     mid_dtype = torch.float32 if w_down.dtype == torch.float32 else h.dtype
     mid = torch.empty((n * top, ff), dtype=mid_dtype, device=h.device)
     experts_gate_up(h, w_gate, w_up, ids, weights, mid, weigh_input=weigh == "input", activation=activation, limit=limit)
-    experts_down(mid, w_down, ids, weights, x, accumulate=accumulate, weigh_output=weigh == "output")
-    return x
+    experts_down(mid, w_down, ids, weights, x, accumulate=accumulate, weigh_output=weigh == "output", h=h)
+    return None
 
 
 # ---------------------------------------------------------------- several copies of the residual stream, the row before a row

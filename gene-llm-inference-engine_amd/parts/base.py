@@ -131,6 +131,8 @@ class FeedForward(Part):
 #                                  None; with it `use_input_weight(view)` (the same matrix as a view of a larger one, to keep instead of its
 #                                  own) and a keyword `projected` of `forward` (float32 [rows, that matrix's rows]: the product, already made).
 #                                  A block whose parts read the same rows may then make their first products as one (`ParallelBlock`).
+#   makes_next_norm(norm)          whether the part, where it writes the residual last, can also make the rows of `norm`, the norm that reads the
+#                                  residual next; `forward` then takes `then` (that norm) and returns the rows ready (`ReadyRows`) or None.
 
 
 # Optional, for a block (an arrangement of parts; of however many halves):
@@ -170,7 +172,8 @@ class StreamPart(Part):
     """Something that changes the residual stream x (float32 [T, hidden]) in place between layers: a second input from the
     tokens, a product that mixes the stream with the token rows again.  It reads what it needs of the step from `ctx` (the
     tokens on the device; `ctx.memo["token_rows"]`, float32 [T, hidden], if it says `needs_token_rows`).  One that says
-    `hands_norm_on` has a block's `first_reader()` and takes a block's keywords `handed` and `next_reader` (behind a layer)."""
+    `hands_norm_on` has a block's `first_reader()` and takes a block's keywords `handed` and `next_reader`; before a run-order entry
+    `handed` is None and next_reader the entry's layer's."""
     needs_token_rows = False
 
     def forward(self, x: torch.Tensor, ctx: StepContext) -> None:
@@ -180,9 +183,16 @@ class StreamPart(Part):
 class RowTransform(Part):
     """An elementwise change of float32 rows in place: what a model may ask for between the token table and the
     first layer, and on the logits.  One that says `needs_context` (behind the token table only) is called with the step's context as
-    well; one that serves so many positions only says how many in `position_limit`."""
+    well; one that serves so many positions only says how many in `position_limit`.  One behind the token table that says
+    `fetches_token_rows` fetches them itself (`fetch(table, x, ctx, cache, keep)`; it must be the first of its list) and may keep a
+    state per request: `cache_need(spec)` is then a `StateNeed`."""
     needs_context = False
+    fetches_token_rows = False
     position_limit: Optional[int] = None
+
+    @classmethod
+    def cache_need(cls, spec):
+        return None
 
     def __call__(self, x: torch.Tensor) -> None:
         raise NotImplementedError

@@ -15,7 +15,7 @@ import torch
 from ..kernels import ops
 from .base import feed_forward_class, mixer_class, norm_class, register_block
 from .linear import linear, takes_handed_norm
-from .norm import NormedRows, norm_to_hand_on
+from .norm import NormedRows, ReadyRows, norm_to_apply, norm_to_hand_on
 
 
 class PreNormBlock:
@@ -175,6 +175,7 @@ register_block("sandwich", SandwichBlock)
 
 class _Readers:
     """The parts that read one norm's rows, asked as one whether they take that norm half applied."""
+    takes_ready_rows = True          # ... or wholly applied by whoever wrote the rows (where all of them read one dtype)
 
     def __init__(self, parts, first_weight=None):
         self.parts, self.first_weight = parts, first_weight          # first_weight(n_rows): the one matrix all of them read at this number of rows, or None
@@ -194,7 +195,8 @@ class ParallelBlock:
     adds its result onto x (the two sums reach x one after the other; neither half reads x).  The block plays the game of
     handing a norm on (`hands_norm_on`, `first_reader`, `handed`, `next_reader`): the half that writes x last does the next
     norm's first share, and a norm so handed to this block is finished by the first products of both halves, where both can
-    (asked beforehand: the second half must not fall back on rows that the first has changed by then)."""
+    (asked beforehand: the second half must not fall back on rows that the first has changed by then).  A norm that does not commute
+    with a product may be made whole by the half that writes x last, if it can (`makes_next_norm`)."""
     hands_norm_on = True
     STACK = True                     # the two halves' first products as one (off: each half makes its own)
     # ... in steps of up to so many rows and with both matrices together up to so many bytes: one launch less a layer where launches
@@ -255,6 +257,9 @@ class ParallelBlock:
         whatever reads x after this block, or None.  Returns that reader's norm handed on, or None."""
         if handed is not None and handed.norm is self.mixer_norm and self._readers.takes_handed_norm(ctx.n_rows):
             rows = lambda part: handed
+        elif isinstance(handed, ReadyRows) and handed.norm is self.mixer_norm and handed.out_dtype == self._readers.in_dtype:
+            h = handed.materialize()
+            rows = lambda part: h
         elif self._readers.in_dtype is not None:      # one set of normed rows serves both halves
             h = self.mixer_norm(x, self._readers.in_dtype)
             rows = lambda part: h
@@ -262,7 +267,7 @@ class ParallelBlock:
             made = {part: self.mixer_norm(x, getattr(part, "in_dtype", ctx.dtype)) for part in self._parts()[1:]}      # (before anything changes x)
             rows = made.__getitem__
         last = self.feed_forward if self.feed_forward is not None else self.mixer
-        then = norm_to_hand_on(next_reader, ctx.n_rows) if getattr(last, "hands_norm_on", False) else None
+        then = norm_to_hand_on(next_reader, ctx.n_rows) if getattr(last, "hands_norm_on", False) else norm_to_apply(next_reader, last)
         own = [{}, {}]                            # what each half is told beyond its rows
         w_first = self._stacked(ctx.n_rows)
         if w_first is not None:

@@ -15,7 +15,7 @@ from ..kernels import ops
 from ..weights.loader import TensorNeed
 from .base import FeedForward, feed_forward_class, register_feed_forward
 from .linear import activation_dtype_for, linear
-from .norm import NormedRows
+from .norm import LayerNorm, NormedRows, ReadyRows
 
 
 class RoutedExperts(FeedForward):
@@ -31,12 +31,14 @@ class RoutedExperts(FeedForward):
             raise ValueError(f"routed experts: the weights weigh an expert's 'input' or its 'output', not {s.weigh!r}")
         if s.activation not in ops.ACTIVATIONS:
             raise ValueError(f"routed experts: unknown activation {s.activation!r}; known: {', '.join(ops.ACTIVATIONS)}")
-        if s.n_experts > ops.ROUTER_MAX_EXPERTS or s.top > ops.ROUTER_MAX_TOP:
+        if s.n_experts + getattr(s, "n_identity", 0) > ops.ROUTER_MAX_EXPERTS or s.top > ops.ROUTER_MAX_TOP:
             raise ValueError(f"routed experts: at most {ops.ROUTER_MAX_EXPERTS} experts and {ops.ROUTER_MAX_TOP} a row")
         self.router = tensors[s.router]
         self.limit = float(getattr(s, "activation_limit", 0.0))
         self.groups = (s.n_groups, s.groups_kept) if getattr(s, "n_groups", 1) > 1 else None
         self.floor = float(getattr(s, "renormalize_floor", 0.0))
+        self.weight_scale = float(getattr(s, "weight_scale", 1.0))
+        self.correction = tensors[s.correction].float().contiguous() if getattr(s, "correction", None) is not None else None
         # the shared feed-forward's gate is one more row of the router's matrix: its logit comes out of the router's product, in 32-bit
         self.shared_gated = getattr(s, "shared_gate", None) is not None
         self.router_all = torch.cat([self.router, tensors[s.shared_gate].reshape(1, -1)], dim=0).contiguous() if self.shared_gated else self.router
@@ -58,7 +60,10 @@ class RoutedExperts(FeedForward):
     @classmethod
     def tensor_needs(cls, spec):
         s, d, i = spec, spec.hidden_size, spec.intermediate_size
-        needs = [TensorNeed(s.router, (s.n_experts, d))]
+        outputs = s.n_experts + getattr(s, "n_identity", 0)
+        needs = [TensorNeed(s.router, (outputs, d))]
+        if getattr(s, "correction", None) is not None:
+            needs.append(TensorNeed(s.correction, (outputs,)))
         for g, u, w in zip(s.gate_projs, s.up_projs, s.down_projs):
             needs += [TensorNeed(g, (i, d)), TensorNeed(u, (i, d)), TensorNeed(w, (d, i))]
         if s.shared is not None:
@@ -73,15 +78,20 @@ class RoutedExperts(FeedForward):
         share = [w[:min(s.top, s.n_experts)] for w in (self.w_gate, self.w_up, self.w_down) if w is not None]
         return [self.router_all, *share] + ([self.shared] if self.shared is not None else [])
 
+    def makes_next_norm(self, norm) -> bool:
+        """The kernel that adds the experts' results onto the residual can take a layer norm behind it (nothing may write in between)."""
+        return isinstance(norm, LayerNorm) and self.shared is None
+
     def forward(self, h, residual, ctx, then=None, overwrite=False):
         s, T, dev = self.spec, ctx.n_rows, ctx.device
         rows = h.materialize() if isinstance(h, NormedRows) else h
         ids = torch.empty((T, s.top), dtype=torch.int32, device=dev)
         weights = torch.empty((T, s.top), dtype=torch.float32, device=dev)
         gate = torch.empty((T, 1), dtype=torch.float32, device=dev) if self.shared_gated else None          # (its logit comes out of the router's product)
-        ops.route_rows(rows, self.router_all, s.top, ids, weights, s.score, s.renormalize, groups=self.groups, floor=self.floor, extra=gate)
-        ops.routed_experts(rows, self.w_gate, self.w_up, self.w_down, ids, weights, residual, accumulate=not overwrite, weigh=s.weigh, activation=s.activation,
-                           limit=self.limit)
+        ops.route_rows(rows, self.router_all, s.top, ids, weights, s.score, s.renormalize, groups=self.groups, floor=self.floor, extra=gate, correction=self.correction,
+                       scale=self.weight_scale)
+        normed = ops.routed_experts(rows, self.w_gate, self.w_up, self.w_down, ids, weights, residual, accumulate=not overwrite, weigh=s.weigh, activation=s.activation,
+                                    limit=self.limit, then=None if then is None else (then.weight, then.bias, then.eps))
         if self.shared is not None and not self.shared_gated:
             self.shared.forward(rows, residual, ctx)
         elif self.shared is not None:          # its result in rows of its own, added times the row's gate
@@ -92,7 +102,7 @@ class RoutedExperts(FeedForward):
                 y = torch.zeros_like(residual)
                 self.shared.forward(rows, y, ctx)
             ops.add_rows_gated(residual, y, gate)
-        return None
+        return None if normed is None else ReadyRows(then, residual, normed)
 
 
 register_feed_forward("routed_experts", RoutedExperts)

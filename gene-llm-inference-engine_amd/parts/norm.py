@@ -1,5 +1,6 @@
-"""RMS norm: out = w * (x * rsqrt(mean(x^2) + eps)), eps inside the root, the weight as stored
-(reference: src/kernels/kernels.cpp:72-83), or, where the spec says so, the stored weight plus a constant.
+"""Norms of rows.  RMS norm: out = w * (x * rsqrt(mean(x^2) + eps)), eps inside the root, the weight as stored
+(reference: src/kernels/kernels.cpp:72-83), or, where the spec says so, the stored weight plus a constant.  Layer norm: the mean
+removed, divided by the standard deviation (eps inside the root), weight and bias.
 
 A norm may be handed on *unapplied* (`deferred`): `NormedRows` names the rows (optionally a
 selection of them), the weight and eps; whoever consumes it asks for the rows (`materialize`), and
@@ -61,6 +62,15 @@ def norm_to_hand_on(reader, n_rows: int):
     return norm
 
 
+def norm_to_apply(reader, part):
+    """reader: as above.  The norm, if `part`, which writes the rows it reads, can make the normed rows on the way (`makes_next_norm(norm)`)
+    for a reader that takes them ready in bfloat16; None otherwise."""
+    norm, reads = reader if reader is not None else (None, None)
+    if norm is None or not hasattr(part, "makes_next_norm") or getattr(reads, "in_dtype", None) != torch.bfloat16 or not getattr(reads, "takes_ready_rows", False):
+        return None
+    return norm if part.makes_next_norm(norm) else None
+
+
 class RmsNorm(Norm):
     graph_safe = True
 
@@ -116,6 +126,30 @@ class RmsNorm(Norm):
         return [self.weight]
 
 
+class LayerNorm(Norm):
+    graph_safe = True
+
+    def __init__(self, spec, tensors, dtype, device):
+        super().__init__(spec, tensors, dtype, device)
+        self.weight, self.bias, self.eps = tensors[spec.weight], tensors[spec.bias], float(spec.eps)
+
+    @classmethod
+    def tensor_needs(cls, spec):
+        return [TensorNeed(spec.weight, (spec.size,), "norm"), TensorNeed(spec.bias, (spec.size,), "norm")]
+
+    def __call__(self, x, out_dtype, rows=None):
+        """The normed rows of x, or of x[rows]."""
+        n = x.shape[0] if rows is None else rows.numel()
+        return ops.layernorm(x, self.weight, self.bias, self.eps, torch.empty((n, x.shape[1]), dtype=out_dtype, device=x.device), rows)
+
+    def join_and_norm(self, x, out_dtype, add=None, vector=None) -> ReadyRows:
+        """x += add + vector (either may be None), and the normed rows of the sum, in one kernel."""
+        return ReadyRows(self, x, ops.layernorm(x, self.weight, self.bias, self.eps, torch.empty(x.shape, dtype=out_dtype, device=x.device), add=add, vector=vector))
+
+    def deferred(self, x, out_dtype, rows=None) -> NormedRows:
+        return NormedRows(self, x, out_dtype, rows)
+
+
 class NoNorm(Norm):
     """The rows as they are, stored as the reader takes them (float32: the rows themselves, no copy)."""
     graph_safe = True
@@ -126,4 +160,5 @@ class NoNorm(Norm):
 
 
 register_norm("rmsnorm", RmsNorm)
+register_norm("layernorm", LayerNorm)
 register_norm("none", NoNorm)

@@ -1,6 +1,6 @@
 """Parts that change the residual stream between layers (`StreamPart`): a second input from the token itself behind a layer
 (`config.spec.TokenSideInputSpec`), and the stream mixed with the token rows again before a run-order entry
-(`config.spec.RejoinSpec`).  The residual stream stays 32-bit; what goes into a product is stored as the compute dtype stores
+(`config.spec.RejoinSpec`; or merely added to, `config.spec.AddRowsSpec`).  The residual stream stays 32-bit; what goes into a product is stored as the compute dtype stores
 a product's rows."""
 from __future__ import annotations
 
@@ -109,5 +109,37 @@ class Rejoin(StreamPart):
             ops.add_vector(x, self.offset)
 
 
+class AddRows(StreamPart):
+    """x += the token rows (where the spec says so) + a vector: one kernel, with the norm that reads x next where that one can join."""
+    graph_safe = True
+    hands_norm_on = True
+
+    def __init__(self, spec, tensors, dtype, device):
+        super().__init__(spec, tensors, dtype, device)
+        self.vector = tensors[spec.offsets][spec.row].clone()          # (a copy: its place in the table need not be aligned)
+        self.needs_token_rows = bool(spec.token_rows)
+
+    @classmethod
+    def tensor_needs(cls, spec):
+        if not 0 <= spec.row < spec.offsets_rows:
+            raise ValueError("rows added to the stream: the vector asked for does not exist")
+        return [TensorNeed(spec.offsets, (spec.offsets_rows, spec.hidden_size))]
+
+    def first_reader(self):
+        return None
+
+    def weights_read_per_step(self):
+        return [self.vector]
+
+    def forward(self, x, ctx, handed=None, next_reader=None):
+        add = ctx.memo["token_rows"] if self.needs_token_rows else None
+        norm, reads = next_reader if next_reader is not None else (None, None)
+        if hasattr(norm, "join_and_norm") and norm.weight.dtype == self.vector.dtype and getattr(reads, "takes_ready_rows", False) and getattr(reads, "in_dtype", None) is not None:
+            return norm.join_and_norm(x, reads.in_dtype, add=add, vector=self.vector)
+        ops.layernorm(x, None, None, 0.0, None, add=add, vector=self.vector)
+        return None
+
+
 register_stream_part("token_side_input", TokenSideInput)
+register_stream_part("add_rows", AddRows)
 register_stream_part("rejoin", Rejoin)
