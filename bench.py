@@ -5,6 +5,7 @@
     python bench.py --rigalorn [--sizes 1b,8b] [--layers L] [--batch B] [--prefill-tokens T]    (another record: see `rigalorn_beside_fekorax`)
     python bench.py --zidevik [--sizes 1b,8b] [--layers L] [--batch B] [--prefill-tokens T]     (another record: see `zidevik_beside_rigalorn`)
     python bench.py --mimitar [--sizes 1b,8b] [--layers L] [--batch B] [--prefill-tokens T]     (another record: see `mimitar_beside_zidevik`)
+    python bench.py --puzorax [--sizes 1b,8b] [--layers L] [--batch B] [--prefill-tokens T]     (another record: see `puzorax_beside_rigalorn`)
 
 A step is one decode step of the whole batch (default batch 8, each request on a 2,048-token
 prompt in a 4,096-token context), through the scheduler with its defaults.  After W warm-up steps,
@@ -310,6 +311,51 @@ def vubenex_beside_fekorax(args) -> int:
     return 0
 
 
+def puzorax_beside_rigalorn(args) -> int:
+    """The Puzorax design at layer shapes of real models beside the Rigalorn design (the nearest the engine has: parallel layers of the
+    delta rule and of attention through latents), the Zidevik design (routed experts, layers walked twice) and the Llama decoder at the
+    same shapes, random weights; measured as `fekorax_beside_llama` measures.  A Puzorax model of L layers here is L/2 times [delta rule
+    with a decay per key channel; attention through latents], the memories and the latents of Rigalorn's sizes here (queries without a
+    latent, a sink per head, a gate per channel, a window of 1,024), the narrow middles one head size wide; every layer has 8 experts of a
+    quarter of the Llama layer's inner size and one that returns its input, of which 2 serve a token.  Layers 0 and 1 are walked twice, so
+    a model of L layers here runs L + 2; a table of 65,536 pairs of tokens.  One JSON line."""
+    import torch
+    T, batch, L, steps = args.prefill_tokens, args.batch, args.layers or 8, args.steps
+    gen = torch.Generator().manual_seed(1)
+    record = {"metric": "Puzorax beside Rigalorn, Zidevik and Llama at equal layer shapes: prefill tok/s, decode ms a step, ms by kernel", "dtype": args.dtype, "layers": L,
+              "prefill_tokens": T, "decode_batch": batch, "data": "synthetic: random weights by formula, uniform random token ids", "sizes": {}}
+    for size in args.sizes.split(","):
+        D, H, G, hd, ff, vocab = FEKORAX_SIZES[size]
+        mlp = dict(kind="dense", ff=ff)
+        llama = dict(architectures=["LlamaForCausalLM"], hidden_size=D, intermediate_size=ff, num_hidden_layers=L, num_attention_heads=H,
+                     num_key_value_heads=G, head_dim=hd, vocab_size=vocab, max_position_embeddings=T + 1024, rope_theta=500000.0, rms_norm_eps=1e-5,
+                     tie_word_embeddings=True)
+        memory = dict(heads=max(1, H // 4), kv_heads=max(1, H // 8), dim=hd, vdim=2 * hd, conv=4)
+        latents = dict(heads=H, dim=hd, rot_dim=hd // 2, vdim=hd, kv_rank=4 * hd, scale=(1.5 * hd) ** -0.5, rot=dict(dims=hd // 2, base=500000.0), mask=dict(size=1024))
+        delta = dict(type="delta", mlp=mlp, mixer=memory)
+        latent = dict(type="latent_attention", mlp=mlp, mixer=dict(latents, q_rank=12 * hd))
+        blended = dict(type="attention", mlp=mlp, mixer=dict(heads=H, kv_heads=G, dim=hd, vdim=hd, scale=hd ** -0.5, v_mix=True, mask=dict(size=1024), rot=dict(
+            dims=hd // 2, base=10000.0, scaling=dict(factor=4.0, original=4096, fast=16.0, slow=2.0))))
+        rigalorn = dict(architecture="Rigalorn", vocab=vocab, width=D, embedding=dict(scale=D ** 0.5), norm=dict(eps=1e-5), max_positions=T + 1024,
+                        layers=([delta, latent, blended, delta] * ((L + 3) // 4))[:L])
+        mixer = dict(left=dict(heads=H, kv_heads=G, dim=hd, vdim=hd, scale=hd ** -0.5, rot=dict(dims=hd // 2, base=500000.0)), left_scale=1.0,
+                     right=dict(inner=2 * D, state=16, dt_rank=D // 16, conv=4), right_scale=1.0)
+        z_moe = dict(kind="moe", router=dict(experts=8, top=2), expert=dict(ff=ff // 4), shared=dict(ff=ff // 2))
+        zidevik = dict(architecture="Zidevik", vocab=vocab, width=D, norm=dict(eps=1e-5), max_positions=T + 1024, logit_softcap=30.0, token_side=dict(dim=256),
+                       loop=dict(start=0, stop=min(2, L), times=2), layers=[dict(type="parallel", mixer=mixer, mlp=mlp if i % 2 == 0 else z_moe) for i in range(L)])
+        moe = dict(kind="moe", router=dict(experts=8, identity=1, top=2, scale=2.0), expert=dict(ff=ff // 4))
+        pair = [dict(type="channel_delta", mlp=moe, mixer=memory), dict(type="latent_attention", mlp=moe, mixer=latents)]
+        puzorax = dict(architecture="Puzorax", vocab=vocab, width=D, norm=dict(eps=1e-5), max_positions=T + 1024, loop=dict(start=0, stop=min(2, L), times=2),
+                       embedding=dict(bigram=dict(buckets=65536, mul_prev=1009, mul_cur=31)), layers=(pair * ((L + 1) // 2))[:L])
+        record["sizes"][size] = {}
+        for name, cfg in (("llama", llama), ("rigalorn", rigalorn), ("zidevik", zidevik), ("puzorax", puzorax)):
+            if args.only and name not in args.only.split(","):
+                continue
+            record["sizes"][size][name] = _measure_design(cfg, args, T, batch, steps, vocab, gen)
+    print(json.dumps(record))
+    return 0
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -326,8 +372,9 @@ def main() -> int:
     ap.add_argument("--zidevik", action="store_true", help="another measurement: the Zidevik design beside Rigalorn and Llama at equal layer shapes (see zidevik_beside_rigalorn)")
     ap.add_argument("--mimitar", action="store_true", help="another measurement: the Mimitar design beside Zidevik, Rigalorn and Llama at equal layer shapes (see mimitar_beside_zidevik)")
     ap.add_argument("--vubenex", action="store_true", help="another measurement: the Vubenex design beside Fekorax and Llama at equal layer shapes (see vubenex_beside_fekorax)")
-    ap.add_argument("--only", default="", help="with --rigalorn, --zidevik, --mimitar or --vubenex: the designs to measure, of llama, fekorax, rigalorn, zidevik, mimitar, vubenex (default: all)")
-    ap.add_argument("--sizes", default="1b,8b", help="with --fekorax, --rigalorn, --zidevik, --mimitar or --vubenex: layer shapes, of " + ", ".join(FEKORAX_SIZES))
+    ap.add_argument("--puzorax", action="store_true", help="another measurement: the Puzorax design beside Rigalorn, Zidevik and Llama at equal layer shapes (see puzorax_beside_rigalorn)")
+    ap.add_argument("--only", default="", help="with --rigalorn, --zidevik, --mimitar, --vubenex or --puzorax: the designs to measure, of llama, fekorax, rigalorn, zidevik, mimitar, vubenex, puzorax (default: all)")
+    ap.add_argument("--sizes", default="1b,8b", help="with --fekorax, --rigalorn, --zidevik, --mimitar, --vubenex or --puzorax: layer shapes, of " + ", ".join(FEKORAX_SIZES))
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py measures one GPU; --gpus {args.gpus} is not supported by this single-GPU engine")
@@ -343,6 +390,8 @@ def main() -> int:
         return mimitar_beside_zidevik(args)
     if args.vubenex:
         return vubenex_beside_fekorax(args)
+    if args.puzorax:
+        return puzorax_beside_rigalorn(args)
 
     import torch
     from geneinfer_amd.config import LlamaConfig

@@ -425,7 +425,8 @@ __global__ __launch_bounds__(64) void delta_scan_kernel(const float* __restrict_
     // A block of TB tokens from `first` on (rows beyond the request's last are read as its last: finite, and never used).
     const int dn = CHANNEL ? dk : 1;             // decays a head
     const size_t ldg = (size_t)n_heads * (dn + 1);
-    item_t kq_reg[PER];
+    // The numbers stay as they come until they are laid into LDS: a condition or a product here would make the wave wait for each.
+    float k_reg[PER], q_reg[PER], d_reg[PER];
     float2 gb_reg;
     float v_reg;
     auto fetch = [&](int first) {
@@ -435,8 +436,7 @@ __global__ __launch_bounds__(64) void delta_scan_kernel(const float* __restrict_
             const size_t t = t0 + min(first + u, n - 1);
             const float* row = qkv + t * ld;
             const int ic = min(i, dk - 1);
-            const float kk = row[k_at + ic], qq = row[q_at + ic], dd = CHANNEL ? gates[t * ldg + h * dk + ic] : 0.f;
-            kq_reg[e] = i < dk ? delta_item((item_t*)nullptr, kk, qq, dd) : item_t{};
+            k_reg[e] = row[k_at + ic], q_reg[e] = row[q_at + ic], d_reg[e] = CHANNEL ? gates[t * ldg + h * dk + ic] : 0.f;
         }
         const int u = min(lane / C, TB - 1), cc = min(vt * C + lane % C, dv - 1);
         v_reg = qkv[(size_t)(t0 + min(first + u, n - 1)) * ld + v_at + cc];
@@ -446,8 +446,9 @@ __global__ __launch_bounds__(64) void delta_scan_kernel(const float* __restrict_
     auto stash = [&](int buf) {
 #pragma unroll
         for (int e = 0; e < PER; ++e) {
-            const int idx = lane + 64 * e;
-            kq_s[buf][idx / KQ][idx % KQ] = kq_reg[e];
+            const int idx = lane + 64 * e, i = idx % KQ, keep = i < dk ? -1 : 0;          // (zeros beyond the key, without a branch)
+            kq_s[buf][idx / KQ][i] = delta_item((item_t*)nullptr, __int_as_float(__float_as_int(k_reg[e]) & keep), __int_as_float(__float_as_int(q_reg[e]) & keep),
+                                                __int_as_float(__float_as_int(d_reg[e]) & keep));
         }
         if (lane < TB * C) v_s[buf][lane / C][lane % C] = v_reg;
         if (lane < TB) gb_s[buf][lane] = gb_reg;
@@ -460,13 +461,35 @@ __global__ __launch_bounds__(64) void delta_scan_kernel(const float* __restrict_
         const int here = min(TB, n - b0);
         const bool more = b0 + TB < n;
         if (more) fetch(b0 + TB);
-        for (int u = 0; u < here; ++u) {
-            const float2 gb = gb_s[buf][u];
-            item_t x[ROWS];
+        auto read = [&](int u, item_t (&x)[ROWS], float2& gb, float& v) {
 #pragma unroll
             for (int rr = 0; rr < ROWS; ++rr) x[rr] = kq_s[buf][u][rr * RG + rg];
-            const float y = delta_token<ROWS, CHANNEL>(S, x, v_s[buf][u][c], gb.x, gb.y);
+            gb = gb_s[buf][u], v = v_s[buf][u][c];
+        };
+        auto token = [&](int u, const item_t (&x)[ROWS], const float2& gb, float v) {
+            const float y = delta_token<ROWS, CHANNEL>(S, x, v, gb.x, gb.y);
             if (rg == 0 && live) out[(size_t)(t0 + b0 + u) * ldo + h * dv + col] = y;
+        };
+        if constexpr (ROWS <= 8) {               // a token's numbers leave LDS while the token before it is worked on
+            item_t xa[ROWS], xb[ROWS];
+            float2 ga, gb;
+            float va, vb;
+            read(0, xa, ga, va);
+            for (int u = 0; u < here; u += 2) {
+                read(min(u + 1, TB - 1), xb, gb, vb);
+                token(u, xa, ga, va);
+                if (u + 1 >= here) break;
+                read(min(u + 2, TB - 1), xa, ga, va);
+                token(u + 1, xb, gb, vb);
+            }
+        } else {
+            for (int u = 0; u < here; ++u) {
+                item_t x[ROWS];
+                float2 gb;
+                float v;
+                read(u, x, gb, v);
+                token(u, x, gb, v);
+            }
         }
         if (more) stash(buf ^ 1);                // (the buffer the block before this one was read from)
         barrier_lds();
