@@ -87,11 +87,18 @@ def latent_attention(h, w, m, eps, store=same):
     c = store(rms_norm(down[:, :rank], w["dkv.norm"], eps))
     k_rot = store(rotate_half_split(down[:, None, rank:], m["rot"]["base"]))[:, 0]
     q_plain, q_rot = store(q[..., :d]), store(rotate_half_split(q[..., d:], m["rot"]["base"]))
-    k = (c @ w["uk"].T).view(T, H, d)
-    v = (c @ w["uv"].T).view(T, H, dv)
-    scores = (torch.einsum("thd,shd->hts", q_plain, k) + torch.einsum("thr,sr->hts", q_rot, k_rot)) * m["scale"]
-    p = sink_softmax(scores, window_mask(T, m["mask"]["size"] if m.get("mask") else None), w["sink"])
-    o = torch.einsum("hts,shd->thd", p, v).reshape(T, H * dv)
+    seen = window_mask(T, m["mask"]["size"] if m.get("mask") else None)
+    rotated = torch.einsum("thr,sr->hts", q_rot, k_rot)
+    if store is same:
+        k = (c @ w["uk"].T).view(T, H, d)
+        v = (c @ w["uv"].T).view(T, H, dv)
+        p = sink_softmax((torch.einsum("thd,shd->hts", q_plain, k) + rotated) * m["scale"], seen, w["sink"])
+        o = torch.einsum("hts,shd->thd", p, v).reshape(T, H * dv)
+    else:       # the same with W_uk folded into the queries and W_uv applied behind the sum over keys, which is where an engine that caches c alone rounds
+        folded = store(torch.einsum("thd,hdc->thc", q_plain, w["uk"].view(H, d, rank)))
+        p = sink_softmax((torch.einsum("thc,sc->hts", folded, c) + rotated) * m["scale"], seen, w["sink"])
+        attended = store(torch.einsum("hts,sc->thc", store(p), c))
+        o = torch.einsum("thc,hvc->thv", attended, w["uv"].view(H, dv, rank)).reshape(T, H * dv)
     return store(o * torch.sigmoid(h @ w["g"].T)) @ w["o"].T
 
 
@@ -182,8 +189,8 @@ def forward(config, tensors, tokens, dtype=torch.float64, layer_outputs=None, st
     """Logits [T, vocab] of a whole sequence.  config: config.json as a dict; tensors: by name.  layer_outputs: a list that
     gets the residual stream after every layer run."""
     t = {k: (v.to(dtype) if v.is_floating_point() else v) for k, v in tensors.items()}
-    eps, bigram = config["norm"]["eps"], config["embedding"]["bigram"]
-    x0 = embedding(tokens, t["embed"], t["bigram"], bigram["mul_prev"], bigram["mul_cur"])
+    eps, bigram = config["norm"]["eps"], (config.get("embedding") or {}).get("bigram")
+    x0 = t["embed"][torch.as_tensor(list(tokens), dtype=torch.long)] if bigram is None else embedding(tokens, t["embed"], t["bigram"], bigram["mul_prev"], bigram["mul_cur"])
     x = x0
     short = lambda p: {k[len(p):]: v for k, v in t.items() if k.startswith(p)}
     parts = [(short(f"l{i}.mix."), short(f"l{i}.mlp.")) for i in range(len(config["layers"]))]
