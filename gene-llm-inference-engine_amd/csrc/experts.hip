@@ -21,6 +21,10 @@
 //   gi_experts_combine   x[row] (+)= the sum over the row's choices of the results at their places (times the score, where it
 //                        weighs the output), the choices one after the other; and, in the same kernel, the layer norm of the new row
 //                        for whoever reads it next
+// For the items of a few rows (decoding steps) in bfloat16 nothing is put in order:
+//   gi_experts_few       a workgroup per (strip of an expert's output rows, expert) finds the items that chose its expert, leaves if there
+//                        are none, and streams its strip of weights once past up to 16 of them on the matrix cores: the gated products into
+//                        mid[item], or the down products into y[item], which gi_experts_combine adds up
 // A number from `n_experts` on stands for an expert that returns its input: it has no weights, no item of it takes a place, and the
 // kernels that add the choices up take the row itself for its result.
 // Nothing of this asks the host how the router chose: the launches' shapes depend on the number of items and experts alone.
@@ -191,12 +195,12 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const TM* __restrict_
     if (lane == 0) x[row * ldx + c] = accumulate ? x[row * ldx + c] + total : total;
 }
 
-// The router's product and choice for one row: a workgroup of four waves; wave w makes the logits of experts w, w + 4, ..., every
-// one a lane's share of the columns in their order and then the lanes by a butterfly; the first wave then chooses as
+// The router's product and choice for one row: a workgroup of NW waves (four; more where the rows are few); wave w makes the logits of
+// experts w, w + NW, ..., every one a lane's share of the columns in their order and then the lanes by a butterfly; the first wave then chooses as
 // `route_top_kernel` does.
 constexpr int ROUTE_MAX_EXPERTS = 64 * ROUTE_PER_LANE;
-template <typename TA, typename TW>
-__global__ __launch_bounds__(256) void route_rows_kernel(const TA* __restrict__ h, long ldh, const TW* __restrict__ router, long ldr, int width, int n_experts, int top,
+template <typename TA, typename TW, int NW>
+__global__ __launch_bounds__(64 * NW) void route_rows_kernel(const TA* __restrict__ h, long ldh, const TW* __restrict__ router, long ldr, int width, int n_experts, int top,
                                                         int score_kind, int renormalize, float floor, int n_groups, int keep, const float* __restrict__ correction, float scale,
                                                         int* __restrict__ ids, float* __restrict__ weights,
                                                         float* __restrict__ logits_out, long ldl, int n_extra, float* __restrict__ extra_out, long lde) {
@@ -204,7 +208,7 @@ __global__ __launch_bounds__(256) void route_rows_kernel(const TA* __restrict__ 
     const size_t t = blockIdx.x;
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const TA* a = h + t * ldh;
-    for (int e = wave; e < n_experts + n_extra; e += 4) {          // (rows behind the experts': products of the same rows that are no expert's, kept for the caller)
+    for (int e = wave; e < n_experts + n_extra; e += NW) {          // (rows behind the experts': products of the same rows that are no expert's, kept for the caller)
         const TW* w = router + (size_t)e * ldr;
         // a lane takes eight neighbouring columns at a time, four such pieces asked for at once; the columns left over one by one
         float s = 0.f;
@@ -246,36 +250,50 @@ __device__ __forceinline__ int wave_sum_int(int v) {
     return v;
 }
 
-// One wave per expert: how many of the items chose it.
-__global__ __launch_bounds__(256) void experts_count_kernel(const int* __restrict__ ids, int n_items, int n_experts, int* __restrict__ count) {
-    const int e = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-    if (e >= n_experts) return;
+constexpr int PLACE_THREADS = 1024;        // of a workgroup that looks through all items for one expert
+
+// One workgroup per expert: how many of the items chose it.
+__global__ __launch_bounds__(PLACE_THREADS) void experts_count_kernel(const int* __restrict__ ids, int n_items, int* __restrict__ count) {
+    __shared__ int part[PLACE_THREADS / 64];
+    const int e = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     int c = 0;
-    for (int i = lane; i < n_items; i += 64) c += ids[i] == e ? 1 : 0;
+    for (int i = threadIdx.x; i < n_items; i += PLACE_THREADS) c += ids[i] == e ? 1 : 0;
     c = wave_sum_int(c);
-    if (lane == 0) count[e] = c;
+    if (lane == 0) part[wave] = c;
+    __syncthreads();
+    if (threadIdx.x == 0) {
+        for (int w = 1; w < PLACE_THREADS / 64; ++w) c += part[w];
+        count[e] = c;
+    }
 }
 
-// One wave per expert: where its run begins (behind the runs of the experts before it, each filled up to whole tiles), its tiles'
-// entries, and its items' places in their order.  The last expert's wave also marks the tiles behind all runs as not in use.
-__global__ __launch_bounds__(256) void experts_place_kernel(const int* __restrict__ ids, int n_items, int n_experts, const int* __restrict__ count,
-                                                           int* __restrict__ place, int* __restrict__ tile_expert, int n_tiles) {
-    const int e = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-    if (e >= n_experts) return;
+// One workgroup per expert: where its run begins (behind the runs of the experts before it, each filled up to whole tiles), its tiles'
+// entries, and its items' places in their order.  The last expert's workgroup also marks the tiles behind all runs as not in use.
+__global__ __launch_bounds__(PLACE_THREADS) void experts_place_kernel(const int* __restrict__ ids, int n_items, int n_experts, const int* __restrict__ count,
+                                                                     int* __restrict__ place, int* __restrict__ tile_expert, int n_tiles) {
+    __shared__ int hits[2][PLACE_THREADS / 64];
+    const int e = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     int before = 0;
     for (int o = lane; o < e; o += 64) before += (count[o] + EXPERT_TILE - 1) / EXPERT_TILE;
     before = wave_sum_int(before);
     const int mine = (count[e] + EXPERT_TILE - 1) / EXPERT_TILE;
-    for (int j = lane; j < mine; j += 64) tile_expert[before + j] = e;
+    for (int j = threadIdx.x; j < mine; j += PLACE_THREADS) tile_expert[before + j] = e;
     if (e == n_experts - 1)
-        for (int j = before + mine + lane; j < n_tiles; j += 64) tile_expert[j] = -1;
-    int at = before * EXPERT_TILE;
-    for (int i0 = 0; i0 < n_items; i0 += 64) {
-        const int i = i0 + lane;
+        for (int j = before + mine + threadIdx.x; j < n_tiles; j += PLACE_THREADS) tile_expert[j] = -1;
+    int at = before * EXPERT_TILE, turn = 0;
+    for (int i0 = 0; i0 < n_items; i0 += PLACE_THREADS, turn ^= 1) {      // (every thread of the workgroup walks every round)
+        const int i = i0 + threadIdx.x;
         const bool hit = i < n_items && ids[i] == e;
         const unsigned long long all = __ballot(hit);
-        if (hit) place[i] = at + __popcll(all & ((1ull << lane) - 1ull));
-        at += __popcll(all);
+        if (lane == 0) hits[turn][wave] = __popcll(all);
+        __syncthreads();
+        int ahead = 0, total = 0;
+        for (int w = 0; w < PLACE_THREADS / 64; ++w) {
+            if (w < wave) ahead += hits[turn][w];
+            total += hits[turn][w];
+        }
+        if (hit) place[i] = at + ahead + __popcll(all & ((1ull << lane) - 1ull));
+        at += total;
     }
 }
 
@@ -312,10 +330,91 @@ __global__ __launch_bounds__(256) void experts_combine_kernel(const float* __res
             total += weights[item] * load_f32(h, row * ldh + c);
             continue;
         }
-        const float v = y[(size_t)place[item] * ldy + c];
+        const float v = y[(place ? (size_t)place[item] : item) * ldy + c];
         total += weigh_output ? weights[item] * v : v;
     }
     x[row * ldx + c] = accumulate ? x[row * ldx + c] + total : total;
+}
+
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef float floatx4 __attribute__((ext_vector_type(4)));
+__device__ __forceinline__ bf16x8 as_bf16x8(uint4 v) { return __builtin_bit_cast(bf16x8, v); }
+
+// One workgroup: 32 rows of expert blockIdx.y's matrix w [rows][K] (two strips of 16: a group of gates and the group of up products behind
+// it, or 32 neighbouring outputs) against the items that chose the expert, 16 at a time as the columns of the 16x16x32 matrix instruction.
+// The eight waves share K out in blocks of 64 (a row's four lanes read 128 contiguous bytes) and add their sums through LDS, in their order.
+constexpr int FEW_MAX_ITEMS = 256;
+template <bool GATED>
+__global__ __launch_bounds__(512) void experts_few_kernel(const bf16_t* __restrict__ a, long lda, int per_row, const int* __restrict__ ids, const float* __restrict__ weigh, int n_items,
+                                                         const bf16_t* __restrict__ w, int K, int n_out, void* __restrict__ out, long ldo, int act, float limit) {
+    constexpr int NW = 8, UB = 2;                        // waves; blocks of k asked for at a time
+    __shared__ int list[FEW_MAX_ITEMS], n_mine;
+    __shared__ float red[NW][8][64];
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r = lane & 15, q4 = lane >> 4;
+    const int e = blockIdx.y, row0 = blockIdx.x * 32, rows = GATED ? 2 * n_out : n_out;
+    if (wave == 0) {
+        int count = 0;
+        for (int base = 0; base < n_items; base += 64) {
+            const bool hit = base + lane < n_items && ids[base + lane] == e;
+            const unsigned long long all = __ballot(hit);
+            if (hit) list[count + __popcll(all & ((1ull << lane) - 1ull))] = base + lane;
+            count += __popcll(all);
+        }
+        if (lane == 0) n_mine = count;
+    }
+    __syncthreads();
+    const int n = n_mine;
+    if (n == 0) return;                                  // (the whole workgroup)
+    const bf16_t* w0 = w + ((size_t)e * rows + min(row0 + r, rows - 1)) * K;
+    const bf16_t* w1 = w + ((size_t)e * rows + min(row0 + 16 + r, rows - 1)) * K;
+    for (int c0 = 0; c0 < n; c0 += 16) {
+        const int item = list[min(c0 + r, n - 1)];
+        const bf16_t* arow = a + (size_t)(item / per_row) * lda;
+        const float s = weigh ? weigh[item] : 1.0f;
+        floatx4 acc0 = floatx4{}, acc1 = floatx4{};
+        for (int k0 = wave * 64; k0 < K; k0 += NW * 64 * UB) {
+            uint4 av[2 * UB], v0[2 * UB], v1[2 * UB];
+#pragma unroll
+            for (int u = 0; u < 2 * UB; ++u) {
+                const int k = min(k0 + (u >> 1) * NW * 64 + 16 * q4 + 8 * (u & 1), K - 8);          // (K is a multiple of 8; pieces beyond it are zeroed below)
+                v0[u] = *reinterpret_cast<const uint4*>(w0 + k);
+                v1[u] = *reinterpret_cast<const uint4*>(w1 + k);
+                av[u] = *reinterpret_cast<const uint4*>(arow + k);
+            }
+#pragma unroll
+            for (int u = 0; u < 2 * UB; ++u) {
+                const int k = k0 + (u >> 1) * NW * 64 + 16 * q4 + 8 * (u & 1);
+                uint32_t* p = reinterpret_cast<uint32_t*>(&av[u]);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    if (weigh) p[i] = f32x2_to_bf16x2(s * __uint_as_float(p[i] << 16), s * __uint_as_float(p[i] & 0xffff0000u));
+                    p[i] = k < K ? p[i] : 0u;
+                }
+                acc0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(v0[u]), as_bf16x8(av[u]), acc0, 0, 0, 0);
+                acc1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(v1[u]), as_bf16x8(av[u]), acc1, 0, 0, 0);
+            }
+        }
+        // element v of an accumulator: output row 4*q4 + v of its strip, item c0 + r
+#pragma unroll
+        for (int v = 0; v < 4; ++v) red[wave][v][lane] = acc0[v], red[wave][4 + v][lane] = acc1[v];
+        __syncthreads();
+        if (tid < 256) {
+            const int l = tid & 63, v = tid >> 6, c = c0 + (l & 15), row = 4 * (l >> 4) + v;
+            float x = 0.f, y = 0.f;
+#pragma unroll
+            for (int i = 0; i < NW; ++i) x += red[i][v][l], y += red[i][4 + v][l];
+            if (c < n) {
+                const size_t at = (size_t)list[c] * ldo;
+                if constexpr (GATED) {
+                    store_f32((bf16_t*)out, at + blockIdx.x * 16 + row, gated_act(x, y, act, limit));
+                } else {
+                    if (row0 + row < n_out) ((float*)out)[at + row0 + row] = x;
+                    if (row0 + 16 + row < n_out) ((float*)out)[at + row0 + 16 + row] = y;
+                }
+            }
+        }
+        __syncthreads();
+    }
 }
 
 __device__ __forceinline__ float4 four(const float* p) { return *reinterpret_cast<const float4*>(p); }
@@ -349,10 +448,11 @@ __global__ __launch_bounds__(256) void experts_combine_norm_kernel(const float* 
     for (int k = 0; k < top; ++k) {
         const size_t item = row * top + k;
         const bool itself = ids[item] >= n_experts;      // (the same for the whole workgroup)
+        const size_t from = itself ? 0 : place ? (size_t)place[item] : item;
         const float s = itself || weigh_output ? weights[item] : 1.0f;
 #pragma unroll
         for (int i = 0; i < PER; ++i) {
-            const float4 r = itself ? four(h + row * ldh + at[i]) : four(y + (size_t)place[item] * ldy + at[i]);
+            const float4 r = itself ? four(h + row * ldh + at[i]) : four(y + from * ldy + at[i]);
             total[i].x += s * r.x; total[i].y += s * r.y; total[i].z += s * r.z; total[i].w += s * r.w;
         }
     }
@@ -446,13 +546,19 @@ GI_API int gi_route_rows(const void* h, int h_dtype, long ldh, const void* route
     GI_REQUIRE(n_rows > 0 && width > 0 && n_experts > 0 && n_experts <= ROUTE_MAX_EXPERTS && top > 0 && top <= n_experts && top <= 64 && ldh >= width && ldr >= width
                && (score_kind == 0 || score_kind == 1) && (logits == nullptr || ldl >= n_experts),
                "route_rows: bad sizes (rows %d, width %d, experts %d, top %d)", n_rows, width, n_experts, top);
-#define LAUNCH(TA, TW) route_rows_kernel<TA, TW><<<n_rows, 256, 0, stream>>>((const TA*)h, ldh, (const TW*)router, ldr, width, n_experts, top, score_kind, renormalize, floor, n_groups, keep, correction, scale, ids, weights, logits, ldl, n_extra, extra, lde)
+#define LAUNCH_NW(TA, TW, NW) route_rows_kernel<TA, TW, NW><<<n_rows, 64 * NW, 0, stream>>>((const TA*)h, ldh, (const TW*)router, ldr, width, n_experts, top, score_kind, renormalize, floor, n_groups, keep, correction, scale, ids, weights, logits, ldl, n_extra, extra, lde)
+#define LAUNCH(TA, TW)                            \
+    do {                                          \
+        if (n_rows <= 64) LAUNCH_NW(TA, TW, 16);  \
+        else LAUNCH_NW(TA, TW, 4);                \
+    } while (0)
     if (h_dtype == GI_BF16 && r_dtype == GI_BF16) LAUNCH(bf16_t, bf16_t);
     else if (h_dtype == GI_F32 && r_dtype == GI_F32) LAUNCH(float, float);
     else if (h_dtype == GI_F32 && r_dtype == GI_BF16) LAUNCH(float, bf16_t);
     else if (h_dtype == GI_BF16 && r_dtype == GI_F32) LAUNCH(bf16_t, float);
     else return gi_fail("route_rows: unknown dtypes %d, %d", h_dtype, r_dtype);
 #undef LAUNCH
+#undef LAUNCH_NW
     GI_CHECK_LAUNCH("route_rows");
     return 0;
 }
@@ -463,9 +569,9 @@ GI_API int gi_experts_tile_rows() { return EXPERT_TILE; }
 GI_API int gi_experts_place(const int* ids, int n_items, int n_experts, int* count, int* place, int* tile_expert, int n_tiles, hipStream_t stream) {
     GI_REQUIRE(n_items > 0 && n_experts > 0 && (long)n_tiles * EXPERT_TILE >= (long)n_items + (long)n_experts * (EXPERT_TILE - 1) - (EXPERT_TILE - 1),
                "experts_place: bad sizes (items %d, experts %d, tiles %d)", n_items, n_experts, n_tiles);
-    experts_count_kernel<<<(n_experts + 3) / 4, 256, 0, stream>>>(ids, n_items, n_experts, count);
+    experts_count_kernel<<<n_experts, PLACE_THREADS, 0, stream>>>(ids, n_items, count);
     GI_CHECK_LAUNCH("experts_count");
-    experts_place_kernel<<<(n_experts + 3) / 4, 256, 0, stream>>>(ids, n_items, n_experts, count, place, tile_expert, n_tiles);
+    experts_place_kernel<<<n_experts, PLACE_THREADS, 0, stream>>>(ids, n_items, n_experts, count, place, tile_expert, n_tiles);
     GI_CHECK_LAUNCH("experts_place");
     return 0;
 }
@@ -479,6 +585,23 @@ GI_API int gi_experts_gather(const void* h, long ldh, const int* ids, const int*
     return 0;
 }
 
+// gated: w [n_experts][2 n_out][K] (groups of 16 gate rows and 16 up rows in turns), out bfloat16 [n_items, ldo]; otherwise w [n_experts][n_out][K], out
+// float32.  Item i's input is row i / per_row of a, times weigh[i] (nullptr: as it is).
+GI_API int gi_experts_few_max_items() { return FEW_MAX_ITEMS; }
+
+GI_API int gi_experts_few(const void* a, long lda, int per_row, const int* ids, const float* weigh, int n_items, int n_experts, const void* w, int K, int n_out, int gated, void* out,
+                          long ldo, int act, float limit, hipStream_t stream) {
+    GI_REQUIRE(n_items > 0 && n_items <= FEW_MAX_ITEMS && per_row > 0 && n_experts > 0 && n_experts <= 65535 && K > 0 && K % 8 == 0 && n_out > 0 && lda % 8 == 0 && lda >= K && ldo >= n_out &&
+               (!gated || n_out % 16 == 0) && act >= 0 && act < GI_N_ACTIVATIONS && (((uintptr_t)a | (uintptr_t)w) & 15) == 0,
+               "experts_few: bad sizes (items %d, experts %d, k %d, outputs %d) or alignment", n_items, n_experts, K, n_out);
+    dim3 grid(gated ? n_out / 16 : (n_out + 31) / 32, n_experts);
+    if (gated) experts_few_kernel<true><<<grid, 512, 0, stream>>>((const bf16_t*)a, lda, per_row, ids, weigh, n_items, (const bf16_t*)w, K, n_out, out, ldo, act, limit);
+    else experts_few_kernel<false><<<grid, 512, 0, stream>>>((const bf16_t*)a, lda, per_row, ids, weigh, n_items, (const bf16_t*)w, K, n_out, out, ldo, act, limit);
+    GI_CHECK_LAUNCH("experts_few");
+    return 0;
+}
+
+// place nullptr: item i's result is row i of y.
 // norm_w, norm_b, out: also the layer norm of the new rows as bfloat16 (nullptr: none); widths gi_experts_combine_norm_takes names, rows at multiples of 16 bytes.
 GI_API int gi_experts_combine_norm_takes(int width) { return width > 0 && width % 4 == 0 && width <= 8192; }
 

@@ -127,6 +127,7 @@ __global__ __launch_bounds__(64) void heads_product_kernel(const bf16_t* __restr
     const bf16_t* arow = a + (size_t)row * lda + (size_t)h * k_dim;
     const bf16_t* wh = w + (size_t)h * n_out * k_dim;
     floatx4 acc[4] = {floatx4{}, floatx4{}, floatx4{}, floatx4{}};
+#pragma unroll 4
     for (int k0 = 0; k0 < k_dim; k0 += 32) {
         const int k = k0 + 8 * q4;
         const bool in = k < k_dim;                       // (k_dim is a multiple of 8: a piece is inside or outside as a whole)

@@ -71,6 +71,27 @@ __device__ __forceinline__ float group_sum(float x) {
     return x;
 }
 
+// w . l with the numbers of l rounded to bfloat16 as a product's rows are: one output of a product behind a narrow middle, made by one
+// lane, eight weights a load where the row allows it.  One ascending sum.
+__device__ __forceinline__ float narrow_dot(const float* __restrict__ l, const bf16_t* __restrict__ w, int rank) {
+    float a = 0.f;
+    if (rank % 8 == 0 && ((uintptr_t)w & 15) == 0) {
+#pragma unroll 4
+        for (int r = 0; r < rank; r += 8) {
+            const uint4 v = *reinterpret_cast<const uint4*>(w + r);
+            const uint32_t p[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                a = fmaf(bf16_to_f32(f32_to_bf16(l[r + 2 * i])), __uint_as_float(p[i] << 16), a);
+                a = fmaf(bf16_to_f32(f32_to_bf16(l[r + 2 * i + 1])), __uint_as_float(p[i] & 0xffff0000u), a);
+            }
+        }
+        return a;
+    }
+    for (int r = 0; r < rank; ++r) a = fmaf(bf16_to_f32(f32_to_bf16(l[r])), bf16_to_f32(w[r]), a);
+    return a;
+}
+
 __device__ __forceinline__ float log_sigmoid(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
 
 template <int ROWS>
@@ -225,16 +246,7 @@ __global__ __launch_bounds__(64) void head_norm_gate_kernel(const float* __restr
     const float r = 1.0f / sqrtf(wave_sum(ss) / (float)dv + eps);
     for (int d = lane; d < dv; d += 64) {
         const float v = den ? orow[d] / by : orow[d];
-        float z;
-        if (low) {
-            const float* l = low + (size_t)t * ldg;
-            const bf16_t* wz = w_up + ((size_t)h * dv + d) * rank;
-            z = 0.f;
-#pragma unroll 8
-            for (int i = 0; i < rank; ++i) z = fmaf(bf16_to_f32(f32_to_bf16(l[i])), bf16_to_f32(wz[i]), z);
-        } else {
-            z = g[(size_t)t * ldg + (size_t)h * dv + d];
-        }
+        const float z = low ? narrow_dot(low + (size_t)t * ldg, w_up + ((size_t)h * dv + d) * rank, rank) : g[(size_t)t * ldg + (size_t)h * dv + d];
         const float gate = (gate_act ? z : 1.0f) / (1.0f + expf(-z));
         store_f32(y, (size_t)t * ldy + (size_t)h * dv + d, load_f32(w, (size_t)h * w_head_stride + d) * (v * r) * gate);
     }
@@ -277,16 +289,7 @@ __global__ __launch_bounds__(64) void delta_prepare_kernel(const float* __restri
         const int h0 = dn > 1 ? item - 2 * n_kv - n_heads : 0, h1 = dn > 1 ? h0 + 1 : n_heads;
         float* out = gates + (size_t)t * n_heads * (dn + 1);
         for (int i = h0 * dn + lane; i < h1 * dn; i += 64) {
-            float a;
-            if (low) {
-                a = 0.f;
-                const float* l = low + (size_t)t * ld;
-                const bf16_t* w = w_up + (size_t)i * rank;
-#pragma unroll 8
-                for (int r = 0; r < rank; ++r) a = fmaf(bf16_to_f32(f32_to_bf16(l[r])), bf16_to_f32(w[r]), a);
-            } else {
-                a = pre_a[(size_t)t * lda + i];
-            }
+            const float a = low ? narrow_dot(low + (size_t)t * ld, w_up + (size_t)i * rank, rank) : pre_a[(size_t)t * lda + i];
             out[i] = expf(-expf(a_log[i / dn]) * softplus_f(a + dt_bias[i]));
         }
         for (int h = h0 + lane; h < h1; h += 64) out[n_heads * dn + h] = 1.0f / (1.0f + expf(-proj[(size_t)t * ld + b_off + h]));
@@ -466,29 +469,26 @@ __global__ __launch_bounds__(64) void delta_scan_kernel(const float* __restrict_
             for (int rr = 0; rr < ROWS; ++rr) x[rr] = kq_s[buf][u][rr * RG + rg];
             gb = gb_s[buf][u], v = v_s[buf][u][c];
         };
-        auto token = [&](int u, const item_t (&x)[ROWS], const float2& gb, float v) {
-            const float y = delta_token<ROWS, CHANNEL>(S, x, v, gb.x, gb.y);
-            if (rg == 0 && live) out[(size_t)(t0 + b0 + u) * ldo + h * dv + col] = y;
-        };
-        if constexpr (ROWS <= 8) {               // a token's numbers leave LDS while the token before it is worked on
-            item_t xa[ROWS], xb[ROWS];
-            float2 ga, gb;
-            float va, vb;
-            read(0, xa, ga, va);
-            for (int u = 0; u < here; u += 2) {
-                read(min(u + 1, TB - 1), xb, gb, vb);
-                token(u, xa, ga, va);
-                if (u + 1 >= here) break;
-                read(min(u + 2, TB - 1), xa, ga, va);
-                token(u + 1, xb, gb, vb);
+        if (ROWS <= 8 && here == TB) {           // a whole block: straight code, tokens' numbers leave LDS ahead of their turn, the results one store
+            float mine = 0.f;                    // (the lanes of a column hold equal results: lane u of it keeps token u's)
+#pragma unroll
+            for (int u = 0; u < TB; ++u) {
+                item_t x[ROWS];
+                float2 gb;
+                float v;
+                read(u, x, gb, v);
+                const float y = delta_token<ROWS, CHANNEL>(S, x, v, gb.x, gb.y);
+                mine = rg == u ? y : mine;
             }
+            if (rg < TB && live) out[(size_t)(t0 + b0 + rg) * ldo + h * dv + col] = mine;
         } else {
             for (int u = 0; u < here; ++u) {
                 item_t x[ROWS];
                 float2 gb;
                 float v;
                 read(u, x, gb, v);
-                token(u, x, gb, v);
+                const float y = delta_token<ROWS, CHANNEL>(S, x, v, gb.x, gb.y);
+                if (rg == 0 && live) out[(size_t)(t0 + b0 + u) * ldo + h * dv + col] = y;
             }
         }
         if (more) stash(buf ^ 1);                // (the buffer the block before this one was read from)

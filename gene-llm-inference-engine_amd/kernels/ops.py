@@ -59,6 +59,7 @@ _SIGNATURES = {
     "gi_experts_gather": [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_long, c_int, c_int, c_void_p],
     "gi_experts_combine": [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_long, c_int, c_int, c_void_p, c_long, c_int, c_void_p, c_void_p, c_int, c_float,
                            c_void_p, c_long, c_void_p],
+    "gi_experts_few": [c_void_p, c_long, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_long, c_int, c_float, c_void_p],
     "gi_layernorm": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_float, c_long, c_long, c_long, c_void_p],
     "gi_embed_pairs": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_long, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p],
     "gi_latent_direct": [c_void_p, c_long, c_void_p, c_long, c_void_p, c_int, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_long, c_void_p, c_long,
@@ -1630,6 +1631,9 @@ def latent_attention_bf16_supports(kd, vd, page_size) -> bool:
     return bool(lib().gi_latent_attention_supports(kd, vd, page_size))
 
 
+LATENT_MAX_SPLITS, LATENT_WAVES, LATENT_SHARE = 64, 2048, 32          # how far a few rows' contexts are shared out: shares a row, waves in all, positions a share at least
+
+
 def latent_attention_prepare():
     """Once, outside any captured pass: the prompt kernel's LDS (more than the default limit) is asked for."""
     if lib().gi_latent_attention_tiles_prepare() != 0:
@@ -1665,7 +1669,7 @@ def latent_attention_bf16(q, cache, out, ctx, table, n_heads, kd, vd, page_size,
     if window:
         span = min(span, int(window) + 31)
     groups = n_single * (-(-n_heads // 16))
-    n_splits = max(1, min(16, 2048 // groups, (span + 63) // 64))
+    n_splits = max(1, min(LATENT_MAX_SPLITS, LATENT_WAVES // groups, (span + LATENT_SHARE - 1) // LATENT_SHARE))
     n_part = n_single * n_heads * n_splits * (vd + 2) if n_splits > 1 else 0
     part = torch.empty(n_part, dtype=torch.float32, device=out.device) if n_part else None
     _call("gi_latent_attention_bf16", q.data_ptr(), cache.data_ptr(), out.data_ptr(), _ptr(part), n_part, _ptr(rows), ctx.row_pos.data_ptr(), ctx.row_slot.data_ptr(),
@@ -1868,6 +1872,7 @@ ROUTER_MAX_EXPERTS, ROUTER_MAX_TOP = 1024, 64
 EXPERT_ROW_GROUP = 16          # rows of a group where an expert's gates and up products lie in one matrix (`interleave_gate_up`)
 EXPERT_TILE_ROWS = 128         # rows of a tile of the product for grouped rows (the library's gi_experts_tile_rows)
 EXPERTS_GROUPED_FROM = 8       # (row, choice) items from which the experts' rows are grouped for the matrix cores
+EXPERTS_FEW_ITEMS = 64         # ... and up to which a workgroup per strip of an expert's rows picks its items itself, where that kernel takes the sizes
 
 
 def _router_groups(what, n_experts, top, groups):
@@ -2008,16 +2013,58 @@ def experts_grouped_supported(h, w_gate, w_up, w_down) -> bool:
     return width % 64 == 0 and ff % 64 == 0 and width >= 128 and 2 * ff >= 128 and h.stride(0) % 8 == 0 and h.data_ptr() % 16 == 0
 
 
+def experts_few_supported(h, w_gate, w_up, w_down) -> bool:
+    """Whether `routed_experts` can take a few items through the kernel that streams an expert's weights once past all items that chose it."""
+    if w_up is not None or not (h.dtype == w_gate.dtype == w_down.dtype == torch.bfloat16):
+        return False
+    return h.shape[1] % 8 == 0 and w_down.shape[2] % EXPERT_ROW_GROUP == 0 and h.stride(0) % 8 == 0 and h.data_ptr() % 16 == 0
+
+
+def experts_few(a, per_row, ids, weigh, w, out, gated=False, limit=0.0):
+    """out[item] = w[e] @ (weigh[item] *) a[item // per_row] for every (row, choice) item with e = ids[item] < experts; gated (an activation's
+    name): w holds gates and up products in turns (`interleave_gate_up`) and out, bfloat16, is act(gate) * up; otherwise out is float32."""
+    _dev(a, ids, weigh, w, out)
+    n_items, K = ids.numel(), w.shape[2]
+    n_out = w.shape[1] // 2 if gated else w.shape[1]
+    if not (a.dtype == w.dtype == torch.bfloat16 and w.dim() == 3 and w.is_contiguous() and a.shape[1] == K and a.stride(1) == 1 and a.shape[0] * per_row >= n_items
+            and out.shape == (n_items, n_out) and out.stride(1) == 1 and out.dtype == (torch.bfloat16 if gated else torch.float32)):
+        raise KernelError("experts_few: a bfloat16 [rows, k], w bfloat16 [experts, outputs, k] and out [items, outputs] are needed")
+    if weigh is not None and not (weigh.dtype == torch.float32 and weigh.is_contiguous() and weigh.numel() == n_items):
+        raise KernelError("experts_few: the weights must be float32, one an item")
+    _i32(ids, "experts_few: ids", n_items)
+    if _profile is not None:
+        _profile.note = (f"{n_items} of {w.shape[0]}x{w.shape[1]}x{K}{' gated' if gated else ''}", min(n_items, w.shape[0]) * w.shape[1] * K * 2)
+    _call("gi_experts_few", a.data_ptr(), a.stride(0), int(per_row), ids.data_ptr(), _ptr(weigh), n_items, w.shape[0], w.data_ptr(), K, n_out, 1 if gated else 0, out.data_ptr(), out.stride(0),
+          ACTIVATIONS[gated] if gated else 0, float(limit), _stream())
+    return out
+
+
 def experts_combine_norm_takes(x, h) -> bool:
     """Whether the kernel that adds the experts' results onto these rows also takes a layer norm behind it."""
     return (bool(lib().gi_experts_combine_norm_takes(x.shape[1])) and x.stride(0) % 4 == 0 and h.stride(0) % 4 == 0 and x.data_ptr() % 16 == 0 and h.data_ptr() % 16 == 0)
 
 
+def _experts_combine(y, ids, place, weights, weigh, x, accumulate, h, n_experts, then):
+    """x[row] (+)= the sum over the row's choices of y at their places (place None: at the items' own numbers); with `then` the norm's rows."""
+    (n, top), width = ids.shape, x.shape[1]
+    norm_w, norm_b, eps, low = None, None, 0.0, None
+    if then is not None and experts_combine_norm_takes(x, h):
+        norm_w, norm_b, eps = then
+        if not (norm_w.shape == norm_b.shape == (width,) and norm_w.is_contiguous() and norm_b.is_contiguous() and norm_w.dtype == norm_b.dtype
+                and norm_w.data_ptr() % 16 == 0 and norm_b.data_ptr() % 16 == 0):
+            raise KernelError("routed_experts: the norm behind needs weight and bias [width] of one dtype, aligned")
+        low = torch.empty((n, width), dtype=torch.bfloat16, device=x.device)
+    _call("gi_experts_combine", y.data_ptr(), y.stride(0), ids.data_ptr(), _ptr(place), weights.data_ptr(), 1 if weigh == "output" else 0, n, top, x.data_ptr(), x.stride(0),
+          width, 1 if accumulate else 0, h.data_ptr(), h.stride(0), n_experts, _ptr(norm_w), _ptr(norm_b), _code(norm_w, "routed_experts: norm") if low is not None else F32, float(eps),
+          _ptr(low), low.stride(0) if low is not None else 0, _stream())
+    return low
+
+
 def routed_experts(h, w_gate, w_up, w_down, ids, weights, x, accumulate=True, weigh="input", activation="silu", limit=0.0, then=None):
     """x[row] (+)= sum over the row's choices of expert(a): the whole mixture behind the router's choice.  weigh "input": a = weight * h[row]
     (stored as h's dtype); "output": a = h[row] and the weight multiplies the expert's result.  w_up None: w_gate holds both (see
-    `experts_gate_up`).  Few items, or 32-bit operands: every item walks its expert's matrices.  Many in bfloat16: the items' rows are
-    put in the order of their experts and all experts' products are two launches on the matrix cores.  A number from `experts` on in ids
+    `experts_gate_up`).  32-bit operands: every item walks its expert's matrices.  A few items in bfloat16: every expert's weights are
+    streamed once past the items that chose it.  Many: the items' rows are put in the order of their experts and all experts' products are two launches on the matrix cores.  A number from `experts` on in ids
     stands for an expert that returns its input (times the choice's weight, whichever `weigh` is).
     then = (weight, bias, eps), the layer norm that reads x next: where the kernel that adds the results up makes its rows on the way
     (bfloat16 [n, width]), they are returned; None otherwise."""
@@ -2026,15 +2073,20 @@ def routed_experts(h, w_gate, w_up, w_down, ids, weights, x, accumulate=True, we
     n, top = ids.shape
     n_experts, width = w_down.shape[0], w_down.shape[1]
     ff = w_down.shape[2]
-    if n * top >= EXPERTS_GROUPED_FROM and activation in FUSED_GATE_ACTIVATIONS and experts_grouped_supported(h, w_gate, w_up, w_down):
+    few = n * top <= EXPERTS_FEW_ITEMS and experts_few_supported(h, w_gate, w_up, w_down)
+    if few or (n * top >= EXPERTS_GROUPED_FROM and activation in FUSED_GATE_ACTIVATIONS and experts_grouped_supported(h, w_gate, w_up, w_down)):
         _dev(h, w_gate, w_down, ids, weights, x)
         _f32_rows(x, "routed_experts: x", n, width)
         if not (ids.dtype == torch.int32 and ids.is_contiguous() and weights.dtype == torch.float32 and weights.shape == (n, top) and weights.is_contiguous()
                 and w_gate.shape == (n_experts, 2 * ff, width) and h.shape == (n, width)):
             raise KernelError("routed_experts: ids int32 and weights float32 [n, top], gates and up products [experts, 2 ff, width] are needed")
+        dev = h.device
+        if few:
+            mid = experts_few(h, top, ids, weights if weigh == "input" else None, w_gate, torch.empty((n * top, ff), dtype=torch.bfloat16, device=dev), gated=activation, limit=limit)
+            y, place = experts_few(mid, 1, ids, None, w_down, torch.empty((n * top, width), dtype=torch.float32, device=dev)), None
+            return _experts_combine(y, ids, place, weights, weigh, x, accumulate, h, n_experts, then)
         tile = EXPERT_TILE_ROWS
         n_tiles = max(1, (n * top + n_experts * (tile - 1)) // tile)
-        dev = h.device
         book = torch.empty(n_experts + n * top + n_tiles, dtype=torch.int32, device=dev)
         count, place, tile_expert = book[:n_experts], book[n_experts:n_experts + n * top], book[n_experts + n * top:]
         _call("gi_experts_place", ids.data_ptr(), n * top, n_experts, count.data_ptr(), place.data_ptr(), tile_expert.data_ptr(), n_tiles, _stream())
@@ -2045,17 +2097,7 @@ def routed_experts(h, w_gate, w_up, w_down, ids, weights, x, accumulate=True, we
         gemm_bf16_grouped(rows, w_gate, mid, tile_expert, gated=True if activation == "silu" else activation, gate_limit=limit)
         y = torch.empty((n_tiles * tile, width), dtype=torch.float32, device=dev)
         gemm_bf16_grouped(mid, w_down, y, tile_expert)
-        norm_w, norm_b, eps, low = None, None, 0.0, None
-        if then is not None and experts_combine_norm_takes(x, h):
-            norm_w, norm_b, eps = then
-            if not (norm_w.shape == norm_b.shape == (width,) and norm_w.is_contiguous() and norm_b.is_contiguous() and norm_w.dtype == norm_b.dtype
-                    and norm_w.data_ptr() % 16 == 0 and norm_b.data_ptr() % 16 == 0):
-                raise KernelError("routed_experts: the norm behind needs weight and bias [width] of one dtype, aligned")
-            low = torch.empty((n, width), dtype=torch.bfloat16, device=dev)
-        _call("gi_experts_combine", y.data_ptr(), y.stride(0), ids.data_ptr(), place.data_ptr(), weights.data_ptr(), 1 if weigh == "output" else 0, n, top, x.data_ptr(), x.stride(0),
-              width, 1 if accumulate else 0, h.data_ptr(), h.stride(0), n_experts, _ptr(norm_w), _ptr(norm_b), _code(norm_w, "routed_experts: norm") if low is not None else F32, float(eps),
-              _ptr(low), low.stride(0) if low is not None else 0, _stream())
-        return low
+        return _experts_combine(y, ids, place, weights, weigh, x, accumulate, h, n_experts, then)
     mid_dtype = torch.float32 if w_down.dtype == torch.float32 else h.dtype
     mid = torch.empty((n * top, ff), dtype=mid_dtype, device=h.device)
     experts_gate_up(h, w_gate, w_up, ids, weights, mid, weigh_input=weigh == "input", activation=activation, limit=limit)

@@ -413,7 +413,9 @@ def test_the_router_s_choice_with_a_correction(experts, identity, top):
 
 @pytest.mark.parametrize("rows, d, ff, E, identity, top, dtype", [(7, 50, 10, 3, 2, 3, "float32"), (1, 64, 24, 5, 1, 2, "float32"), (33, 128, 64, 8, 2, 3, "bfloat16"),
                                                                   (150, 256, 96, 4, 1, 2, "bfloat16"), (300, 128, 128, 16, 4, 4, "bfloat16"), (2, 128, 64, 4, 1, 2, "bfloat16"),
-                                                                  (700, 192, 320, 5, 3, 1, "bfloat16"), (20, 128, 64, 1, 5, 2, "bfloat16"), (9, 2112, 64, 3, 1, 2, "bfloat16")])
+                                                                  (700, 192, 320, 5, 3, 1, "bfloat16"), (20, 128, 64, 1, 5, 2, "bfloat16"), (9, 2112, 64, 3, 1, 2, "bfloat16"),
+                                                                  (3, 72, 48, 6, 1, 3, "bfloat16"), (30, 200, 80, 2, 1, 2, "bfloat16"), (1, 1000, 1040, 40, 0, 8, "bfloat16"),
+                                                                  (21, 136, 16, 1, 1, 2, "bfloat16")])
 def test_experts_that_return_their_input_and_the_norm_behind_them(rows, d, ff, E, identity, top, dtype):
     from geneinfer_amd.kernels import ops
     g = torch.Generator().manual_seed(rows + d)
@@ -446,9 +448,10 @@ def test_experts_that_return_their_input_and_the_norm_behind_them(rows, d, ff, E
     z = dev(start)
     ready = ops.routed_experts(dev(h), wg, wu, wd, ids, weights, z, weigh="output", then=(norm_w, norm_b, 1e-5))
     assert relative_error(z, x) < 1e-6
-    grouped = rows * top >= ops.EXPERTS_GROUPED_FROM and ops.experts_grouped_supported(dev(h), wg, wu, wd)
-    assert (ready is not None) == grouped
-    if grouped:
+    many = rows * top >= ops.EXPERTS_GROUPED_FROM and ops.experts_grouped_supported(dev(h), wg, wu, wd)
+    few = rows * top <= ops.EXPERTS_FEW_ITEMS and ops.experts_few_supported(dev(h), wg, wu, wd)
+    assert (ready is not None) == (many or few)
+    if ready is not None:
         ln = ops.layernorm(z.clone(), norm_w, norm_b, 1e-5, torch.empty(rows, d, device=DEV))
         assert relative_error(ready, ln) < 4e-3
 
