@@ -229,9 +229,9 @@ __global__ __launch_bounds__(64) void mlstm_scan_kernel(const float* __restrict_
 // With `den` [rows, heads], o is what the rows hold divided by den[t, h] (the matrix memory's sums and their divisor).
 // w_head_stride: dv where every head has weights of its own, 0 where all heads share one [dv]; gate_act 0: sigmoid(g), 1: SiLU, g sigmoid(g).
 // With `low` (float32 rows of stride ldg, `rank` numbers each) g is made here, g[t, i] = w_up[i] . low[t], the numbers rounded to bfloat16 as a
-// product's rows are: the form for a few rows.
-template <typename TW, typename TO>
-__global__ __launch_bounds__(64) void head_norm_gate_kernel(const float* __restrict__ o, long ldo, const float* __restrict__ den,
+// product's rows are: the form for a few rows, whose workgroups are NT = 256 threads (a wave otherwise).
+template <typename TW, typename TO, int NT>
+__global__ __launch_bounds__(NT) void head_norm_gate_kernel(const float* __restrict__ o, long ldo, const float* __restrict__ den,
                                                            const float* __restrict__ g, long ldg, const TW* __restrict__ w,
                                                            TO* __restrict__ y, long ldy, int n_heads, int dv, float eps, int w_head_stride, int gate_act,
                                                            const float* __restrict__ low, int rank, const bf16_t* __restrict__ w_up) {
@@ -239,12 +239,18 @@ __global__ __launch_bounds__(64) void head_norm_gate_kernel(const float* __restr
     const float* orow = o + (size_t)t * ldo + (size_t)h * dv;
     const float by = den ? den[(size_t)t * n_heads + h] : 1.0f;
     float ss = 0.f;
-    for (int d = lane; d < dv; d += 64) {
+    for (int d = lane; d < dv; d += NT) {
         const float v = den ? orow[d] / by : orow[d];
         ss = fmaf(v, v, ss);
     }
-    const float r = 1.0f / sqrtf(wave_sum(ss) / (float)dv + eps);
-    for (int d = lane; d < dv; d += 64) {
+    if constexpr (NT == 64) {
+        ss = wave_sum(ss);
+    } else {
+        __shared__ float red[NT / 64];
+        ss = block_sum<NT>(ss, red);
+    }
+    const float r = 1.0f / sqrtf(ss / (float)dv + eps);
+    for (int d = lane; d < dv; d += NT) {
         const float v = den ? orow[d] / by : orow[d];
         const float z = low ? narrow_dot(low + (size_t)t * ldg, w_up + ((size_t)h * dv + d) * rank, rank) : g[(size_t)t * ldg + (size_t)h * dv + d];
         const float gate = (gate_act ? z : 1.0f) / (1.0f + expf(-z));
@@ -648,13 +654,19 @@ GI_API int gi_head_norm_gate(const float* o, long ldo, const float* den, const f
     GI_REQUIRE(gate_act == 0 || gate_act == 1, "head_norm_gate: the gate is a sigmoid (0) or SiLU (1)");
     dim3 grid(n_rows, n_heads);
     const int w_head_stride = shared_weight ? 0 : dv;
-#define GO(TW, TO) head_norm_gate_kernel<TW, TO><<<grid, 64, 0, stream>>>(o, ldo, den, g, ldg, (const TW*)w, (TO*)y, ldy, n_heads, dv, eps, w_head_stride, gate_act, low, rank, (const bf16_t*)w_up)
+#define GO_NT(TW, TO, NT) head_norm_gate_kernel<TW, TO, NT><<<grid, NT, 0, stream>>>(o, ldo, den, g, ldg, (const TW*)w, (TO*)y, ldy, n_heads, dv, eps, w_head_stride, gate_act, low, rank, (const bf16_t*)w_up)
+#define GO(TW, TO)                           \
+    do {                                     \
+        if (low && dv > 64) GO_NT(TW, TO, 256); \
+        else GO_NT(TW, TO, 64);              \
+    } while (0)
     if (w_dtype == GI_F32 && y_dtype == GI_F32) GO(float, float);
     else if (w_dtype == GI_F32 && y_dtype == GI_BF16) GO(float, bf16_t);
     else if (w_dtype == GI_BF16 && y_dtype == GI_BF16) GO(bf16_t, bf16_t);
     else if (w_dtype == GI_BF16 && y_dtype == GI_F32) GO(bf16_t, float);
     else return gi_fail("head_norm_gate: unknown dtypes %d, %d", w_dtype, y_dtype);
 #undef GO
+#undef GO_NT
     GI_CHECK_LAUNCH("head_norm_gate");
     return 0;
 }

@@ -89,7 +89,7 @@ class LatentAttention(Mixer):
         self.q_norm, self.w_uq = (None, None) if self.direct else (tensors[s.dq_norm], tensors[s.uq_proj])
         self.sinks = tensors[s.sinks].float().contiguous() if getattr(s, "sinks", None) is not None else None
         # per head: W_uk_h^T [kv_rank, head_dim] (folded into the queries) and W_uv_h [value_dim, kv_rank] (applied to the attended latent)
-        self.w_uk_t = tensors[s.uk_proj].view(s.n_heads, s.head_dim, s.kv_rank).transpose(1, 2).contiguous()
+        self.w_uk_t = tensors[s.uk_proj].view(s.n_heads, s.head_dim, s.kv_rank).transpose(1, 2).reshape(-1).view(s.n_heads, s.kv_rank, s.head_dim)      # (strides of a row of one number are right so)
         self.w_uv = tensors[s.uv_proj].view(s.n_heads, s.value_dim, s.kv_rank).contiguous()
         self.w_o = tensors[s.o_proj]
         self.in_dtype = activation_dtype_for(self.w_down, dtype)

@@ -65,7 +65,7 @@ PUZORAX_D = dict(architecture="Puzorax", vocab=128, width=48, norm=dict(eps=1e-5
 # Attention only: a window of one position, and one longer than any sequence here; the last layer walked once.
 PUZORAX_E = dict(architecture="Puzorax", vocab=260, width=64, norm=dict(eps=1e-5), embedding=_pairs(50, 1, 1), loop=dict(start=1, stop=2, times=1), layers=[
     _att(2, 8, 8, 16, 24, 0.3, 100.0, 1, _moe(4, 1, 2, 48, 2.0)),
-    _att(16, 8, 8, 8, 40, 0.3, 20.0, 4096),
+    _att(16, 1, 8, 8, 40, 0.3, 20.0, 4096),
 ])
 CONFIGS = {"A": PUZORAX_A, "B": PUZORAX_B, "C": PUZORAX_C, "D": PUZORAX_D, "E": PUZORAX_E}
 RANKS = {"A": (6, 10), "B": (24, 40), "C": (5, 1), "D": (50, 3), "E": (1, 1)}          # (decays' middle, gates' middle)
