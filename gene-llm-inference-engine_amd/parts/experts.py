@@ -3,8 +3,9 @@
 The router's logits are a 32-bit product of the normed rows (as the compute dtype stores them) with the router's matrix; the
 same kernel turns them into every row's choice of experts and their weights.  The experts' matrices lie in stacks
 [experts, ...] (in bfloat16 an expert's gates and up products interleaved in one matrix, for the product with the gate inside).
-A few (row, choice) items walk their own expert's matrices each; many are put in the order of their experts on the device and
-go through the matrix cores, all experts in one launch.  Either way nothing of a step's shape depends on the router's choices,
+In bfloat16 a few (row, choice) items are picked up by the workgroups that stream their experts' weights; many are put in the order of
+their experts on the device and go through the matrix cores, all experts in one launch; in 32-bit every item walks its own expert's
+matrices.  Any way nothing of a step's shape depends on the router's choices,
 so a captured pass may contain the part.  A shared feed-forward, if the spec names one, is a part of its own kind and adds onto the
 same rows."""
 from __future__ import annotations
